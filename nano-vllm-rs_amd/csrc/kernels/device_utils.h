@@ -48,6 +48,8 @@ __device__ __forceinline__ float dot2(half2_t a, half2_t b, float c) {
 // v_exp_f32 + v_rcp_f32 (1 ulp each in f32, far below the fp16 / bf16 rounding that follows) instead of the ~10-instruction IEEE division
 // — the epilogue of the 256^2 gate_up GEMM is not overlapped with matrix work: -3..5 % on that kernel.
 __device__ __forceinline__ float sigmoid_fast(float x) { return __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
+// what the gate g of a gated feed-forward is multiplied by: silu(g) = g sigmoid(g); the tanh form of gelu, g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) / 2 = g sigmoid(2 sqrt(2/pi) (g + 0.044715 g^3))
+__device__ __forceinline__ float gate_factor(float g, bool gelu) { return sigmoid_fast(gelu ? 1.5957691216057308f * (g + 0.044715f * g * g * g) : g); }
 
 // Activation block x[T, cols] (row stride ldx, columns col0 .. col0 + 8*cpr) -> LDS image of ROWS rows x cpr 16-byte chunks, chunk ch of
 // row r at slot ch ^ (r & 7) (conflict-free ds_read_b128 of MFMA B fragments); rows >= T repeat row T-1.  FB loads are requested per

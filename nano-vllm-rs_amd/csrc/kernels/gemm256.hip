@@ -32,7 +32,8 @@
 
 namespace nvr { namespace NVR_DT_NS {
 
-enum { GEPI_F16 = 0, GEPI_RESID = 1, GEPI_SILU = 2, GEPI_ROPE = 3, GEPI_LMHEAD = 4, GEPI_RELU2 = 5 };   // RELU2: y = max(x·Wᵀ, 0)² (the product rounded to 16 bits first, as the unfused pair of launches does)
+enum { GEPI_F16 = 0, GEPI_RESID = 1, GEPI_SILU = 2, GEPI_ROPE = 3, GEPI_LMHEAD = 4, GEPI_RELU2 = 5, GEPI_GELU = 6 };   // RELU2: y = max(x·Wᵀ, 0)² (the product rounded to 16 bits first, as the unfused pair of launches does)
+constexpr bool g_glu(int epi) { return epi == GEPI_SILU || epi == GEPI_GELU; }      // gate and up rows in one tile, out = act(gate) * up (GELU: the tanh form)
 //   // RESID: y is the residual stream: y <- fp16(y + fp16(x·Wᵀ)) (qwen3.rs:382,389)
 // LMHEAD (r06): the LM head over >= 128 rows (ParallelLMHead::compute_logits, embed_head.rs:292-306, + the greedy branch of Sampler::forward,
 // sampler.rs:109-112): W = the [V, hidden] head, nothing is written as fp16 — every tile leaves (max, lowest vocabulary index) of its 256
@@ -62,7 +63,7 @@ __device__ __forceinline__ int g_w_thr(int r0) {
 }
 template <int EPI, int RD>
 __device__ __forceinline__ int g_w_uni(int hA, int i, int N) {
-    if (EPI == GEPI_SILU) return hA * N + i * 64;
+    if (g_glu(EPI)) return hA * N + i * 64;
     if (EPI == GEPI_ROPE) return i * 128 + hA * (RD / 2);
     return hA * 128 + i * 64;
 }
@@ -119,7 +120,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
     int wrows_left = 0x3fffffff;                                           // LM head: N - 1 - bx * 256 when the tile's vocabulary block is ragged
     auto set_sources = [&](int tile) {
         const int bx = tile % tiles_x, m0 = (tile / tiles_x) * 256;
-        wb = W + (int64_t)bx * ((EPI == GEPI_SILU) ? 128 : 256) * K;
+        wb = W + (int64_t)bx * (g_glu(EPI) ? 128 : 256) * K;
         if (GRP) wb += (int64_t)epi.row_w[tile / tiles_x] * epi.w_stride;
         xb = x + (int64_t)m0 * ldx;
         rows_left = m0 + 256 > T ? T - 1 - m0 : 0x3fffffff;
@@ -217,7 +218,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
 #define G256_S(HT_) if (more) stage(HT_, skt, g + 1);
 #define G256_W(NOMORE_) if (more) { G256_R_END(4) } else { G256_R_END(NOMORE_) }
 
-    constexpr int OUTC = (EPI == GEPI_SILU) ? 128 : 256;                  // output columns of a tile
+    constexpr int OUTC = g_glu(EPI) ? 128 : 256;                  // output columns of a tile
     const int64_t ldy = (EPI == GEPI_ROPE) ? (int64_t)(epi.H + 2 * epi.KVH) * RD : (int64_t)N;
     constexpr int hd2 = (EPI == GEPI_ROPE) ? RD / 2 : 1;
 
@@ -351,7 +352,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
         // halves stage below), so that the second half's results do not sit in f32 under the first half's store phase: the RoPE
         // store phase holds 64 registers of cos / sin next to them, and a spill here is a global-memory round trip (scratch)
         half4_t pk[2][4][2][2];
-        if (EPI != GEPI_SILU && EPI != GEPI_LMHEAD) {
+        if (!g_glu(EPI) && EPI != GEPI_LMHEAD) {
 #pragma unroll
             for (int a = 0; a < 2; ++a)
 #pragma unroll
@@ -394,14 +395,14 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
                             const int colo = (EPI == GEPI_ROPE) ? (rho / hd2) * RD + a * hd2 + rho % hd2 : a * 128 + rho;
                             put(ml, colo, pk[a][i][hB][j]);
                         }
-                } else if (EPI == GEPI_SILU) {
+                } else if (g_glu(EPI)) {
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         half4_t h;
 #pragma unroll
                         for (int e = 0; e < 4; ++e) {
                             const float gf = (float)to_half_rn(acc[0][i][hB][j][e]), uf = (float)to_half_rn(acc[1][i][hB][j][e]);
-                            const float sg = sigmoid_fast(gf);
+                            const float sg = gate_factor(gf, EPI == GEPI_GELU);
                             h[e] = to_half_rn(__fmul_rn(__fmul_rn(gf, sg), uf));
                         }
                         put(ml, wn * 64 + i * 16 + q * 4, h);
@@ -502,7 +503,7 @@ static int g256_prepare() {                                               // 128
                          reinterpret_cast<const void *>(&gemm256_kernel<GEPI_ROPE, 128>), reinterpret_cast<const void *>(&gemm256_kernel<GEPI_ROPE, 64>),
                          reinterpret_cast<const void *>(&gemm256_kernel<GEPI_RESID>), reinterpret_cast<const void *>(&gemm256_kernel<GEPI_LMHEAD>),
                          reinterpret_cast<const void *>(&gemm256_kernel<GEPI_F16, 0, true>), reinterpret_cast<const void *>(&gemm256_kernel<GEPI_SILU, 0, true>),
-                         reinterpret_cast<const void *>(&gemm256_kernel<GEPI_RELU2>)};
+                         reinterpret_cast<const void *>(&gemm256_kernel<GEPI_RELU2>), reinterpret_cast<const void *>(&gemm256_kernel<GEPI_GELU>)};
     for (const void *f : fns) {
         hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 2 * G_BUF + 4096);
         if (e != hipSuccess) return nvr::fail(NVR_ERR_HIP, "gemm256: hipFuncSetAttribute: %s", hipGetErrorString(e));
@@ -590,6 +591,15 @@ int gemm256_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_
     gemm256_kernel<GEPI_SILU><<<dim3((unsigned)g256_grid(tt)), dim3(512), 2 * G_BUF, s>>>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K,
                                                                                          (int)I, (int)(2 * I), (half_t *)out, G256Epi{}, tx, tt / tx, g256_cg(tx, tt / tx, false));
     return g256_check("gemm256_silu_mul");
+}
+// out = gelu(gate) * up with the tanh form of gelu
+int gemm256_gelu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s) {
+    if (!gemm256_silu_ok(T, K, I, ldx)) return nvr::fail(NVR_ERR_UNSUPPORTED, "gemm256_gelu_mul: T=%ld K=%ld I=%ld", (long)T, (long)K, (long)I);
+    if (int rc = g256_prepare()) return rc;
+    const int tx = (int)(I / 128), tt = tx * (int)((T + 255) / 256);
+    gemm256_kernel<GEPI_GELU><<<dim3((unsigned)g256_grid(tt)), dim3(512), 2 * G_BUF, s>>>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K,
+                                                                                         (int)I, (int)(2 * I), (half_t *)out, G256Epi{}, tx, tt / tx, g256_cg(tx, tt / tx, false));
+    return g256_check("gemm256_gelu_mul");
 }
 int gemm256_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t D,
                            const int64_t *positions, const int32_t *slots, const float *cos_t, const float *sin_t, half_bits *qkv,

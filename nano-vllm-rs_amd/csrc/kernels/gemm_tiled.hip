@@ -33,6 +33,7 @@ struct TileEpi {
     float *logits; float *pval; int32_t *pidx;
     // TEPI_SLAB: blockIdx.z owns k in [z*kslice, (z+1)*kslice) and writes its f32 partial tile to slabs[z][T][N]
     float *slabs; int64_t slab_stride; int32_t kslice;
+    int32_t gelu;                          // TEPI_SILU: gelu (tanh form) instead of silu
 };
 
 constexpr int BM = 128, BN = 128, BK = 64;
@@ -288,7 +289,7 @@ __global__ __launch_bounds__(256) void gemm_tiled_kernel(const half_t *__restric
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const float gf = (float)to_half_rn(acc[i][j][e]), uf = (float)to_half_rn(acc[i + 2][j][e]);
-                    const float sg = sigmoid_fast(gf);
+                    const float sg = gate_factor(gf, epi.gelu);
                     h[e] = to_half_rn(__fmul_rn(__fmul_rn(gf, sg), uf));
                 }
                 stash(ml, wn * 32 + i * 16 + q * 4, h);
@@ -550,19 +551,20 @@ int gemm_tiled(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, i
     NVR_TILED_LAUNCH(TEPI_F16, grid, T, (const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)N, (int)N, (half_t *)y, TileEpi{});
     return tiled_check("gemm_tiled");
 }
-int gemm_tiled_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s) {
+int gemm_tiled_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s, bool gelu) {
     if (!gemm_tiled_ok(T, K, I, ldx) || I % 64) return nvr::fail(NVR_ERR_UNSUPPORTED, "gemm_tiled_silu_mul: T=%ld K=%ld I=%ld", (long)T, (long)K, (long)I);
     dim3 grid((unsigned)(I / 64), (unsigned)((T + BM - 1) / BM));
     if (int rc = gemm_tiled_prepare()) return rc;
     {   // 96-row tiles when they put a workgroup on (nearly) every CU where the 128-row tiles leave a quarter of them idle (T = 512, I = 3072: 256 against 192;
         // T = 321..384: 192 against 144)
         const int64_t ty = (T + BM - 1) / BM, w128 = (I / 64) * ty, w96 = (I / 48) * ty;
-        if (I % 48 == 0 && tiled_mt(T, I / 64) == 4 && tiled_ring((unsigned)w128) && w96 <= 256 && w96 > w128 && w128 * 8 <= w96 * 7) {
+        if (!gelu && I % 48 == 0 && tiled_mt(T, I / 64) == 4 && tiled_ring((unsigned)w128) && w96 <= 256 && w96 > w128 && w128 * 8 <= w96 * 7) {
             gemm_tiled_silu96_kernel<<<dim3((unsigned)(I / 48), (unsigned)ty), dim3(256), RING96 * S96_BUF, s>>>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (half_t *)out);
             return tiled_check("gemm_tiled_silu_mul (96-row tiles)");
         }
     }
-    NVR_TILED_LAUNCH(TEPI_SILU, grid, T, (const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (int)(2 * I), (half_t *)out, TileEpi{});
+    TileEpi e{}; e.gelu = gelu ? 1 : 0;
+    NVR_TILED_LAUNCH(TEPI_SILU, grid, T, (const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (int)(2 * I), (half_t *)out, e);
     return tiled_check("gemm_tiled_silu_mul");
 }
 int gemm_tiled_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t D,

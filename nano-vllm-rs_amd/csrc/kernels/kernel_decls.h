@@ -63,6 +63,8 @@ int add_rmsnorm_slabs(half_bits *h, const float *slabs, int64_t S, const half_bi
 // qkv -> RoPE(q,k) + KV store, W [(H+2KVH)D, K] -> qkv [T,(H+2KVH)D] (roped q,k; v) and cache rows at slots
 int linear_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I,
                     half_bits *out, hipStream_t s, const half_bits *Wt = nullptr);
+// the same with gelu (tanh form) in silu's place
+int linear_gelu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s);
 int linear_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H,
                           int64_t KVH, int64_t D, const int64_t *positions, const int32_t *slots, const float *cos_t,
                           const float *sin_t, half_bits *qkv, half_bits *k_cache, half_bits *v_cache, hipStream_t s,
@@ -81,7 +83,7 @@ bool linear_stream_rope_ok(int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t
 int linear_stream(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s,
                   const half_bits *Wt = nullptr);
 int linear_stream_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s,
-                           const half_bits *Wt = nullptr);
+                           const half_bits *Wt = nullptr, bool gelu = false);
 int linear_stream_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t D,
                                  const int64_t *positions, const int32_t *slots, const float *cos_t, const float *sin_t, half_bits *qkv,
                                  half_bits *k_cache, half_bits *v_cache, hipStream_t s, const half_bits *Wt = nullptr);
@@ -98,7 +100,7 @@ int gemm_tiled_lm_head(const half_bits *x, int64_t ldx, const half_bits *W, int6
 bool gemm_tiled_ok(int64_t T, int64_t K, int64_t N, int64_t ldx);
 int gemm_tiled(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s);
 int gemm_tiled_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out,
-                        hipStream_t s);
+                        hipStream_t s, bool gelu = false);
 int gemm_tiled_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H, int64_t KVH,
                               int64_t D, const int64_t *positions, const int32_t *slots, const float *cos_t, const float *sin_t,
                               half_bits *qkv, half_bits *k_cache, half_bits *v_cache, hipStream_t s);
@@ -119,6 +121,7 @@ int gemm256_lm_head(const half_bits *x, int64_t ldx, const half_bits *W, int64_t
                     int32_t *part_idx, int32_t *nparts, hipStream_t s);
 bool gemm256_preferred(int64_t T, int64_t K, int64_t N, int64_t ldx);     // linear() would take the 256x256 kernel for this shape
 int gemm256_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s);
+int gemm256_gelu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s);
 int gemm256_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t D,
                            const int64_t *positions, const int32_t *slots, const float *cos_t, const float *sin_t, half_bits *qkv,
                            half_bits *k_cache, half_bits *v_cache, hipStream_t s, bool kv_cache_only = false);

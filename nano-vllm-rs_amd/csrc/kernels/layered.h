@@ -151,7 +151,8 @@ int grouped_linear(const GroupedLinearArgs &a, bool bf16, hipStream_t s);
 
 // out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, N(v) = v / sqrt(mean(v^2) + eps) over the F numbers of a row; coef: 4 floats on the device
 int poly_norm(const void *z, int64_t ldz, int64_t T, int64_t F, float eps, const float *coef, void *out, int64_t ldo, bool bf16, hipStream_t s);
-// out = silu(gate) * up; gu: rows [2 F] (gate columns, then up columns)
+// out = silu(gate) * up, or gelu(gate) * up (the tanh form); gu: rows [2 F] (gate columns, then up columns)
+int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 
 // Router of a mixture of experts: logits wr h in f32 (wr: [E][W] f32), the top largest per token -> sel / score (= sigmoid of the logit) [T][top]; then the rows
@@ -159,15 +160,17 @@ int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool 
 // (places then run up to (T top / pad + E) pad) and row_w[block] names the expert of each of the nblocks blocks of pad rows: the form a tiled product over whole
 // row blocks wants, with the rows brought together by moe_gather (xs[place] = h[token] * score).
 // softmax: score is the chosen experts' share of the softmax over ALL experts, divided by the sum of the chosen shares (+ 1e-20), instead of the sigmoid.
+// correction (softmax, [E] f32): the choice is made by share + correction, the scores stay the shares.  identity > 0: the last `identity` of the E outputs have no matrix (their expert
+// returns its input): a token that chose one gets place -1 there, and the groups, off and row_w are those of the E - identity others.
 // extra > 0: rows E .. E + extra - 1 of wr are further f32 projections of h that leave as they are in extra_out[t * extra + i] (a shared expert's gate).
 int moe_route(const void *h, int64_t ldh, int64_t T, int64_t W, const float *wr, int64_t E, int64_t top, int32_t *sel, float *score, int32_t *off, int32_t *order,
               int32_t *place_of, int64_t pad, int32_t *row_w, int64_t nblocks, bool bf16, hipStream_t s, bool softmax = false, int64_t extra = 0, float *extra_out = nullptr,
-              const float *logits = nullptr, int64_t ldl = 0);   // logits (f32 rows of E + extra numbers, stride ldl): the products wr h formed beforehand (wr is then not read)
+              const float *logits = nullptr, int64_t ldl = 0, const float *correction = nullptr, int64_t identity = 0);   // logits (f32 rows of E + extra numbers, stride ldl): the products wr h formed beforehand (wr is then not read)
 int moe_gather(const void *h, int64_t ldh, int64_t T, int64_t W, int64_t top, const int32_t *place_of, const float *score, void *xs, bool bf16, hipStream_t s);
 // out[t] = sum_k y[place_of[t * top + k]] + shared[t] (shared may be null).  With score ([T][top] f32) choice k is weighted by score[t * top + k]; with shared_gate
-// ([T] f32, stride gate_ld) the shared row is multiplied by sigmoid(shared_gate[t * gate_ld]).
+// ([T] f32, stride gate_ld) the shared row is multiplied by sigmoid(shared_gate[t * gate_ld]).  A choice with place -1 contributes ident's row t (operand type, stride ldi).
 int moe_combine(const void *y, const int32_t *place_of, int64_t T, int64_t top, const void *shared, int64_t W, void *out, bool bf16, hipStream_t s,
-                const float *score = nullptr, const float *shared_gate = nullptr, int64_t gate_ld = 1);
+                const float *score = nullptr, const float *shared_gate = nullptr, int64_t gate_ld = 1, const void *ident = nullptr, int64_t ldi = 0);
 
 // The per-layer token input is y = Wp (gelu_tanh(Wg x) * E[id][ecol .. ecol + dim)), x += y / rms(y) * wn: two ordinary products with this between them
 // (z = Wg x rows of dim numbers -> g), and its last step inside layer_tail.
@@ -265,5 +268,35 @@ int shift_mixes(const void *m, int64_t ldm, const Batch &b, int64_t W, int32_t n
 
 // y = tanh(y) in place (rows of N numbers, stride ld)
 int tanh_rows(void *y, int64_t ld, int64_t T, int64_t N, bool bf16, hipStream_t s);
+
+// ---------------------------------------------------------------------------------------------------------------------------------------------------
+// Blocks of layers whose residual is a set of parallel streams (layered_streams.hip).
+int prepare_streams();                                  // LDS opt-ins (call once, outside captures)
+
+// S residual streams per row, x: [T][S][W] f32.  One launch ends a sublayer and starts the next one:
+//   x_q <- sum_s mix[s][q] x_s + wout[q] y (all new streams from the old ones; y rows of the operand type, stride ldy), u = sum_s win[s] x_s,
+//   out = (u - mean(u)) / sqrt(var(u) + eps) * w (layer norm without a bias; operand type, stride ldo).
+// E (operand type, [vocab][W]) not null: the start — every stream of row t becomes E[ids[t]] first, nothing is written from y.  sum: the end — u is the sum of the new streams, which
+// are not stored, of the T rows rows[0 .. T-1] (null: all); out row r belongs to rows[r].  mix: [S][S] (from, to); mix / wout / win / w f32 on the device.
+struct StreamArgs {
+    float *x; int32_t S, W; int64_t T; float eps;
+    const void *E; const int64_t *ids;
+    const void *y; int64_t ldy; const float *mix, *wout;
+    const float *win, *w; void *out; int64_t ldo;
+    const int32_t *rows; bool sum;
+};
+int stream_step(const StreamArgs &a, bool bf16, hipStream_t s);
+
+// Queries, keys and values on their way from the projections to an attention over pages.  In row t of proj: q += bq, k += bk, v += bv (each may be null); the first `rot` numbers of
+// every q / k head turned by position * freq[i] — pairs: numbers (2i, 2i + 1), else (i, i + rot / 2) —; unit: every q / k head divided by sqrt(mean^2 + eps) behind the rotation;
+// q stays in proj, k -> the K page row of the position.  v_keep (may be null): this step's values as they are now, [T][G Dv]; v_first (may be null): v <- (1 - lambda) v + lambda v_first
+// with rows like v_keep's; v -> the V page row (layouts as kv_store).
+struct QkvRopeArgs {
+    void *proj; int64_t ld, qcol, kcol, vcol; int32_t H, G, D, Dv, rot; const float *freq; bool pairs;
+    const float *bq, *bk, *bv; bool unit; float eps;
+    void *v_keep; const void *v_first; const float *lambda;
+    void *kc, *vc; bool v_grouped;
+};
+int qkv_rope_store(const QkvRopeArgs &a, const Batch &b, bool bf16, hipStream_t s);
 
 }}  // namespace nvr::kl

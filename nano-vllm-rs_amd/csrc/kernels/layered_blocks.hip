@@ -496,14 +496,28 @@ __global__ __launch_bounds__(256) void poly_norm_kernel(const OT *__restrict__ z
     for (int c = threadIdx.x; c < F; c += 256) { const float v = ld_f(z, t * ldz + c); st_f(out, t * ldo + c, v * i1 + v * v * i2 + v * v * v * i3 + e); }
 }
 
-// out = silu(gate) * up; gu rows [2 F] (gate columns, then up columns)
-template <class OT>
-__global__ __launch_bounds__(256) void silu_mul_kernel(const OT *__restrict__ gu, int64_t T, int64_t F, OT *__restrict__ out, int64_t ldo) {
+// out = act(gate) * up; gu rows [2 F] (gate columns, then up columns); GELU: the tanh form, else silu
+template <class OT, bool GELU>
+__global__ __launch_bounds__(256) void gated_mul_kernel(const OT *__restrict__ gu, int64_t T, int64_t F, OT *__restrict__ out, int64_t ldo) {
     const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (idx >= T * F) return;
     const int64_t t = idx / F, c = idx - t * F;
     const float g = ld_f(gu, t * 2 * F + c);
-    st_f(out, t * ldo + c, g * sigmoid_f(g) * ld_f(gu, t * 2 * F + F + c));
+    st_f(out, t * ldo + c, (GELU ? gelu_tanh_f(g) : g * sigmoid_f(g)) * ld_f(gu, t * 2 * F + F + c));
+}
+
+// 16-bit rows, 8 numbers per thread (F and the stride multiples of 8, 16-byte aligned rows)
+template <bool GELU>
+__global__ __launch_bounds__(256) void gated_mul8_kernel(const bf16_t *__restrict__ gu, int64_t T, int64_t F8, bf16_t *__restrict__ out, int64_t ldo) {
+    const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (idx >= T * F8) return;
+    const int64_t t = idx / F8, c = (idx - t * F8) * 8;
+    uint4 gv = *reinterpret_cast<const uint4 *>(gu + t * 16 * F8 + c);
+    const uint4 uv = *reinterpret_cast<const uint4 *>(gu + t * 16 * F8 + 8 * F8 + c);
+    bf16_t *ge = reinterpret_cast<bf16_t *>(&gv); const bf16_t *ue = reinterpret_cast<const bf16_t *>(&uv);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) { const float g = ld_f(ge, k); st_f(ge, k, (GELU ? gelu_tanh_f(g) : g * sigmoid_f(g)) * ld_f(ue, k)); }
+    *reinterpret_cast<uint4 *>(out + t * ldo + c) = gv;
 }
 
 // ------------------------------------------------------------------------------------------------ mixture of experts
@@ -513,8 +527,8 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(const OT *__restrict__ gu
 template <class OT>
 __global__ __launch_bounds__(256) void moe_route_kernel(const OT *__restrict__ h, int64_t ldh, int W, const float *__restrict__ wr, int E, int top,
                                                         int32_t *__restrict__ sel, float *__restrict__ score, int softmax, int extra, float *__restrict__ extra_out,
-                                                        const float *__restrict__ logits, int64_t ldl) {
-    extern __shared__ float sc[];                       // [E + extra]
+                                                        const float *__restrict__ logits, int64_t ldl, const float *__restrict__ correction) {
+    extern __shared__ float sc[];                       // [E + extra], with a correction also [E] choice scores
     const int64_t t = blockIdx.x; const int lane = threadIdx.x & 63;
     if (logits)                                         // the products were formed by a matrix product before this launch
         for (int e = threadIdx.x; e < E + extra; e += 256) { const float d = logits[t * ldl + e]; sc[e] = d; if (e >= E) extra_out[t * extra + (e - E)] = d; }
@@ -536,11 +550,16 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const OT *__restrict__ h
         for (int e = lane; e < E; e += 64) zsum += expf(sc[e] - zmax);
         zsum = wave_sum(zsum);
     }
+    float *ch = sc;                                     // what the choice compares: the logits, or share + correction
+    if (correction) {
+        ch = sc + E + extra;
+        if (threadIdx.x < 64) for (int e = lane; e < E; e += 64) ch[e] = expf(sc[e] - zmax) / zsum + correction[e];       // (a lane reads its own entries back)
+    }
     float chosen = 0.f;                                 // (lane 0: the sum of the chosen shares)
     for (int k = 0; k < top; ++k) {                     // the first wave: top times the arg-max over the experts' logits
         if (threadIdx.x < 64) {
             float best = -INFINITY; int bi = E;
-            for (int e = lane; e < E; e += 64) if (sc[e] > best || (sc[e] == best && e < bi)) { best = sc[e]; bi = e; }
+            for (int e = lane; e < E; e += 64) if (ch[e] > best || (ch[e] == best && e < bi)) { best = ch[e]; bi = e; }
 #pragma unroll
             for (int o = 32; o > 0; o >>= 1) {
                 const float ob = __shfl_xor(best, o, 64); const int oi = __shfl_xor(bi, o, 64);
@@ -548,8 +567,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const OT *__restrict__ h
             }
             if (bi >= E) bi = E - 1;                        // (logits that are not numbers compare false everywhere: the index still has to be an expert's)
             if (lane == 0) {
-                const float sv = softmax ? expf(best - zmax) / zsum : sigmoid_f(best);
-                sel[t * top + k] = bi; score[t * top + k] = sv; chosen += sv; sc[bi] = -INFINITY;
+                const float z = correction ? sc[bi] : best;
+                const float sv = softmax ? expf(z - zmax) / zsum : sigmoid_f(z);
+                sel[t * top + k] = bi; score[t * top + k] = sv; chosen += sv; ch[bi] = -INFINITY;
             }
         }
         __syncthreads();
@@ -558,13 +578,13 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const OT *__restrict__ h
 }
 
 // One workgroup: counts per expert, offsets, and a place for every (token, choice) among its expert's rows.  order[place] = token * top + choice;
-// place_of[token * top + choice] = place.  Which place inside its expert a row gets is left to the atomics: a row's result does not depend on it.
+// place_of[token * top + choice] = place (-1: a choice >= E has no group).  Which place inside its expert a row gets is left to the atomics: a row's result does not depend on it.
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restrict__ sel, int n, int E, int pad, int nblocks, int32_t *__restrict__ off,
                                                          int32_t *__restrict__ order, int32_t *__restrict__ place_of, int32_t *__restrict__ row_w) {
     extern __shared__ int32_t cnt[];                    // [E + 1] counts, then running offsets
     for (int e = threadIdx.x; e <= E; e += 1024) cnt[e] = 0;
     __syncthreads();
-    for (int i = threadIdx.x; i < n; i += 1024) atomicAdd(&cnt[sel[i]], 1);
+    for (int i = threadIdx.x; i < n; i += 1024) if (sel[i] < E) atomicAdd(&cnt[sel[i]], 1);
     __syncthreads();
     if (threadIdx.x == 0) {                             // an expert's rows start at a multiple of pad; row_w names the expert of every block of pad rows
         int run = 0;
@@ -578,7 +598,11 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restri
         if (row_w) for (int bk = run / pad; bk < nblocks; ++bk) row_w[bk] = 0;      // (blocks behind the last expert: any matrix, their rows are nobody's)
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < n; i += 1024) { const int place = atomicAdd(&cnt[sel[i]], 1); order[place] = i; place_of[i] = place; }
+    for (int i = threadIdx.x; i < n; i += 1024) {
+        if (sel[i] >= E) { place_of[i] = -1; continue; }
+        const int place = atomicAdd(&cnt[sel[i]], 1);
+        order[place] = i; place_of[i] = place;
+    }
 }
 
 // xs[place_of[i]] = h[i / top] * score[i] (the expert's input, in the order of the grouped rows)
@@ -586,6 +610,7 @@ template <class OT>
 __global__ __launch_bounds__(256) void moe_gather_kernel(const OT *__restrict__ h, int64_t ldh, int W, int top, const int32_t *__restrict__ place_of, const float *__restrict__ score,
                                                          OT *__restrict__ xs) {
     const int64_t i = blockIdx.x, t = i / top;
+    if (place_of[i] < 0) return;                        // (an expert without a matrix)
     const float sc = score[i];
     OT *dst = xs + (int64_t)place_of[i] * W;
     for (int c = threadIdx.x; c < W; c += 256) st_f(dst, c, ld_f(h, t * ldh + c) * sc);
@@ -594,12 +619,16 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const OT *__restrict__ 
 // out[t] = sum_k y[place_of[t * top + k]] (+ shared[t]) in the operand type
 template <class OT>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const OT *__restrict__ y, const int32_t *__restrict__ place_of, int top, const OT *__restrict__ shared, int W,
-                                                          OT *__restrict__ out, const float *__restrict__ score, const float *__restrict__ shared_gate, int64_t gate_ld) {
+                                                          OT *__restrict__ out, const float *__restrict__ score, const float *__restrict__ shared_gate, int64_t gate_ld,
+                                                          const OT *__restrict__ ident, int64_t ldi) {
     const int64_t t = blockIdx.x;
     const float sg = (shared && shared_gate) ? sigmoid_f(shared_gate[t * gate_ld]) : 1.f;
     for (int c = threadIdx.x; c < W; c += 256) {
         float v = shared ? ld_f(shared, t * W + c) * sg : 0.f;
-        for (int k = 0; k < top; ++k) v += ld_f(y, (int64_t)place_of[t * top + k] * W + c) * (score ? score[t * top + k] : 1.f);
+        for (int k = 0; k < top; ++k) {
+            const int64_t place = place_of[t * top + k];
+            v += (place < 0 ? ld_f(ident, t * ldi + c) : ld_f(y, place * W + c)) * (score ? score[t * top + k] : 1.f);
+        }
         st_f(out, t * W + c, v);
     }
 }
@@ -780,26 +809,35 @@ int poly_norm(const void *z, int64_t ldz, int64_t T, int64_t F, float eps, const
     return launched("poly_norm");
 }
 
-int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) {
+template <bool GELU>
+static int gated_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) {
     if (T * F == 0) return 0;
+    if (bf16 && F % 8 == 0 && ldo % 8 == 0 && aligned16(gu) && aligned16(out)) {
+        gated_mul8_kernel<GELU><<<dim3((unsigned)((T * (F / 8) + 255) / 256)), dim3(256), 0, s>>>((const bf16_t *)gu, T, F / 8, (bf16_t *)out, ldo);
+        return launched("gated_mul");
+    }
     const dim3 grid((unsigned)((T * F + 255) / 256));
-    if (bf16) silu_mul_kernel<bf16_t><<<grid, dim3(256), 0, s>>>((const bf16_t *)gu, T, F, (bf16_t *)out, ldo);
-    else silu_mul_kernel<float><<<grid, dim3(256), 0, s>>>((const float *)gu, T, F, (float *)out, ldo);
-    return launched("silu_mul");
+    if (bf16) gated_mul_kernel<bf16_t, GELU><<<grid, dim3(256), 0, s>>>((const bf16_t *)gu, T, F, (bf16_t *)out, ldo);
+    else gated_mul_kernel<float, GELU><<<grid, dim3(256), 0, s>>>((const float *)gu, T, F, (float *)out, ldo);
+    return launched("gated_mul");
 }
+int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) { return gated_mul<false>(gu, T, F, out, ldo, bf16, s); }
+int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) { return gated_mul<true>(gu, T, F, out, ldo, bf16, s); }
 
 int moe_route(const void *h, int64_t ldh, int64_t T, int64_t W, const float *wr, int64_t E, int64_t top, int32_t *sel, float *score, int32_t *off, int32_t *order,
               int32_t *place_of, int64_t pad, int32_t *row_w, int64_t nblocks, bool bf16, hipStream_t s, bool softmax, int64_t extra, float *extra_out,
-              const float *logits, int64_t ldl) {
+              const float *logits, int64_t ldl, const float *correction, int64_t identity) {
     if (T == 0) return 0;
+    if (correction && !softmax) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: a correction belongs to softmax scores");
+    if (identity < 0 || identity >= E) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: %ld of %ld experts without a matrix", (long)identity, (long)E);
     if (extra < 0 || (extra > 0 && !extra_out)) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: %ld further rows without a place for them", (long)extra);
     if (top < 1 || top > E) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: %ld of %ld experts", (long)top, (long)E);
-    if ((size_t)(E + 1) * 4 > 60000) return nvr::fail(NVR_ERR_UNSUPPORTED, "moe_route: %ld experts", (long)E);
-    if (bf16) moe_route_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra) * 4, s>>>((const bf16_t *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl);
-    else moe_route_kernel<float><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra) * 4, s>>>((const float *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl);
+    if ((size_t)(2 * E + extra + 1) * 4 > 60000) return nvr::fail(NVR_ERR_UNSUPPORTED, "moe_route: %ld experts", (long)E);
+    if (bf16) moe_route_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra + (correction ? E : 0)) * 4, s>>>((const bf16_t *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
+    else moe_route_kernel<float><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra + (correction ? E : 0)) * 4, s>>>((const float *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
     if (int rc = launched("moe_route")) return rc;
     if (pad < 1) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: rows padded to %ld", (long)pad);
-    moe_group_kernel<<<dim3(1), dim3(1024), (size_t)(E + 1) * 4, s>>>(sel, (int)(T * top), (int)E, (int)pad, (int)nblocks, off, order, place_of, row_w);
+    moe_group_kernel<<<dim3(1), dim3(1024), (size_t)(E - identity + 1) * 4, s>>>(sel, (int)(T * top), (int)(E - identity), (int)pad, (int)nblocks, off, order, place_of, row_w);
     return launched("moe_group");
 }
 
@@ -811,10 +849,10 @@ int moe_gather(const void *h, int64_t ldh, int64_t T, int64_t W, int64_t top, co
 }
 
 int moe_combine(const void *y, const int32_t *place_of, int64_t T, int64_t top, const void *shared, int64_t W, void *out, bool bf16, hipStream_t s,
-                const float *score, const float *shared_gate, int64_t gate_ld) {
+                const float *score, const float *shared_gate, int64_t gate_ld, const void *ident, int64_t ldi) {
     if (T == 0) return 0;
-    if (bf16) moe_combine_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), 0, s>>>((const bf16_t *)y, place_of, (int)top, (const bf16_t *)shared, (int)W, (bf16_t *)out, score, shared_gate, gate_ld);
-    else moe_combine_kernel<float><<<dim3((unsigned)T), dim3(256), 0, s>>>((const float *)y, place_of, (int)top, (const float *)shared, (int)W, (float *)out, score, shared_gate, gate_ld);
+    if (bf16) moe_combine_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), 0, s>>>((const bf16_t *)y, place_of, (int)top, (const bf16_t *)shared, (int)W, (bf16_t *)out, score, shared_gate, gate_ld, (const bf16_t *)ident, ldi);
+    else moe_combine_kernel<float><<<dim3((unsigned)T), dim3(256), 0, s>>>((const float *)y, place_of, (int)top, (const float *)shared, (int)W, (float *)out, score, shared_gate, gate_ld, (const float *)ident, ldi);
     return launched("moe_combine");
 }
 

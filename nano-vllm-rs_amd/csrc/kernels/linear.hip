@@ -41,6 +41,7 @@ struct LinEpi {
     int32_t kslice; int64_t slab_stride;
     // W is the TILED copy [N/16][K/32][16][32] (retile_weight): one wave-instruction reads 1 KiB contiguous
     int32_t tiled;
+    int32_t gelu;                          // EPI_SILU: gelu (tanh form) instead of silu
 };
 
 // W row handled by local row r (0..15) of n-tile i of workgroup bx
@@ -173,7 +174,7 @@ __global__ __launch_bounds__(WAVES * 64) void linear_skinny_kernel(const half_t 
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const float gf = (float)to_half_rn(g4[e]), uf = (float)to_half_rn(u4[e]);
-                    const float sg = sigmoid_fast(gf);
+                    const float sg = gate_factor(gf, epi.gelu);
                     h[e] = to_half_rn(__fmul_rn(__fmul_rn(gf, sg), uf));
                 }
                 *reinterpret_cast<half4_t *>(reinterpret_cast<half_t *>(y) + (int64_t)m * N + n) = h;
@@ -340,17 +341,17 @@ int linear_splitk(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T
 }
 
 // gate_up GEMM + SiluAndMul: W [2I, K] (gate rows then up rows), out [T, I]
-int linear_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I,
-                    half_bits *out, hipStream_t s, const half_bits *Wt) {
+static int linear_glu(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I,
+                      half_bits *out, hipStream_t s, const half_bits *Wt, bool gelu) {
     if (K % 32 || I % 16 || ldx % 8)
         return nvr::fail(NVR_ERR_UNSUPPORTED, "linear_silu_mul: K=%ld must be a multiple of 32, I=%ld of 16", (long)K, (long)I);
     if (T == 0) return 0;
-    if (gemm256_silu_ok(T, K, I, ldx) && prefer_256(T, K, 2 * I)) return gemm256_silu_mul(x, ldx, W, T, K, I, out, s);   // see linear()
-    if (gemm_tiled_ok(T, K, I, ldx) && I % 64 == 0 && !prefer_stream(T, 2 * I)) return gemm_tiled_silu_mul(x, ldx, W, T, K, I, out, s);
-    if (linear_stream_silu_ok(T, K, I, ldx)) return linear_stream_silu_mul(x, ldx, W, T, K, I, out, s, Wt);              // large weights
+    if (gemm256_silu_ok(T, K, I, ldx) && prefer_256(T, K, 2 * I)) return gelu ? gemm256_gelu_mul(x, ldx, W, T, K, I, out, s) : gemm256_silu_mul(x, ldx, W, T, K, I, out, s);   // see linear()
+    if (gemm_tiled_ok(T, K, I, ldx) && I % 64 == 0 && !prefer_stream(T, 2 * I)) return gemm_tiled_silu_mul(x, ldx, W, T, K, I, out, s, gelu);
+    if (linear_stream_silu_ok(T, K, I, ldx)) return linear_stream_silu_mul(x, ldx, W, T, K, I, out, s, Wt, gelu);              // large weights
     const half_t *xx = (const half_t *)x, *ww = (const half_t *)(Wt ? Wt : W);
     LinEpi e{};
-    e.tiled = Wt != nullptr;
+    e.tiled = Wt != nullptr; e.gelu = gelu ? 1 : 0;
     const unsigned gx = (unsigned)(I / 16);
     const int wv = waves_for(K);
     // few column tiles (the shard of a tensor-parallel rank): 16-token workgroups double the workgroup count (the second token
@@ -366,6 +367,13 @@ int linear_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t
         else launch<2, 2, 4, EPI_SILU>(xx, ldx, ww, (int)T, (int)K, (int)I, out, e, gx, s);
     }
     return launch_check("linear_silu_mul");
+}
+int linear_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s, const half_bits *Wt) {
+    return linear_glu(x, ldx, W, T, K, I, out, s, Wt, false);
+}
+// the same with gelu (tanh form) in silu's place
+int linear_gelu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s) {
+    return linear_glu(x, ldx, W, T, K, I, out, s, nullptr, true);
 }
 
 // qkv GEMM + RoPE on q,k heads + store of k,v rows into the paged caches

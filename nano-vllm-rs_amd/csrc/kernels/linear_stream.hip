@@ -29,6 +29,7 @@ struct StreamEpi {
     half_t *kc, *vc;
     int32_t H, KVH, D;
     int32_t tiled;                       // W is the retile_weight copy [N/16][K/32][16][32] (SEPI_ROPE: mode 1, tiles in s_w_row order)
+    int32_t gelu;                        // SEPI_SILU: gelu (tanh form) instead of silu
 };
 
 // W row behind local row r (0..15) of part nt (SiLU: 0 = gate, 1 = up) of tile t
@@ -363,7 +364,7 @@ __global__ __launch_bounds__(WAVES * 64) void linear_stream_kernel(const half_t 
 #pragma unroll
                     for (int e = 0; e < 4; ++e) {
                         const float gf = (float)to_half_rn(g4[e]), uf = (float)to_half_rn(u4[e]);
-                        const float sg = sigmoid_fast(gf);
+                        const float sg = gate_factor(gf, epi.gelu);
                         h[e] = to_half_rn(__fmul_rn(__fmul_rn(gf, sg), uf));
                     }
                     *reinterpret_cast<half4_t *>(y + (int64_t)m * N + n) = h;
@@ -505,9 +506,9 @@ int linear_stream(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T
     return stream_launch<1, 2, 4, SEPI_F16>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)N, (int)(N / 16), (half_t *)y, e, s);
 }
 int linear_stream_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s,
-                           const half_bits *Wt) {
+                           const half_bits *Wt, bool gelu) {
     if (!linear_stream_silu_ok(T, K, I, ldx)) return nvr::fail(NVR_ERR_UNSUPPORTED, "linear_stream_silu_mul: T=%ld K=%ld I=%ld", (long)T, (long)K, (long)I);
-    StreamEpi e{};
+    StreamEpi e{}; e.gelu = gelu ? 1 : 0;
     if (Wt) { W = Wt; e.tiled = 1; }
     if (T <= 16) return stream_launch<2, 1, 2, SEPI_SILU>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (int)(I / 16), (half_t *)out, e, s);
     if (T > 32) return stream_launch<2, 4, 2, SEPI_SILU>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (int)(I / 16), (half_t *)out, e, s);

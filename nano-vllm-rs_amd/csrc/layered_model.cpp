@@ -68,7 +68,7 @@ int LayeredModel::init(nvr_model_runner &r) {
     r.device = r.cfg.device_ordinal;
     NVR_HIP_CHECK(hipSetDevice(r.device));
     NVR_HIP_CHECK(hipStreamCreateWithFlags(&r.stream, hipStreamNonBlocking));
-    RC(kl::prepare()); RC(kl::prepare_blocks());
+    RC(kl::prepare()); RC(kl::prepare_blocks()); RC(kl::prepare_streams());
     if (r.f32) RC(nvr::kf::prepare());
     else { RC(nvr::kb::linear_stream_prepare()); RC(nvr::kb::gemm_tiled_prepare()); }
     { int v = 0; if (hipDeviceGetAttribute(&v, hipDeviceAttributeMultiprocessorCount, r.device) == hipSuccess && v > 0) r.num_cus = v; }
@@ -76,6 +76,7 @@ int LayeredModel::init(nvr_model_runner &r) {
     if (spec.layout == LayeredSpec::SEQUENTIAL) RC(init_sequential(r));
     else if (spec.layout == LayeredSpec::SCALED) RC(init_scaled(r));
     else if (spec.layout == LayeredSpec::JOINT) RC(init_joint(r));
+    else if (spec.layout == LayeredSpec::STREAMS) RC(init_streams(r));
     else {
     // weights (zero until loaded)
     const int64_t taps = spec.taps;
@@ -162,8 +163,8 @@ int LayeredModel::init(nvr_model_runner &r) {
     RC(dmalloc(&xsel, (size_t)(std::max(MT, logit_rows_cap) * W * esz)));
     RC(dmalloc(&r.logits, (size_t)(logit_rows_cap * V * 4)));
 
-    // step inputs: ids | row_seq | want | cu | start | slot | par | block tables
-    in_bytes = (size_t)(MT * 8 + MT * 4 * 2 + (r.max_seqs + 1) * 4 + r.max_seqs * 4 * 3 + r.max_seqs * r.max_blocks_per_seq * 4 + 256) +
+    // step inputs: ids | row_seq | want | cu | start | slot | par | context lengths | block tables
+    in_bytes = (size_t)(MT * 8 + MT * 4 * 2 + (r.max_seqs + 1) * 4 + r.max_seqs * 4 * 4 + r.max_seqs * r.max_blocks_per_seq * 4 + 256) +
                (attn_groups.size() + 2 * flash_groups.size()) * (size_t)((MT + r.max_seqs) * sizeof(kl::AttnTile) + 16);
     attn_ws_bytes = kl::sink_attention_workspace_bytes(4 * r.num_cus);
     NVR_HIP_CHECK(hipMalloc(&attn_ws, attn_ws_bytes));
@@ -207,6 +208,7 @@ int LayeredModel::load_tensor(nvr_model_runner &r, const char *name_in, int dtyp
     if (spec.layout == LayeredSpec::SEQUENTIAL) return load_sequential(r, name, dtype, shape, ndim, data);
     if (spec.layout == LayeredSpec::SCALED) return load_scaled(r, name, dtype, shape, ndim, data);
     if (spec.layout == LayeredSpec::JOINT) return load_joint(r, name, dtype, shape, ndim, data);
+    if (spec.layout == LayeredSpec::STREAMS) return load_streams(r, name, dtype, shape, ndim, data);
     const int64_t W = spec.width, V = spec.vocab;
     auto is2 = [&](int64_t a, int64_t b) { return ndim == 2 && shape[0] == a && shape[1] == b; };
     auto bad = [&]() { return fail(NVR_ERR_LEN_MISMATCH, "load_tensor: '%s' has the wrong shape", name_in); };
@@ -289,7 +291,7 @@ int LayeredModel::execute(nvr_model_runner &r, nvr_seq *const *seqs, size_t nseq
     size_t off = 0;
     auto carve = [&](size_t bytes) { size_t o = off; off += (bytes + 15) / 16 * 16; return o; };
     const size_t o_ids = carve((size_t)T * 8), o_rs = carve((size_t)T * 4), o_want = carve(std::max<size_t>(R, 1) * 4), o_cu = carve((nseq + 1) * 4), o_st = carve(nseq * 4),
-                 o_sl = carve(nseq * 4), o_par = carve(nseq * 4), o_bt = carve(nseq * (size_t)MB * 4);
+                 o_sl = carve(nseq * 4), o_par = carve(nseq * 4), o_ctx = carve(nseq * 4), o_bt = carve(nseq * (size_t)MB * 4);
     // query tiles of the matrix-core attention, one list per distinct group size g = H / G: 64 / g positions of one sequence each
     std::vector<size_t> o_tiles(attn_groups.size()); std::vector<int32_t> n_tiles(attn_groups.size(), 0);
     for (size_t gi = 0; gi < attn_groups.size(); ++gi) {
@@ -323,11 +325,11 @@ int LayeredModel::execute(nvr_model_runner &r, nvr_seq *const *seqs, size_t nseq
             for (int64_t r0 = 0; r0 < (int64_t)seqs[i]->chunk_len; r0 += pw) *tl++ = kl::AttnTile{(int32_t)i, (int32_t)r0};
     }
     int64_t *ids = (int64_t *)(in_host + o_ids); int32_t *rowseq = (int32_t *)(in_host + o_rs), *wnt = (int32_t *)(in_host + o_want), *cu = (int32_t *)(in_host + o_cu),
-            *stt = (int32_t *)(in_host + o_st), *sl = (int32_t *)(in_host + o_sl), *par = (int32_t *)(in_host + o_par), *bt = (int32_t *)(in_host + o_bt);
+            *stt = (int32_t *)(in_host + o_st), *sl = (int32_t *)(in_host + o_sl), *par = (int32_t *)(in_host + o_par), *ctx = (int32_t *)(in_host + o_ctx), *bt = (int32_t *)(in_host + o_bt);
     int64_t t = 0;
     for (size_t i = 0; i < nseq; ++i) {
         const nvr_seq *s = seqs[i];
-        cu[i] = (int32_t)t; stt[i] = (int32_t)s->chunk_start; sl[i] = s->state_slot;
+        cu[i] = (int32_t)t; stt[i] = (int32_t)s->chunk_start; sl[i] = s->state_slot; ctx[i] = (int32_t)(s->chunk_start + s->chunk_len);
         if (s->chunk_start == 0) slot_par[(size_t)s->state_slot] = 0;     // a sequence's first tokens read no history: whatever the slot held is dead
         par[i] = slot_par[(size_t)s->state_slot];
         for (size_t j = 0; j < s->chunk_len; ++j, ++t) {
@@ -352,6 +354,7 @@ int LayeredModel::execute(nvr_model_runner &r, nvr_seq *const *seqs, size_t nseq
     for (size_t i = 0; i < nseq && decode_sized; ++i) decode_sized = seqs[i]->chunk_len == 1;
     StepPlan plan{b, d_want, (int64_t)R, T, max_ctx, o_tiles, n_tiles, o_ftiles, n_ftiles, decode_sized};
     plan.whole_prompts = !decode_sized;
+    plan.d_ctx = (const int32_t *)(in_dev + o_ctx);
     for (size_t i = 0; i < nseq && plan.whole_prompts; ++i) plan.whole_prompts = seqs[i]->chunk_start == 0;
     if (decode_sized && !r.cfg.enforce_eager) {
         const int64_t bucket = (max_ctx + 255) / 256 * 256;
@@ -392,6 +395,7 @@ int LayeredModel::forward(nvr_model_runner &r, const StepPlan &p) {
     if (spec.layout == LayeredSpec::SEQUENTIAL) return forward_sequential(r, p);
     if (spec.layout == LayeredSpec::SCALED) return forward_scaled(r, p);
     if (spec.layout == LayeredSpec::JOINT) return forward_joint(r, p);
+    if (spec.layout == LayeredSpec::STREAMS) return forward_streams(r, p);
     const kl::Batch &b = p.b;
     const int32_t *d_want = p.d_want;
     const int64_t T = p.T, R = p.R, max_ctx = p.max_ctx;

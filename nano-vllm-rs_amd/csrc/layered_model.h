@@ -20,6 +20,11 @@
 //                          decay per token and key channel, a bonus for the current token), each branch normed, half their sum; the feed-forward is a mixture of
 //                          clamped gated experts (softmax router, renormalised top-k, a gated shared expert); a range of layers runs several times with the same
 //                          weights, every pass starting with a product over [x ; embedding output] (layered_joint.cpp).
+//   streams (Negunex)    — the residual is a set of parallel streams (hyper-connections): every sublayer reads a weighted sum of them through a layer norm, and its result
+//                          joins all of them while a small matrix mixes them; the mixer is softmax attention with projection biases, rotated number pairs (frequencies
+//                          stretched for long contexts), unit norms per head behind the rotation, values mixed with the first such layer's and an output gate; the
+//                          feed-forward is dense with a gated GELU or a mixture of experts some of which return their input, chosen by corrected scores
+//                          (layered_streams.cpp).
 //
 // The family shares the runner's step interface (sequences with a chunk [start, start + len) each: whole prompts, portions of prompts and
 // single decoded tokens in one batch), the block manager's tables (K/V pages) and state slots (recurrent state, convolution history), the
@@ -39,9 +44,9 @@ struct nvr_model_runner;
 namespace nvr {
 
 struct LayeredSpec {
-    enum Mixer { ATTENTION = 0, RETENTION = 1, LATENT = 2, GLA = 3, MLSTM = 4, ATTN_GRU = 5, SSM = 6, ATTN_TMIX = 7 };
-    enum Ff { FF_NONE = 0, FF_CLAMPED_GLU = 1, FF_POLY = 2, FF_MOE = 3, FF_RELU2 = 4, FF_MOE_GLU = 5 };
-    enum Layout { PARALLEL = 0, SEQUENTIAL = 1, SCALED = 2, JOINT = 3 };
+    enum Mixer { ATTENTION = 0, RETENTION = 1, LATENT = 2, GLA = 3, MLSTM = 4, ATTN_GRU = 5, SSM = 6, ATTN_TMIX = 7, ATTN_UNIT = 8 };
+    enum Ff { FF_NONE = 0, FF_CLAMPED_GLU = 1, FF_POLY = 2, FF_MOE = 3, FF_RELU2 = 4, FF_MOE_GLU = 5, FF_GEGLU = 6, FF_MOE_IDENT = 7 };
+    enum Layout { PARALLEL = 0, SEQUENTIAL = 1, SCALED = 2, JOINT = 3, STREAMS = 4 };
     struct Layer {
         int mixer = ATTENTION;
         int64_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
@@ -67,6 +72,9 @@ struct LayeredSpec {
         // attention over chunks without softmax: position i sees j <= i with floor(j / chunk) == floor(i / chunk); scores capped at softcap (0: not); the rotation's
         // frequencies are divided by rot_factor
         int64_t chunk = 0; double softcap = 0.0, rot_factor = 1.0;
+        // streams layout: the rotation's frequencies stretched by wavelength (rot_original 0: not) — kept below rot_original / rot_high, divided by rot_factor above
+        // rot_original / rot_low, blended between —, values mixed with the first v_mix layer's, experts without a matrix behind the `experts` others
+        double rot_low = 1.0, rot_high = 1.0, rot_original = 0.0; bool v_mix = false; int64_t identity = 0;
         int64_t t_heads = 0, t_dim = 0;                     // the time-mixing recurrence beside the attention: heads of t_dim x t_dim states
     };
     int layout = PARALLEL;
@@ -74,6 +82,7 @@ struct LayeredSpec {
     int64_t side_dim = 0;                                   // per-layer token input: numbers per layer and token (0: none)
     int64_t vocab = 0, width = 0;
     double embedding_scale = 1.0, eps = 1e-5, residual_mult = 1.0;
+    int64_t streams = 1;                                    // streams layout: parallel residual streams
     int64_t max_positions = 0;                              // learned position vectors (0: none)
     double logit_scale = 1.0;
     int64_t taps = 1;                                       // causal convolution in front of every sublayer (1: a pointwise gain)
@@ -86,6 +95,7 @@ struct LayeredSpec {
     static int parse_pusunex(const Json &cfg, LayeredSpec *out);
     static int parse_sosutar(const Json &cfg, LayeredSpec *out);
     static int parse_sokalorn(const Json &cfg, LayeredSpec *out);
+    static int parse_negunex(const Json &cfg, LayeredSpec *out);
 };
 
 class LayeredModel {
@@ -127,6 +137,10 @@ public:
         void *w4 = nullptr, *w1 = nullptr, *w2 = nullptr; int64_t t_rank = 0;         // time mixing: r / k / v / g stacked [4][Ht Dt][W]; decay projections [rank][W], [Ht Dt][rank]
         float *w0 = nullptr, *bonus = nullptr, *tnorm = nullptr;                      // [Ht Dt] each
         void *router_op = nullptr;                                                   // [E + 1, padded to 16][W] operand type: the router's rows, then the shared expert's gate
+        // streams layout: what a sublayer reads from the streams [S], writes into them [S], and their mixing matrix [S][S] (from, to); projection biases; the share of the first
+        // layer's values; the experts' choice correction
+        float *hin[2] = {nullptr, nullptr}, *hout[2] = {nullptr, nullptr}, *hmix[2] = {nullptr, nullptr};
+        float *bq = nullptr, *bk = nullptr, *bv = nullptr, *vmix = nullptr, *ecorr = nullptr;
     };
     struct RunState { void *kc = nullptr, *vc = nullptr; float *state = nullptr, *hist = nullptr; bool borrowed = false; void *rows = nullptr; float *mstate = nullptr;
                       float *shist = nullptr, *chist = nullptr; };   // joint layout: hist the norm output before the step [2][slots][W], shist the mixer input's (time mixing), chist the convolution's inputs   // mstate: a matrix memory's running maxima [slots][H]   // borrowed: another run's pages (a shared latent)
@@ -148,6 +162,9 @@ public:
     void *conv_o = nullptr, *mixes = nullptr, *tproj = nullptr, *tlow = nullptr, *tz = nullptr, *tcat = nullptr; float *shared_g = nullptr;
     int64_t tlow_cap = 0; float *rlogits = nullptr;                          // router logits of a step [max tokens][experts + 1, padded]
     float *lm_part = nullptr;                          // arg-max partials of the 256 x 256 product with f32 output (not read)
+    // streams layout
+    void *v_first = nullptr;                                                // the step's values of the first layer that mixes: [max tokens][G Dv]
+    void *dec_ws = nullptr; size_t dec_ws_bytes = 0; unsigned int *dec_tickets = nullptr; int64_t dec_tickets_n = 0;   // the dense graph's decode attention: split partials, arrival counters (zero between launches)
     std::vector<void *> owned;                                              // device allocations of the sequential layout (freed with the model)
     // activations
     float *x = nullptr, *ret_o = nullptr;                                  // residual stream, retention outputs: f32
@@ -172,7 +189,8 @@ public:
 
 private:
     struct StepPlan { kl::Batch b; const int32_t *d_want; int64_t R, T, max_ctx; std::vector<size_t> o_tiles; std::vector<int32_t> n_tiles;
-                      std::vector<size_t> o_ftiles; std::vector<int32_t> n_ftiles; bool decode_sized; bool whole_prompts = false; };
+                      std::vector<size_t> o_ftiles; std::vector<int32_t> n_ftiles; bool decode_sized; bool whole_prompts = false;
+                      const int32_t *d_ctx = nullptr; };                     // d_ctx: keys each sequence's last row of the step sees
     int forward(nvr_model_runner &r, const StepPlan &p);
     int init_sequential(nvr_model_runner &r);
     int load_sequential(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
@@ -183,6 +201,9 @@ private:
     int init_joint(nvr_model_runner &r);
     int load_joint(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
     int forward_joint(nvr_model_runner &r, const StepPlan &p);
+    int init_streams(nvr_model_runner &r);
+    int load_streams(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
+    int forward_streams(nvr_model_runner &r, const StepPlan &p);
     template <class T> int own(T **p, size_t bytes);
     int gemm(nvr_model_runner &r, const void *a, int64_t lda, const void *w, int64_t T, int64_t K, int64_t N, void *y, bool y_f32 = false);
     int put(nvr_model_runner &r, void *dst, int64_t dst_ld, int64_t rows, int64_t cols, int dtype, const void *src, bool as_operand);

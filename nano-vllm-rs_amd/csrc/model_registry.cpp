@@ -70,6 +70,11 @@ int parse_sokalorn_spec(const Json &c, nvr_model_spec *out) {
     return LayeredSpec::parse_sokalorn(c, &out->layered);
 }
 
+int parse_negunex_spec(const Json &c, nvr_model_spec *out) {
+    out->family = 1;
+    return LayeredSpec::parse_negunex(c, &out->layered);
+}
+
 struct Entry { const char *name; int (*parse)(const Json &, nvr_model_spec *); };
 const Entry kRegistry[] = {
     {"Qwen3ForCausalLM", parse_qwen3},
@@ -77,6 +82,7 @@ const Entry kRegistry[] = {
     {"Pusunex", parse_pusunex_spec},
     {"Sosutar", parse_sosutar_spec},
     {"Sokalorn", parse_sokalorn_spec},
+    {"Negunex", parse_negunex_spec},
 };
 
 }  // namespace
@@ -375,6 +381,81 @@ int LayeredSpec::parse_sokalorn(const Json &c, LayeredSpec *s) {
         for (int64_t i = b; i < n; ++i) { s->runs.push_back((int)i); s->pass_start.push_back(0); }
     } else
         for (int64_t i = 0; i < n; ++i) { s->runs.push_back((int)i); s->pass_start.push_back(0); }
+    return NVR_OK;
+}
+
+// Negunex: `streams` parallel residual streams; every sublayer reads a weighted sum of them through a layer norm and writes into all of them.  Mixer 'attention'
+// (mixer.{heads, kv_heads, dim, vdim, scale}, optional rot.{dims, base, scaling.{factor, low, high, original}}, optional v_mix); feed-forward 'dense' (gated GELU) or 'moe'
+// (expert.ff, router.{experts, top, optional identity}) or none.
+int LayeredSpec::parse_negunex(const Json &c, LayeredSpec *s) {
+    Reader rd;
+    s->layout = STREAMS; s->taps = 1; s->residual_mult = 1.0; s->norm_groups = 1; s->embedding_scale = 1.0;
+    s->vocab = rd.integer(c, "vocab", ""); s->width = rd.integer(c, "width", ""); s->streams = rd.integer(c, "streams", "");
+    if (const Json *n = rd.need(c, "norm", "")) s->eps = rd.num(*n, "eps", "norm.");
+    const Json *layers = rd.need(c, "layers", "");
+    if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+    if (layers->kind != Json::Arr || layers->arr.empty()) return fail(NVR_ERR_INVALID_ARG, "config: 'layers' is not a list of layers");
+    if (s->vocab < 1 || s->width < 1 || s->streams < 1) return fail(NVR_ERR_INVALID_ARG, "config: vocab, width and streams must be positive");
+    s->layers.clear(); s->runs.clear();
+    int64_t first_mix = -1;
+    for (size_t i = 0; i < layers->arr.size(); ++i) {
+        const Json &lj = layers->arr[i];
+        const std::string w = "layers[" + std::to_string(i) + "].", wm = w + "mixer.";
+        Layer L;
+        const Json *type = rd.need(lj, "type", w), *mx = rd.need(lj, "mixer", w);
+        if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+        if (!(type->kind == Json::Str && type->str == "attention")) return fail(NVR_ERR_UNSUPPORTED, "config: layer type '%s' (attention)", type->kind == Json::Str ? type->str.c_str() : "");
+        L.mixer = ATTN_UNIT; L.out_gate = true;
+        L.heads = rd.integer(*mx, "heads", wm); L.kv_heads = rd.integer(*mx, "kv_heads", wm); L.dim = rd.integer(*mx, "dim", wm); L.vdim = rd.integer(*mx, "vdim", wm);
+        L.scale = rd.num(*mx, "scale", wm);
+        const Json *rot = mx->get("rot");
+        if (rot && !rot->is_null()) {
+            L.rot_dims = rd.integer(*rot, "dims", wm + "rot."); L.rot_base = rd.num(*rot, "base", wm + "rot.");
+            const Json *sc = rot->get("scaling");
+            if (sc && !sc->is_null()) {
+                const std::string ws = wm + "rot.scaling.";
+                L.rot_factor = rd.num(*sc, "factor", ws); L.rot_low = rd.num(*sc, "low", ws); L.rot_high = rd.num(*sc, "high", ws); L.rot_original = rd.num(*sc, "original", ws);
+                if (rd.err.empty() && !(L.rot_factor > 0 && L.rot_low > 0 && L.rot_high >= L.rot_low && L.rot_original > 0))
+                    return fail(NVR_ERR_INVALID_ARG, "config: %s factor, low and original must be positive and high at least low", ws.c_str());
+            }
+        }
+        if (rd.err.empty() && (L.rot_dims < 0 || L.rot_dims % 2 || L.rot_dims > L.dim || !(L.rot_base > 0)))
+            return fail(NVR_ERR_INVALID_ARG, "config: %s needs an even rot.dims <= dim and a positive base", wm.c_str());
+        const Json *vm = mx->get("v_mix");
+        if (vm && !vm->is_null()) {
+            if (vm->kind != Json::Bool) return fail(NVR_ERR_INVALID_ARG, "config: '%sv_mix' is not true or false", wm.c_str());
+            L.v_mix = vm->b;
+        }
+        const Json *mlp = lj.get("mlp");
+        if (mlp && !mlp->is_null()) {
+            const Json *kind = rd.need(*mlp, "kind", w + "mlp.");
+            L.has_mlp = true;
+            if (kind && kind->kind == Json::Str && kind->str == "dense") {
+                L.ff_kind = FF_GEGLU; L.ff = rd.integer(*mlp, "ff", w + "mlp.");
+                if (rd.err.empty() && L.ff < 1) return fail(NVR_ERR_INVALID_ARG, "config: '%smlp.ff' must be positive", w.c_str());
+            } else if (kind && kind->kind == Json::Str && kind->str == "moe") {
+                L.ff_kind = FF_MOE_IDENT;
+                const Json *ex = rd.need(*mlp, "expert", w + "mlp."), *ro = rd.need(*mlp, "router", w + "mlp.");
+                if (ex) L.expert_ff = rd.integer(*ex, "ff", w + "mlp.expert.");
+                if (ro) {
+                    L.experts = rd.integer(*ro, "experts", w + "mlp.router."); L.top = rd.integer(*ro, "top", w + "mlp.router.");
+                    const Json *id = ro->get("identity");
+                    if (id && !id->is_null()) L.identity = rd.integer(*ro, "identity", w + "mlp.router.");
+                }
+                if (rd.err.empty() && (L.expert_ff < 1 || L.experts < 1 || L.identity < 0 || L.top < 1 || L.top > L.experts + L.identity))
+                    return fail(NVR_ERR_INVALID_ARG, "config: %smlp needs positive expert sizes, identity >= 0 and 1 <= top <= experts + identity", w.c_str());
+            } else if (kind) return fail(NVR_ERR_UNSUPPORTED, "config: '%smlp.kind' (dense or moe)", w.c_str());
+        }
+        if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+        if (L.heads < 1 || L.dim < 1 || L.vdim < 1 || L.kv_heads < 1 || L.heads % L.kv_heads)
+            return fail(NVR_ERR_INVALID_ARG, "config: %s %ld heads over %ld key/value heads of %ld / %ld", w.c_str(), (long)L.heads, (long)L.kv_heads, (long)L.dim, (long)L.vdim);
+        if (L.v_mix) {
+            if (first_mix < 0) first_mix = (int64_t)i;
+            else if (s->layers[(size_t)first_mix].kv_heads * s->layers[(size_t)first_mix].vdim != L.kv_heads * L.vdim)
+                return fail(NVR_ERR_INVALID_ARG, "config: '%sv_mix' mixes values of other sizes than layer %ld's", wm.c_str(), (long)first_mix);
+        }
+        s->layers.push_back(L); s->runs.push_back((int)i);
+    }
     return NVR_OK;
 }
 
