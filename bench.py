@@ -703,7 +703,7 @@ def main() -> None:
                          "retention, clamped gated feed-forward; Pusunex: latent attention, gated linear attention, experts; Sosutar: matrix memory, windowed attention beside a gated recurrence; Sokalorn: state-space mixer, chunked sigmoid attention beside time mixing, clamped experts) beside the dense Qwen3 graph at equal "
                          "layer sizes, random weights, one JSON line per size")
     ap.add_argument("--layered-sizes", default="w1024,w2048", help="sizes of --layered-compare (w1024, w2048, w4096)")
-    ap.add_argument("--layered-models", default="rugudra,qwen3", help="models of --layered-compare (rugudra, pusunex, sosutar, sokalorn, qwen3)")
+    ap.add_argument("--layered-models", default="rugudra,qwen3", help="models of --layered-compare (rugudra, pusunex, sosutar, sokalorn, negunex, negunex4, qwen3)")
     args = ap.parse_args()
     if args.layered_compare:
         import importlib

@@ -46,7 +46,7 @@ struct G256Epi {
     int32_t H, KVH, D;
     int32_t kv_cache_only;             // GEPI_ROPE: k and v rows go to the caches only (the attention that follows reads them there)
     float *logits; float *pval; int32_t *pidx;   // GEPI_LMHEAD: f32 logits [T][N] (nullable), arg-max partials [tiles_x][T]
-    const int32_t *row_w; int64_t w_stride;      // GRP (rows grouped by expert): row block rb of 256 rows multiplies the matrix W + row_w[rb] * w_stride
+    const int32_t *row_w; int64_t w_stride; const int32_t *rows_used;      // (rows_used, on the device: rows behind it are nobody's; null: all T) GRP (rows grouped by expert): row block rb of 256 rows multiplies the matrix W + row_w[rb] * w_stride
 };
 
 constexpr int G_BK = 64, G_HT = 128, G_HALF = G_HT * G_BK * 2;          // 16 KiB per half-tile
@@ -86,7 +86,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
     // groups x 8/CG row groups; an XCD owns the columns of its group (its W slice stays L2-resident) and every
     // (8/CG)-th row block, and its workgroups walk that set column-fastest, so the workgroups that share an x row block
     // run on ONE XCD at the same time: x is fetched from HBM CG times instead of once per XCD that happens to see it.
-    const int tiles_total = tiles_x * tiles_y;
+    const int tiles_total = tiles_x * (GRP && epi.rows_used ? min(tiles_y, (*epi.rows_used + 255) / 256) : tiles_y);     // (row blocks are the slow index of the tile order)
     int xcd_step = 0, u = 0, nbx = 0, bx0 = 0, rg = 0, RG = 1, n_u = 0;
     if (CG > 0) {
         const int c = blockIdx.x & 7;
@@ -556,19 +556,19 @@ int gemm256_relu2(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T
 }
 // Rows grouped by expert (a mixture of experts over many tokens): T is a multiple of 256 and row block rb multiplies the matrix W + row_w[rb] * w_stride
 // (row_w on the device: the host does not know how many rows an expert got).  y = x . W_e^T, or out = silu(gate) * up with W_e = [gate rows; up rows].
-int gemm256_grouped(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s) {
+int gemm256_grouped(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s, const int32_t *rows_used) {
     if (!gemm256_ok(T, K, N, ldx) || T % 256) return nvr::fail(NVR_ERR_UNSUPPORTED, "gemm256_grouped: T=%ld K=%ld N=%ld", (long)T, (long)K, (long)N);
     if (int rc = g256_prepare()) return rc;
-    G256Epi e{}; e.row_w = row_w; e.w_stride = w_stride;
+    G256Epi e{}; e.row_w = row_w; e.w_stride = w_stride; e.rows_used = rows_used;
     const int tx = (int)(N / 256), tt = tx * (int)(T / 256);
     gemm256_kernel<GEPI_F16, 0, true><<<dim3((unsigned)g256_grid(tt)), dim3(512), 2 * G_BUF, s>>>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)N, (int)N, (half_t *)y, e, tx,
                                                                                                   tt / tx, 0);
     return g256_check("gemm256_grouped");
 }
-int gemm256_grouped_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s) {
+int gemm256_grouped_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s, const int32_t *rows_used) {
     if (!gemm256_silu_ok(T, K, I, ldx) || T % 256) return nvr::fail(NVR_ERR_UNSUPPORTED, "gemm256_grouped_silu_mul: T=%ld K=%ld I=%ld", (long)T, (long)K, (long)I);
     if (int rc = g256_prepare()) return rc;
-    G256Epi e{}; e.row_w = row_w; e.w_stride = w_stride;
+    G256Epi e{}; e.row_w = row_w; e.w_stride = w_stride; e.rows_used = rows_used;
     const int tx = (int)(I / 128), tt = tx * (int)(T / 256);
     gemm256_kernel<GEPI_SILU, 0, true><<<dim3((unsigned)g256_grid(tt)), dim3(512), 2 * G_BUF, s>>>((const half_t *)x, ldx, (const half_t *)W, (int)T, (int)K, (int)I, (int)(2 * I), (half_t *)out, e,
                                                                                                    tx, tt / tx, 0);

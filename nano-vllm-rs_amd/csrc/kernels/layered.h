@@ -157,7 +157,7 @@ int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool 
 
 // Router of a mixture of experts: logits wr h in f32 (wr: [E][W] f32), the top largest per token -> sel / score (= sigmoid of the logit) [T][top]; then the rows
 // grouped by expert: off [E + 1], order [T top] (place -> token * top + choice), place_of (its inverse).  With pad > 1 every expert's rows start at a multiple of pad
-// (places then run up to (T top / pad + E) pad) and row_w[block] names the expert of each of the nblocks blocks of pad rows: the form a tiled product over whole
+// (places then run up to (T top / pad + E) pad) and row_w[block] names the expert of each of the nblocks blocks of pad rows (and has room for 1024 further numbers behind them): the form a tiled product over whole
 // row blocks wants, with the rows brought together by moe_gather (xs[place] = h[token] * score).
 // softmax: score is the chosen experts' share of the softmax over ALL experts, divided by the sum of the chosen shares (+ 1e-20), instead of the sigmoid.
 // correction (softmax, [E] f32): the choice is made by share + correction, the scores stay the shares.  identity > 0: the last `identity` of the E outputs have no matrix (their expert
@@ -284,6 +284,9 @@ struct StreamArgs {
     const void *y; int64_t ldy; const float *mix, *wout;
     const float *win, *w; void *out; int64_t ldo;
     const int32_t *rows; bool sum;
+    // place not null ([T][top], -1: none): y of row t is the weighted sum of a token's chosen experts' rows, sum_k score[t][k] * (place < 0 ? ident row t : y row place) — what
+    // moe_combine would have stored, unrounded
+    const int32_t *place; int32_t top; const float *score; const void *ident; int64_t ldi;
 };
 int stream_step(const StreamArgs &a, bool bf16, hipStream_t s);
 

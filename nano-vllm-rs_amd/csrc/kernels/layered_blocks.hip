@@ -577,6 +577,80 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const OT *__restrict__ h
     if (softmax && threadIdx.x == 0) for (int k = 0; k < top; ++k) score[t * top + k] /= chosen + 1e-20f;
 }
 
+// The same for logits formed beforehand and at most 64 experts: a wave per token, the experts across its lanes, nothing in LDS.  Lane k < top leaves with choice k and its score.
+__device__ __forceinline__ void route_wave(int64_t t, int E, int top, int softmax, int extra, float *__restrict__ extra_out, const float *__restrict__ logits, int64_t ldl,
+                                           const float *__restrict__ correction, int &my, float &mine) {
+    const int lane = threadIdx.x & 63;
+    const float *lr = logits + t * ldl;
+    if (lane < extra) extra_out[t * extra + lane] = lr[E + lane];
+    const float z = lane < E ? lr[lane] : -INFINITY;
+    float sv = 0.f;
+    if (softmax) {
+        float zmax = z;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) zmax = fmaxf(zmax, __shfl_xor(zmax, o, 64));
+        sv = lane < E ? expf(z - zmax) : 0.f;
+        sv /= wave_sum(sv);
+    } else if (lane < E) sv = sigmoid_f(z);
+    const float ch = lane < E ? (correction ? sv + correction[lane] : z) : -INFINITY;      // what the choice compares
+    bool open = lane < E;                               // not chosen yet
+    float chosen = 0.f;
+    my = -1; mine = 0.f;
+    for (int k = 0; k < top; ++k) {
+        float best = open ? ch : -INFINITY; int bi = open ? lane : 64;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ob = __shfl_xor(best, o, 64); const int oi = __shfl_xor(bi, o, 64);
+            if (ob > best || (ob == best && oi < bi) || (bi == 64 && oi < 64)) { best = ob; bi = oi; }
+        }
+        bi = min(bi, E - 1);                            // (choices that are not numbers: the index still has to be an expert's)
+        const float s = __shfl(sv, bi, 64);
+        if (lane == k) { my = bi; mine = s; }
+        chosen += s;
+        if (lane == bi) open = false;
+    }
+    if (softmax) mine /= chosen + 1e-20f;
+}
+__global__ __launch_bounds__(256) void moe_route_wave_kernel(int T, int E, int top, int32_t *__restrict__ sel, float *__restrict__ score, int softmax, int extra,
+                                                             float *__restrict__ extra_out, const float *__restrict__ logits, int64_t ldl, const float *__restrict__ correction) {
+    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6); const int lane = threadIdx.x & 63;
+    if (t >= T) return;                                 // (a whole wave)
+    int my; float mine;
+    route_wave(t, E, top, softmax, extra, extra_out, logits, ldl, correction, my, mine);
+    if (lane < top) { sel[t * top + lane] = my; score[t * top + lane] = mine; }
+}
+
+// Few tokens: both of the two steps above and below in one workgroup — the choices of up to 1024 (token, choice) pairs, then the experts' groups (rows not padded).
+__global__ __launch_bounds__(1024) void moe_route_group_kernel(int T, int E, int El, int top, int32_t *__restrict__ sel, float *__restrict__ score, int softmax, int extra,
+                                                               float *__restrict__ extra_out, const float *__restrict__ logits, int64_t ldl, const float *__restrict__ correction,
+                                                               int32_t *__restrict__ off, int32_t *__restrict__ order, int32_t *__restrict__ place_of) {
+    __shared__ int32_t chosen_e[1024], cnt[65];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    if (threadIdx.x < 65) cnt[threadIdx.x] = 0;
+    __syncthreads();
+    for (int t = wave; t < T; t += 16) {
+        int my; float mine;
+        route_wave(t, E, top, softmax, extra, extra_out, logits, ldl, correction, my, mine);
+        if (lane < top) { sel[t * top + lane] = my; score[t * top + lane] = mine; chosen_e[t * top + lane] = my; if (my < El) atomicAdd(&cnt[my], 1); }
+    }
+    __syncthreads();
+    if (wave == 0) {                                    // exclusive sum over the experts, one per lane
+        const int c = lane < El ? cnt[lane] : 0;
+        int run = c;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) { const int v = __shfl_up(run, o, 64); if (lane >= o) run += v; }
+        if (lane < El) { cnt[lane] = run - c; off[lane] = run - c; }
+        if (lane == El - 1) off[El] = run;
+    }
+    __syncthreads();
+    const int i = threadIdx.x;
+    if (i < T * top) {
+        const int e = chosen_e[i];
+        if (e >= El) place_of[i] = -1;
+        else { const int place = atomicAdd(&cnt[e], 1); order[place] = i; place_of[i] = place; }
+    }
+}
+
 // One workgroup: counts per expert, offsets, and a place for every (token, choice) among its expert's rows.  order[place] = token * top + choice;
 // place_of[token * top + choice] = place (-1: a choice >= E has no group).  Which place inside its expert a row gets is left to the atomics: a row's result does not depend on it.
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restrict__ sel, int n, int E, int pad, int nblocks, int32_t *__restrict__ off,
@@ -605,6 +679,49 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restri
     }
 }
 
+// The same over many choices, in two launches of nb workgroups with a stretch of the choices each: counts[b][e] first; then every workgroup adds up the counts before its own, so that its
+// places start where the stretches before it end (workgroup 0 also writes the offsets and the blocks' experts).
+__global__ __launch_bounds__(256) void moe_count_kernel(const int32_t *__restrict__ sel, int n, int per, int E, int32_t *__restrict__ counts) {
+    extern __shared__ int32_t cnt[];                    // [E]
+    for (int e = threadIdx.x; e < E; e += 256) cnt[e] = 0;
+    __syncthreads();
+    const int i0 = blockIdx.x * per, i1 = min(n, i0 + per);
+    for (int i = i0 + threadIdx.x; i < i1; i += 256) if (sel[i] < E) atomicAdd(&cnt[sel[i]], 1);
+    __syncthreads();
+    for (int e = threadIdx.x; e < E; e += 256) counts[blockIdx.x * E + e] = cnt[e];
+}
+__global__ __launch_bounds__(256) void moe_place_kernel(const int32_t *__restrict__ sel, int n, int per, int E, int pad, int nblocks, const int32_t *__restrict__ counts, int nb,
+                                                        int32_t *__restrict__ off, int32_t *__restrict__ order, int32_t *__restrict__ place_of, int32_t *__restrict__ row_w) {
+    extern __shared__ int32_t sh[];                     // [E] the next place of every expert, [E + 1] offsets
+    int32_t *next = sh, *start = sh + E;
+    for (int e = threadIdx.x; e < E; e += 256) {
+        int before = 0, total = 0;
+        for (int b = 0; b < nb; ++b) { const int c = counts[b * E + e]; if (b < (int)blockIdx.x) before += c; total += c; }
+        next[e] = before; start[e] = total;
+    }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        int run = 0;
+        for (int e = 0; e < E; ++e) { const int padded = (start[e] + pad - 1) / pad * pad; start[e] = run; next[e] += run; run += padded; }
+        start[E] = run;
+    }
+    __syncthreads();
+    if (blockIdx.x == 0) {
+        for (int e = threadIdx.x; e <= E; e += 256) off[e] = start[e];
+        for (int bk = threadIdx.x; bk < nblocks; bk += 256) {         // (behind the last expert: any matrix, their rows are nobody's)
+            int w = 0;
+            if (bk * pad < start[E]) for (int e = 1; e < E; ++e) if (start[e] <= bk * pad) w = e;
+            row_w[bk] = w;
+        }
+    }
+    const int i0 = blockIdx.x * per, i1 = min(n, i0 + per);
+    for (int i = i0 + threadIdx.x; i < i1; i += 256) {
+        if (sel[i] >= E) { place_of[i] = -1; continue; }
+        const int place = atomicAdd(&next[sel[i]], 1);
+        order[place] = i; place_of[i] = place;
+    }
+}
+
 // xs[place_of[i]] = h[i / top] * score[i] (the expert's input, in the order of the grouped rows)
 template <class OT>
 __global__ __launch_bounds__(256) void moe_gather_kernel(const OT *__restrict__ h, int64_t ldh, int W, int top, const int32_t *__restrict__ place_of, const float *__restrict__ score,
@@ -614,6 +731,24 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(const OT *__restrict__ 
     const float sc = score[i];
     OT *dst = xs + (int64_t)place_of[i] * W;
     for (int c = threadIdx.x; c < W; c += 256) st_f(dst, c, ld_f(h, t * ldh + c) * sc);
+}
+
+// 16-bit rows, 8 numbers per thread (W and the stride multiples of 8, 16-byte aligned rows)
+__global__ __launch_bounds__(256) void moe_gather8_kernel(const bf16_t *__restrict__ h, int64_t ldh, int W8, int top, int64_t n, const int32_t *__restrict__ place_of,
+                                                          const float *__restrict__ score, bf16_t *__restrict__ xs) {
+    const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x, t = idx / W8;        // (token, piece): the piece is read once for all of the token's choices
+    if (t >= n) return;
+    const int64_t c = (idx - t * W8) * 8;
+    const uint4 v = *reinterpret_cast<const uint4 *>(h + t * ldh + c); const bf16_t *ve = reinterpret_cast<const bf16_t *>(&v);
+    for (int k = 0; k < top; ++k) {
+        const int64_t place = place_of[t * top + k];
+        if (place < 0) continue;
+        const float sc = score[t * top + k];
+        uint4 o; bf16_t *oe = reinterpret_cast<bf16_t *>(&o);
+#pragma unroll
+        for (int y = 0; y < 8; ++y) st_f(oe, y, ld_f(ve, y) * sc);
+        *reinterpret_cast<uint4 *>(xs + place * W8 * 8 + c) = o;
+    }
 }
 
 // out[t] = sum_k y[place_of[t * top + k]] (+ shared[t]) in the operand type
@@ -631,6 +766,45 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const OT *__restrict__
         }
         st_f(out, t * W + c, v);
     }
+}
+
+// 16-bit rows, 8 numbers per thread (W and the strides multiples of 8, 16-byte aligned rows); the choices' rows are requested four at a time
+__global__ __launch_bounds__(256) void moe_combine8_kernel(const bf16_t *__restrict__ y, const int32_t *__restrict__ place_of, int top, const bf16_t *__restrict__ shared, int W8, int64_t T,
+                                                           bf16_t *__restrict__ out, const float *__restrict__ score, const float *__restrict__ shared_gate, int64_t gate_ld,
+                                                           const bf16_t *__restrict__ ident, int64_t ldi) {
+    const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x, t = idx / W8;
+    if (t >= T) return;
+    const int64_t c = (idx - t * W8) * 8, W = (int64_t)W8 * 8;
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+    if (shared) {
+        const float sg = shared_gate ? sigmoid_f(shared_gate[t * gate_ld]) : 1.f;
+        const uint4 v = *reinterpret_cast<const uint4 *>(shared + t * W + c); const bf16_t *ve = reinterpret_cast<const bf16_t *>(&v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] = ld_f(ve, e) * sg;
+    }
+    for (int k0 = 0; k0 < top; k0 += 4) {
+        uint4 v[4]; float sc[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const bool on = k0 + k < top;
+            const int64_t i = t * top + (on ? k0 + k : 0), place = place_of[i];
+            sc[k] = on ? (score ? score[i] : 1.f) : 0.f;
+            v[k] = *reinterpret_cast<const uint4 *>(place < 0 ? ident + t * ldi + c : y + place * W + c);
+        }
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            if (k0 + k >= top) break;
+            const bf16_t *ve = reinterpret_cast<const bf16_t *>(&v[k]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[e] += ld_f(ve, e) * sc[k];
+        }
+    }
+    uint4 o; bf16_t *oe = reinterpret_cast<bf16_t *>(&o);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) st_f(oe, e, acc[e]);
+    *reinterpret_cast<uint4 *>(out + t * W + c) = o;
 }
 
 // ------------------------------------------------------------------------------------------------ end of a layer
@@ -833,16 +1007,33 @@ int moe_route(const void *h, int64_t ldh, int64_t T, int64_t W, const float *wr,
     if (extra < 0 || (extra > 0 && !extra_out)) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: %ld further rows without a place for them", (long)extra);
     if (top < 1 || top > E) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: %ld of %ld experts", (long)top, (long)E);
     if ((size_t)(2 * E + extra + 1) * 4 > 60000) return nvr::fail(NVR_ERR_UNSUPPORTED, "moe_route: %ld experts", (long)E);
-    if (bf16) moe_route_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra + (correction ? E : 0)) * 4, s>>>((const bf16_t *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
+    if (logits && E <= 64 && extra <= 64 && T * top <= 1024 && pad == 1 && !row_w) {
+        moe_route_group_kernel<<<dim3(1), dim3(1024), 0, s>>>((int)T, (int)E, (int)(E - identity), (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction, off, order, place_of);
+        return launched("moe_route");
+    }
+    if (logits && E <= 64 && extra <= 64)
+        moe_route_wave_kernel<<<dim3((unsigned)((T + 3) / 4)), dim3(256), 0, s>>>((int)T, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
+    else if (bf16) moe_route_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra + (correction ? E : 0)) * 4, s>>>((const bf16_t *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
     else moe_route_kernel<float><<<dim3((unsigned)T), dim3(256), (size_t)(E + extra + (correction ? E : 0)) * 4, s>>>((const float *)h, ldh, (int)W, wr, (int)E, (int)top, sel, score, softmax ? 1 : 0, (int)extra, extra_out, logits, ldl, correction);
     if (int rc = launched("moe_route")) return rc;
     if (pad < 1) return nvr::fail(NVR_ERR_INVALID_ARG, "moe_route: rows padded to %ld", (long)pad);
+    if (row_w && T * top >= 4096 && E - identity <= 256) {            // many choices: the counts of the workgroups go behind row_w
+        const int64_t n = T * top, El = E - identity, nb = std::min<int64_t>((n + 1023) / 1024, std::max<int64_t>(1, 1024 / El)), per = (n + nb - 1) / nb;
+        int32_t *counts = row_w + nblocks;
+        moe_count_kernel<<<dim3((unsigned)nb), dim3(256), (size_t)El * 4, s>>>(sel, (int)n, (int)per, (int)El, counts);
+        moe_place_kernel<<<dim3((unsigned)nb), dim3(256), (size_t)(2 * El + 1) * 4, s>>>(sel, (int)n, (int)per, (int)El, (int)pad, (int)nblocks, counts, (int)nb, off, order, place_of, row_w);
+        return launched("moe_place");
+    }
     moe_group_kernel<<<dim3(1), dim3(1024), (size_t)(E - identity + 1) * 4, s>>>(sel, (int)(T * top), (int)(E - identity), (int)pad, (int)nblocks, off, order, place_of, row_w);
     return launched("moe_group");
 }
 
 int moe_gather(const void *h, int64_t ldh, int64_t T, int64_t W, int64_t top, const int32_t *place_of, const float *score, void *xs, bool bf16, hipStream_t s) {
     if (T * top == 0) return 0;
+    if (bf16 && W % 8 == 0 && ldh % 8 == 0 && aligned16(h) && aligned16(xs)) {
+        moe_gather8_kernel<<<dim3((unsigned)((T * (W / 8) + 255) / 256)), dim3(256), 0, s>>>((const bf16_t *)h, ldh, (int)(W / 8), (int)top, T, place_of, score, (bf16_t *)xs);
+        return launched("moe_gather");
+    }
     if (bf16) moe_gather_kernel<bf16_t><<<dim3((unsigned)(T * top)), dim3(256), 0, s>>>((const bf16_t *)h, ldh, (int)W, (int)top, place_of, score, (bf16_t *)xs);
     else moe_gather_kernel<float><<<dim3((unsigned)(T * top)), dim3(256), 0, s>>>((const float *)h, ldh, (int)W, (int)top, place_of, score, (float *)xs);
     return launched("moe_gather");
@@ -851,6 +1042,11 @@ int moe_gather(const void *h, int64_t ldh, int64_t T, int64_t W, int64_t top, co
 int moe_combine(const void *y, const int32_t *place_of, int64_t T, int64_t top, const void *shared, int64_t W, void *out, bool bf16, hipStream_t s,
                 const float *score, const float *shared_gate, int64_t gate_ld, const void *ident, int64_t ldi) {
     if (T == 0) return 0;
+    if (bf16 && W % 8 == 0 && ldi % 8 == 0 && aligned16(y) && aligned16(shared) && aligned16(out) && aligned16(ident)) {
+        moe_combine8_kernel<<<dim3((unsigned)((T * (W / 8) + 255) / 256)), dim3(256), 0, s>>>((const bf16_t *)y, place_of, (int)top, (const bf16_t *)shared, (int)(W / 8), T, (bf16_t *)out, score, shared_gate,
+                                                                                             gate_ld, (const bf16_t *)ident, ldi);
+        return launched("moe_combine");
+    }
     if (bf16) moe_combine_kernel<bf16_t><<<dim3((unsigned)T), dim3(256), 0, s>>>((const bf16_t *)y, place_of, (int)top, (const bf16_t *)shared, (int)W, (bf16_t *)out, score, shared_gate, gate_ld, (const bf16_t *)ident, ldi);
     else moe_combine_kernel<float><<<dim3((unsigned)T), dim3(256), 0, s>>>((const float *)y, place_of, (int)top, (const float *)shared, (int)W, (float *)out, score, shared_gate, gate_ld, (const float *)ident, ldi);
     return launched("moe_combine");

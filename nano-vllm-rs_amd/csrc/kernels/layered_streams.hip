@@ -61,7 +61,14 @@ __global__ __launch_bounds__(256) void stream_step_kernel(StreamArgs a) {
             const float v = ld_f(er, c);
             for (int s = 0; s < S; ++s) { xr[(int64_t)s * W + c] = v; u += a.win[s] * v; }
         } else {
-            const float y = ld_f(yr, c);
+            float y;
+            if (a.place) {
+                y = 0.f;
+                for (int k = 0; k < a.top; ++k) {
+                    const int64_t pl = a.place[t * a.top + k];
+                    y += a.score[t * a.top + k] * (pl < 0 ? ld_f((const OT *)a.ident, t * a.ldi + c) : ld_f((const OT *)a.y, pl * a.ldy + c));
+                }
+            } else y = ld_f(yr, c);
             for (int s = 0; s < S; ++s) old[s * 256 + tid] = xr[(int64_t)s * W + c];
             for (int q = 0; q < S; ++q) {
                 float v = a.wout[q] * y;
@@ -81,30 +88,56 @@ __global__ __launch_bounds__(256) void stream_step_kernel(StreamArgs a) {
 
 // The step for 16-bit operands and widths that are multiples of 4: NT threads per row (64: a wave, four rows per workgroup, no barrier; 256: the workgroup), a row's
 // streams, result and u in registers, 16-byte loads and stores of the streams.
-template <int S, int NT, int NV>
+// KIND: the start, a step, or a step whose y is the weighted sum of a token's chosen experts' rows.
+enum { K_START = 0, K_STEP = 1, K_EXPERTS = 2 };
+template <int S, int NT, int NV, int KIND>
 __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
+    constexpr bool START = KIND == K_START;
     __shared__ float red[4];
     const int W = a.W, W4 = W >> 2, l = threadIdx.x & (NT - 1);
-    const int64_t t = (int64_t)blockIdx.x * (256 / NT) + threadIdx.x / NT;
-    if (NT == 64 && t >= a.T) return;                   // (a whole wave: nobody waits for it)
+    const int64_t r = (int64_t)blockIdx.x * (256 / NT) + threadIdx.x / NT;
+    if (NT == 64 && r >= a.T) return;                   // (a whole wave: nobody waits for it)
+    const int64_t t = a.rows ? a.rows[r] : r;
+    const bool sum = !START && a.sum;                   // (the end: u is the sum of the new streams, which stay where they were)
     float *xr = a.x + t * S * W;
-    const bf16_t *yr = (const bf16_t *)a.y + t * a.ldy;
-    float4 xs[NV][S]; uint2 ys[NV];
+    const bf16_t *yr = START ? (const bf16_t *)a.E + a.ids[t] * (int64_t)W : (const bf16_t *)a.y + t * a.ldy;      // (the start: every stream is this row)
+    float4 xs[NV][START ? 1 : S], yf[NV]; uint2 ys[NV];
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
         const int c4 = l + k * NT;
         if (c4 < W4) {
 #pragma unroll
-            for (int s = 0; s < S; ++s) xs[k][s] = *reinterpret_cast<const float4 *>(xr + (int64_t)s * W + c4 * 4);
-            ys[k] = *reinterpret_cast<const uint2 *>(yr + c4 * 4);
+            for (int s = 0; s < (START ? 0 : S); ++s) xs[k][s] = *reinterpret_cast<const float4 *>(xr + (int64_t)s * W + c4 * 4);
+            if (KIND != K_EXPERTS) ys[k] = *reinterpret_cast<const uint2 *>(yr + c4 * 4);
+        }
+    }
+    auto unpack = [](uint2 v) { return float4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)}; };
+    if (KIND == K_EXPERTS) {                            // the choices' rows are requested four at a time
+#pragma unroll
+        for (int k = 0; k < NV; ++k) yf[k] = float4{0.f, 0.f, 0.f, 0.f};
+        for (int j0 = 0; j0 < a.top; j0 += 4) {
+            uint2 v[4][NV]; float sc[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int64_t i = t * a.top + min(j0 + j, a.top - 1), pl = a.place[i];
+                sc[j] = a.score[i];
+                const bf16_t *row = pl < 0 ? (const bf16_t *)a.ident + t * a.ldi : (const bf16_t *)a.y + pl * a.ldy;
+#pragma unroll
+                for (int k = 0; k < NV; ++k) if (l + k * NT < W4) v[j][k] = *reinterpret_cast<const uint2 *>(row + (l + k * NT) * 4);
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                if (j0 + j < a.top)
+#pragma unroll
+                    for (int k = 0; k < NV; ++k) if (l + k * NT < W4) { const float4 e = unpack(v[j][k]); yf[k].x += sc[j] * e.x; yf[k].y += sc[j] * e.y; yf[k].z += sc[j] * e.z; yf[k].w += sc[j] * e.w; }
         }
     }
     float mix[S][S], wo[S], wi[S];
 #pragma unroll
     for (int s = 0; s < S; ++s) {
-        wo[s] = a.wout[s]; wi[s] = a.win[s];
+        wo[s] = START ? 1.f : a.wout[s]; wi[s] = sum ? 1.f : a.win[s];
 #pragma unroll
-        for (int q = 0; q < S; ++q) mix[s][q] = a.mix[s * S + q];
+        for (int q = 0; q < S; ++q) mix[s][q] = START ? 0.f : a.mix[s * S + q];
     }
     float4 u[NV]; float sum = 0.f;
 #pragma unroll
@@ -112,13 +145,13 @@ __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
         const int c4 = l + k * NT;
         u[k] = float4{0.f, 0.f, 0.f, 0.f};
         if (c4 < W4) {
-            const float y0 = __uint_as_float(ys[k].x << 16), y1 = __uint_as_float(ys[k].x & 0xffff0000u), y2 = __uint_as_float(ys[k].y << 16), y3 = __uint_as_float(ys[k].y & 0xffff0000u);
+            if (KIND != K_EXPERTS) yf[k] = unpack(ys[k]);
 #pragma unroll
             for (int q = 0; q < S; ++q) {
-                float4 v{wo[q] * y0, wo[q] * y1, wo[q] * y2, wo[q] * y3};
+                float4 v{wo[q] * yf[k].x, wo[q] * yf[k].y, wo[q] * yf[k].z, wo[q] * yf[k].w};
 #pragma unroll
-                for (int s = 0; s < S; ++s) { v.x += mix[s][q] * xs[k][s].x; v.y += mix[s][q] * xs[k][s].y; v.z += mix[s][q] * xs[k][s].z; v.w += mix[s][q] * xs[k][s].w; }
-                *reinterpret_cast<float4 *>(xr + (int64_t)q * W + c4 * 4) = v;
+                for (int s = 0; s < (START ? 0 : S); ++s) { v.x += mix[s][q] * xs[k][s].x; v.y += mix[s][q] * xs[k][s].y; v.z += mix[s][q] * xs[k][s].z; v.w += mix[s][q] * xs[k][s].w; }
+                if (!sum) *reinterpret_cast<float4 *>(xr + (int64_t)q * W + c4 * 4) = v;
                 u[k].x += wi[q] * v.x; u[k].y += wi[q] * v.y; u[k].z += wi[q] * v.z; u[k].w += wi[q] * v.w;
             }
             sum += (u[k].x + u[k].y) + (u[k].z + u[k].w);
@@ -130,7 +163,7 @@ __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
     for (int k = 0; k < NV; ++k)
         if (l + k * NT < W4) { const float a0 = u[k].x - mean, a1 = u[k].y - mean, a2 = u[k].z - mean, a3 = u[k].w - mean; var += (a0 * a0 + a1 * a1) + (a2 * a2 + a3 * a3); }
     const float f = 1.0f / sqrtf((NT == 64 ? wave_sum(var) : block_sum(var, red)) / (float)W + a.eps);
-    bf16_t *o = (bf16_t *)a.out + t * a.ldo;
+    bf16_t *o = (bf16_t *)a.out + r * a.ldo;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
         const int c4 = l + k * NT;
@@ -279,22 +312,22 @@ __global__ __launch_bounds__(256) void qkv_rope8_kernel(QkvRopeArgs a, Batch b) 
 const size_t kMaxLds = 160 * 1024 - 2048;
 bool aligned16(const void *p) { return ((uintptr_t)p & 15) == 0; }
 
-template <int S>
+template <int S, int KIND>
 void step4(const StreamArgs &a, hipStream_t s) {
     const int W4 = a.W / 4;
     // many rows: a wave per row up to 1024 numbers; few rows: a workgroup per row
     if (a.T >= 1024 && W4 <= 256) {
         const dim3 grid((unsigned)((a.T + 3) / 4));
-        if (W4 <= 64) stream_step4_kernel<S, 64, 1><<<grid, dim3(256), 0, s>>>(a);
-        else if (W4 <= 128) stream_step4_kernel<S, 64, 2><<<grid, dim3(256), 0, s>>>(a);
-        else stream_step4_kernel<S, 64, 4><<<grid, dim3(256), 0, s>>>(a);
+        if (W4 <= 64) stream_step4_kernel<S, 64, 1, KIND><<<grid, dim3(256), 0, s>>>(a);
+        else if (W4 <= 128) stream_step4_kernel<S, 64, 2, KIND><<<grid, dim3(256), 0, s>>>(a);
+        else stream_step4_kernel<S, 64, 4, KIND><<<grid, dim3(256), 0, s>>>(a);
         return;
     }
     const dim3 grid((unsigned)a.T);
-    if (W4 <= 256) stream_step4_kernel<S, 256, 1><<<grid, dim3(256), 0, s>>>(a);
-    else if (W4 <= 512) stream_step4_kernel<S, 256, 2><<<grid, dim3(256), 0, s>>>(a);
-    else if (W4 <= 1024) stream_step4_kernel<S, 256, 4><<<grid, dim3(256), 0, s>>>(a);
-    else stream_step4_kernel<S, 256, 8><<<grid, dim3(256), 0, s>>>(a);
+    if (W4 <= 256) stream_step4_kernel<S, 256, 1, KIND><<<grid, dim3(256), 0, s>>>(a);
+    else if (W4 <= 512) stream_step4_kernel<S, 256, 2, KIND><<<grid, dim3(256), 0, s>>>(a);
+    else if (W4 <= 1024) stream_step4_kernel<S, 256, 4, KIND><<<grid, dim3(256), 0, s>>>(a);
+    else stream_step4_kernel<S, 256, 8, KIND><<<grid, dim3(256), 0, s>>>(a);
 }
 
 template <int LP>
@@ -316,10 +349,12 @@ int prepare_streams() {
 int stream_step(const StreamArgs &a, bool bf16, hipStream_t s) {
     if (a.T == 0) return 0;
     const bool start = a.E != nullptr, sum = !start && a.sum;
-    if (a.S < 1 || !a.out || !a.w || (start ? !a.ids || !a.win : !a.y || !a.mix || !a.wout || (!sum && !a.win)) || (a.rows && !sum))
+    if (a.S < 1 || !a.out || !a.w || (start ? !a.ids || !a.win : !a.y || !a.mix || !a.wout || (!sum && !a.win)) || (a.rows && !sum) || (a.place && (start || a.top < 1 || !a.score || !a.ident)))
         return nvr::fail(NVR_ERR_INVALID_ARG, "stream_step: incomplete arguments (%d streams)", a.S);
-    if (bf16 && !start && !sum && a.S <= 4 && a.W % 4 == 0 && a.W <= 8192 && a.ldy % 4 == 0 && a.ldo % 4 == 0 && aligned16(a.x) && aligned16(a.y) && aligned16(a.out) && aligned16(a.w)) {
-        if (a.S == 1) step4<1>(a, s); else if (a.S == 2) step4<2>(a, s); else if (a.S == 3) step4<3>(a, s); else step4<4>(a, s);
+    if (bf16 && a.S <= 4 && a.W % 4 == 0 && a.W <= 8192 && a.ldo % 4 == 0 && aligned16(a.x) && aligned16(a.out) && aligned16(a.w) && (start ? aligned16(a.E) : a.ldy % 4 == 0 && aligned16(a.y)) && (!a.place || (a.ldi % 4 == 0 && aligned16(a.ident)))) {
+#define NVR_ST(S_) do { if (start) step4<S_, K_START>(a, s); else if (a.place) step4<S_, K_EXPERTS>(a, s); else step4<S_, K_STEP>(a, s); } while (0)
+        if (a.S == 1) NVR_ST(1); else if (a.S == 2) NVR_ST(2); else if (a.S == 3) NVR_ST(3); else NVR_ST(4);
+#undef NVR_ST
         return launched("stream_step");
     }
     const size_t lds = ((size_t)a.W + (start ? 0 : (size_t)a.S * 256)) * 4;

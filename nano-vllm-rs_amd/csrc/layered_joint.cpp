@@ -313,9 +313,9 @@ int LayeredModel::forward_joint(nvr_model_runner &r, const StepPlan &p) {
                              true, fs ? 1 : 0, fs ? shared_g : nullptr, rlogits, ne));
             if (blocks) {
                 RC(kl::moe_gather(a2, W, T, W, L.top, place_of, gfloor, e_x, bf16, s));
-                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_x, W, (const uint16_t *)w.egu, 2 * f * W, row_w, nblocks * 256, W, 2 * f, (uint16_t *)e_gu, s));
+                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_x, W, (const uint16_t *)w.egu, 2 * f * W, row_w, nblocks * 256, W, 2 * f, (uint16_t *)e_gu, s, off + L.experts));
                 RC(kl::clamped_glu(e_gu, nblocks * 256, f, (float)L.limit, 1.702f, e_act, f, bf16, s));
-                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_act, f, (const uint16_t *)w.edown, W * f, row_w, nblocks * 256, f, W, (uint16_t *)e_y, s));
+                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_act, f, (const uint16_t *)w.edown, W * f, row_w, nblocks * 256, f, W, (uint16_t *)e_y, s, off + L.experts));
             } else {
                 kl::GroupedLinearArgs g{}; g.a = a2; g.lda = W; g.w = w.egu; g.y = e_gu; g.ldy = 2 * f; g.off = off; g.groups = (int32_t)L.experts; g.K = (int32_t)W; g.N = (int32_t)(2 * f);
                 g.max_rows = (int32_t)n; g.src = order; g.rscale = gfloor; g.src_div = (int32_t)L.top;

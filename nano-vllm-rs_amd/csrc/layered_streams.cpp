@@ -265,8 +265,8 @@ int LayeredModel::forward_streams(nvr_model_runner &r, const StepPlan &p) {
                              true, 0, nullptr, rlogits, ne, w.ecorr, L.identity));
             if (blocks) {
                 RC(kl::moe_gather(a2, W, T, W, L.top, place_of, gfloor, e_x, bf16, s));
-                RC(nvr::kb::gemm256_grouped_silu_mul((const uint16_t *)e_x, W, (const uint16_t *)w.egu, 2 * f * W, row_w, nblocks * 256, W, f, (uint16_t *)e_act, s));
-                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_act, f, (const uint16_t *)w.edown, W * f, row_w, nblocks * 256, f, W, (uint16_t *)e_y, s));
+                RC(nvr::kb::gemm256_grouped_silu_mul((const uint16_t *)e_x, W, (const uint16_t *)w.egu, 2 * f * W, row_w, nblocks * 256, W, f, (uint16_t *)e_act, s, off + L.experts));
+                RC(nvr::kb::gemm256_grouped((const uint16_t *)e_act, f, (const uint16_t *)w.edown, W * f, row_w, nblocks * 256, f, W, (uint16_t *)e_y, s, off + L.experts));
             } else {
                 kl::GroupedLinearArgs gl{}; gl.a = a2; gl.lda = W; gl.w = w.egu; gl.y = e_gu; gl.ldy = 2 * f; gl.off = off; gl.groups = (int32_t)L.experts; gl.K = (int32_t)W; gl.N = (int32_t)(2 * f);
                 gl.max_rows = (int32_t)n; gl.src = order; gl.rscale = gfloor; gl.src_div = (int32_t)L.top;
@@ -275,9 +275,9 @@ int LayeredModel::forward_streams(nvr_model_runner &r, const StepPlan &p) {
                 kl::GroupedLinearArgs d{}; d.a = e_act; d.lda = f; d.w = w.edown; d.y = e_y; d.ldy = W; d.off = off; d.groups = (int32_t)L.experts; d.K = (int32_t)f; d.N = (int32_t)W; d.max_rows = (int32_t)n;
                 RC(kl::grouped_linear(d, bf16, s));
             }
-            RC(kl::moe_combine(e_y, place_of, T, L.top, nullptr, W, tmp, bf16, s, moe_score, nullptr, 1, a2, W));
+            st.place = place_of; st.top = (int32_t)L.top; st.score = moe_score; st.ident = a2; st.ldi = W; st.y = e_y;      // (the choices' rows are summed up where they join the streams)
         }
-        if (L.has_mlp) RC(join(i, 1));
+        if (L.has_mlp) { RC(join(i, 1)); st.place = nullptr; st.y = tmp; }
     }
     return gemm(r, xsel, W, head, R, W, spec.vocab, r.logits, true);
 }

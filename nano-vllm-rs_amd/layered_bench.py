@@ -1,4 +1,4 @@
-"""Prefill and decode throughput of the layer-list designs (Rugudra, Pusunex, Sosutar, Sokalorn) beside the dense Qwen3 graph at equal sizes (bench.py --layered-compare).
+"""Prefill and decode throughput of the layer-list designs (Rugudra, Pusunex, Sosutar, Sokalorn, Negunex) beside the dense Qwen3 graph at equal sizes (bench.py --layered-compare).
 
 Random weights, layer shapes that resemble a real model's; both models go through the same engine (scheduler, block manager, runner step).
 Per size one JSON object: tokens/s of one prefill step over BATCH prompts of PROMPT tokens and of the decode steps that follow, for both."""
@@ -228,6 +228,54 @@ def sokalorn_weights(cfg, seed=0, t_rank=64):
     return out
 
 
+def negunex_config(s, streams=2):
+    """Every layer: attention with the values mixed from the first layer's, the whole head rotated with stretched frequencies.  Feed-forwards in turn: gated GELU of ff, and eight
+    experts of ff / 4 beside four that return their input, four of the twelve per token."""
+    H, G, D, W = s["heads"], s["kv_heads"], s["dim"], s["width"]
+    layers = []
+    for i in range(s["layers"]):
+        mlp = {"kind": "dense", "ff": s["ff"]} if i % 2 == 0 else {"kind": "moe", "expert": {"ff": s["ff"] // 4}, "router": {"experts": 8, "top": 4, "identity": 4}}
+        layers.append({"type": "attention", "mlp": mlp,
+                       "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "v_mix": True,
+                                 "rot": {"dims": D, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}})
+    return {"architecture": "Negunex", "vocab": s["vocab"], "width": W, "streams": streams, "norm": {"eps": 1e-5}, "layers": layers}
+
+
+def negunex_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    W, V, S = cfg["width"], cfg["vocab"], cfg["streams"]
+
+    def lin(o, i, g=1.0):
+        return (rng.standard_normal((o, i), dtype=np.float32) * (g / np.sqrt(i))).astype(np.float32)
+
+    def around(mean, spread, *shape):
+        return (mean + spread * rng.standard_normal(shape)).astype(np.float32)
+    out = {"embed": rng.standard_normal((V, W), dtype=np.float32), "head": lin(V, W), "final.norm": around(1.0, 0.1, W)}
+    for i, L in enumerate(cfg["layers"]):
+        m, p, mlp = L["mixer"], "l%d." % i, L["mlp"]
+        H, G, D, Dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for q in ("1", "2"):
+            out[p + "norm" + q], out[p + "hc%s.in" % q], out[p + "hc%s.out" % q] = around(1.0, 0.1, W), around(1.0 / S, 0.1, S), around(1.0, 0.2, S)
+            out[p + "hc%s.mix" % q] = (np.eye(S) + 0.1 * rng.standard_normal((S, S))).astype(np.float32)
+        for n, o in (("q", H * D), ("k", G * D), ("v", G * Dv)):
+            out[p + "mix." + n], out[p + "mix.%s.b" % n] = lin(o, W), around(0.0, 0.2, o)
+        out[p + "mix.g"], out[p + "mix.o"], out[p + "mix.vmix"] = lin(H * Dv, W), lin(W, H * Dv), np.float32(0.4)
+        if mlp["kind"] == "dense":
+            out[p + "mlp.gate"], out[p + "mlp.up"], out[p + "mlp.down"] = lin(mlp["ff"], W), lin(mlp["ff"], W), lin(W, mlp["ff"])
+        else:
+            E, f = mlp["router"]["experts"], mlp["expert"]["ff"]
+            n = E + mlp["router"]["identity"]
+            out[p + "mlp.router"], out[p + "mlp.correction"] = lin(n, W), around(0.0, 0.05, n)
+            for e in range(E):
+                out[p + "mlp.e%d.gate" % e], out[p + "mlp.e%d.up" % e], out[p + "mlp.e%d.down" % e] = lin(f, W), lin(f, W), lin(W, f)
+    return out
+
+
+LAYERED = {"rugudra": (rugudra_config, random_weights), "pusunex": (pusunex_config, pusunex_weights), "sosutar": (sosutar_config, sosutar_weights),
+           "sokalorn": (sokalorn_config, sokalorn_weights), "negunex": (negunex_config, negunex_weights),
+           "negunex4": (lambda s: negunex_config(s, streams=4), negunex_weights)}      # (four streams instead of two)
+
+
 def _run(nvr, engine, vocab, batch, prompt, steps, warmup):
     sp = nvr.SamplingParams(temperature=0.0, max_tokens=steps + warmup + 1, ignore_eos=True)
     for i in range(batch):
@@ -258,37 +306,15 @@ def compare(nvr, sizes=("w1024", "w2048"), batch=16, prompt=1024, steps=32, warm
         ecfg = dict(max_num_seqs=batch, max_num_batched_tokens=batch * prompt, max_model_len=prompt + steps + warmup + 8, kvcache_block_size=bs,
                     num_kvcache_blocks=batch * ((prompt + steps + warmup + 8 + bs - 1) // bs + 1), dtype=dtype)
         line = {"size": name, "shape": s, "batch": batch, "prompt_len": prompt, "decode_steps": steps, "dtype": dtype}
-        if "rugudra" in which:
-            cfg = rugudra_config(s)
+        for name_m, (config, weights) in LAYERED.items():
+            if name_m not in which:
+                continue
+            cfg = config(s)
             eng = nvr.LLMEngine(nvr.Config(**ecfg), nvr.ModelSpec(cfg))
-            for k, v in random_weights(cfg).items():
+            for k, v in weights(cfg).items():
                 eng.model_runner.load_tensor(k, np.asarray(v))
             _run(nvr, eng, s["vocab"], 2, 64, 2, 1)                       # first launches
-            line["rugudra"] = _run(nvr, eng, s["vocab"], batch, prompt, steps, warmup)
-            del eng
-        if "pusunex" in which:
-            cfg = pusunex_config(s)
-            eng = nvr.LLMEngine(nvr.Config(**ecfg), nvr.ModelSpec(cfg))
-            for k, v in pusunex_weights(cfg).items():
-                eng.model_runner.load_tensor(k, np.asarray(v))
-            _run(nvr, eng, s["vocab"], 2, 64, 2, 1)
-            line["pusunex"] = _run(nvr, eng, s["vocab"], batch, prompt, steps, warmup)
-            del eng
-        if "sosutar" in which:
-            cfg = sosutar_config(s)
-            eng = nvr.LLMEngine(nvr.Config(**ecfg), nvr.ModelSpec(cfg))
-            for k, v in sosutar_weights(cfg).items():
-                eng.model_runner.load_tensor(k, np.asarray(v))
-            _run(nvr, eng, s["vocab"], 2, 64, 2, 1)
-            line["sosutar"] = _run(nvr, eng, s["vocab"], batch, prompt, steps, warmup)
-            del eng
-        if "sokalorn" in which:
-            cfg = sokalorn_config(s)
-            eng = nvr.LLMEngine(nvr.Config(**ecfg), nvr.ModelSpec(cfg))
-            for k, v in sokalorn_weights(cfg).items():
-                eng.model_runner.load_tensor(k, np.asarray(v))
-            _run(nvr, eng, s["vocab"], 2, 64, 2, 1)
-            line["sokalorn"] = _run(nvr, eng, s["vocab"], batch, prompt, steps, warmup)
+            line[name_m] = _run(nvr, eng, s["vocab"], batch, prompt, steps, warmup)
             del eng
         if "qwen3" in which:
             m = nvr.ModelConfig(vocab_size=s["vocab"], hidden_size=s["width"], intermediate_size=s["ff"], num_hidden_layers=s["layers"], num_attention_heads=s["heads"],
