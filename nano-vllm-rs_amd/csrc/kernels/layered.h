@@ -156,7 +156,7 @@ int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool 
 int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 
 // Router of a mixture of experts: logits wr h in f32 (wr: [E][W] f32), the top largest per token -> sel / score (= sigmoid of the logit) [T][top]; then the rows
-// grouped by expert: off [E + 1], order [T top] (place -> token * top + choice), place_of (its inverse).  With pad > 1 every expert's rows start at a multiple of pad
+// grouped by expert: off [E + 1], order [T top] (place -> token * top + choice; not written with pad > 1), place_of (its inverse).  With pad > 1 every expert's rows start at a multiple of pad
 // (places then run up to (T top / pad + E) pad) and row_w[block] names the expert of each of the nblocks blocks of pad rows (and has room for 1024 further numbers behind them): the form a tiled product over whole
 // row blocks wants, with the rows brought together by moe_gather (xs[place] = h[token] * score).
 // softmax: score is the chosen experts' share of the softmax over ALL experts, divided by the sum of the chosen shares (+ 1e-20), instead of the sigmoid.

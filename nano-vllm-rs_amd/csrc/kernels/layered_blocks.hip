@@ -675,7 +675,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restri
     for (int i = threadIdx.x; i < n; i += 1024) {
         if (sel[i] >= E) { place_of[i] = -1; continue; }
         const int place = atomicAdd(&cnt[sel[i]], 1);
-        order[place] = i; place_of[i] = place;
+        place_of[i] = place;
+        if (pad == 1) order[place] = i;                 // (padded places run past the choices; the padded form is read through place_of)
     }
 }
 
@@ -718,7 +719,8 @@ __global__ __launch_bounds__(256) void moe_place_kernel(const int32_t *__restric
     for (int i = i0 + threadIdx.x; i < i1; i += 256) {
         if (sel[i] >= E) { place_of[i] = -1; continue; }
         const int place = atomicAdd(&next[sel[i]], 1);
-        order[place] = i; place_of[i] = place;
+        place_of[i] = place;
+        if (pad == 1) order[place] = i;                 // (padded places run past the choices; the padded form is read through place_of)
     }
 }
 

@@ -98,7 +98,7 @@ __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
     const int64_t r = (int64_t)blockIdx.x * (256 / NT) + threadIdx.x / NT;
     if (NT == 64 && r >= a.T) return;                   // (a whole wave: nobody waits for it)
     const int64_t t = a.rows ? a.rows[r] : r;
-    const bool sum = !START && a.sum;                   // (the end: u is the sum of the new streams, which stay where they were)
+    const bool fin = !START && a.sum;                   // (the end: u is the sum of the new streams, which stay where they were)
     float *xr = a.x + t * S * W;
     const bf16_t *yr = START ? (const bf16_t *)a.E + a.ids[t] * (int64_t)W : (const bf16_t *)a.y + t * a.ldy;      // (the start: every stream is this row)
     float4 xs[NV][START ? 1 : S], yf[NV]; uint2 ys[NV];
@@ -135,7 +135,7 @@ __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
     float mix[S][S], wo[S], wi[S];
 #pragma unroll
     for (int s = 0; s < S; ++s) {
-        wo[s] = START ? 1.f : a.wout[s]; wi[s] = sum ? 1.f : a.win[s];
+        wo[s] = START ? 1.f : a.wout[s]; wi[s] = fin ? 1.f : a.win[s];
 #pragma unroll
         for (int q = 0; q < S; ++q) mix[s][q] = START ? 0.f : a.mix[s * S + q];
     }
@@ -151,7 +151,7 @@ __global__ __launch_bounds__(256) void stream_step4_kernel(StreamArgs a) {
                 float4 v{wo[q] * yf[k].x, wo[q] * yf[k].y, wo[q] * yf[k].z, wo[q] * yf[k].w};
 #pragma unroll
                 for (int s = 0; s < (START ? 0 : S); ++s) { v.x += mix[s][q] * xs[k][s].x; v.y += mix[s][q] * xs[k][s].y; v.z += mix[s][q] * xs[k][s].z; v.w += mix[s][q] * xs[k][s].w; }
-                if (!sum) *reinterpret_cast<float4 *>(xr + (int64_t)q * W + c4 * 4) = v;
+                if (!fin) *reinterpret_cast<float4 *>(xr + (int64_t)q * W + c4 * 4) = v;
                 u[k].x += wi[q] * v.x; u[k].y += wi[q] * v.y; u[k].z += wi[q] * v.z; u[k].w += wi[q] * v.w;
             }
             sum += (u[k].x + u[k].y) + (u[k].z + u[k].w);

@@ -17,8 +17,10 @@ def moe(experts=6, top=2, ff=24, identity=2):
     return {"kind": "moe", "expert": {"ff": ff}, "router": r}
 
 
-def layer(heads=4, kv_heads=2, dim=16, vdim=24, scale=None, rot=16, base=500.0, scaling=(4.0, 1.0, 4.0, 64), v_mix=True, mlp="dense"):
+def layer(heads=4, kv_heads=2, dim=16, vdim=24, scale=None, rot="default", base=500.0, scaling=(4.0, 1.0, 4.0, 64), v_mix=True, mlp="dense"):
     m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale if scale is not None else 1.5 * dim ** -0.5, "v_mix": v_mix}
+    if rot == "default":
+        rot = min(16, dim // 2 * 2)
     if rot is not None:
         m["rot"] = {"dims": rot, "base": base}
         if scaling is not None:
