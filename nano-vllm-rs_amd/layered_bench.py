@@ -230,11 +230,11 @@ def sokalorn_weights(cfg, seed=0, t_rank=64):
 
 def negunex_config(s, streams=2):
     """Every layer: attention with the values mixed from the first layer's, the whole head rotated with stretched frequencies.  Feed-forwards in turn: gated GELU of ff, and eight
-    experts of ff / 4 beside four that return their input, four of the twelve per token."""
+    experts of ff / 4 beside two that return their input, three of the ten per token."""
     H, G, D, W = s["heads"], s["kv_heads"], s["dim"], s["width"]
     layers = []
     for i in range(s["layers"]):
-        mlp = {"kind": "dense", "ff": s["ff"]} if i % 2 == 0 else {"kind": "moe", "expert": {"ff": s["ff"] // 4}, "router": {"experts": 8, "top": 4, "identity": 4}}
+        mlp = {"kind": "dense", "ff": s["ff"]} if i % 2 == 0 else {"kind": "moe", "expert": {"ff": s["ff"] // 4}, "router": {"experts": 8, "top": 3, "identity": 2}}
         layers.append({"type": "attention", "mlp": mlp,
                        "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "v_mix": True,
                                  "rot": {"dims": D, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}})

@@ -47,7 +47,7 @@ MECHANISMS = {
     "heads_of_64_in_groups_of_four": make_config([layer(heads=4, kv_heads=1, dim=64, vdim=64, rot=32), layer(heads=4, kv_heads=1, dim=64, vdim=64)], width=96),
     "heads_of_64_in_groups_of_eight": make_config([layer(heads=8, kv_heads=1, dim=64, vdim=64)], width=64),
     "heads_of_128_ungrouped": make_config([layer(heads=2, kv_heads=2, dim=128, vdim=128, rot=128), layer(heads=2, kv_heads=2, dim=128, vdim=128, rot=96, mlp=None)], width=128),
-    "keys_of_64_values_of_48": make_config([layer(heads=4, kv_heads=2, dim=64, vdim=48, rot=40)], width=96),
+    "keys_of_64_values_of_32": make_config([layer(heads=6, kv_heads=2, dim=64, vdim=32, rot=40)], width=96),
     "keys_of_32_values_of_80": make_config([layer(heads=6, kv_heads=2, dim=32, vdim=80, rot=30)]),
     "keys_of_160_values_of_96": make_config([layer(heads=2, kv_heads=1, dim=160, vdim=96, rot=160), layer(heads=2, kv_heads=1, dim=256, vdim=96, rot=64)]),
     "keys_of_520": make_config([layer(heads=1, kv_heads=1, dim=520, vdim=16, rot=520)]),
@@ -113,10 +113,10 @@ def bf16_ramp(n):
 # ------------------------------------------------------------------------------------------------ a model with everything, in portions and batches
 def everything(vocab=113, width=96, streams=3):
     return make_config([layer(heads=4, kv_heads=2, dim=32, vdim=32, rot=16, v_mix=False, mlp="dense"),
-                        layer(heads=6, kv_heads=1, dim=16, vdim=48, mlp=moe(experts=5, top=3, ff=40, identity=2)),
-                        layer(heads=3, kv_heads=1, dim=24, vdim=48, rot=24, mlp=None),
-                        layer(heads=4, kv_heads=1, dim=64, vdim=48, base=9000.0, scaling=(8.0, 1.0, 3.0, 100), mlp=moe(experts=3, top=1, ff=56, identity=1)),
-                        layer(heads=2, kv_heads=1, dim=64, vdim=48, rot=None, scale=0.2, mlp=dense(72))],
+                        layer(heads=6, kv_heads=1, dim=16, vdim=80, mlp=moe(experts=5, top=3, ff=40, identity=2)),
+                        layer(heads=3, kv_heads=1, dim=24, vdim=80, rot=24, mlp=None),
+                        layer(heads=5, kv_heads=1, dim=64, vdim=80, base=9000.0, scaling=(8.0, 1.0, 3.0, 100), mlp=moe(experts=3, top=1, ff=56, identity=1)),
+                        layer(heads=2, kv_heads=1, dim=64, vdim=80, rot=None, scale=0.2, mlp=dense(72))],
                        vocab=vocab, width=width, streams=streams)
 
 
@@ -202,7 +202,7 @@ PROBE_LAYERS = {
     "small_heads": (dict(heads=4, kv_heads=2, dim=16, vdim=16, rot=8), 48),
     "heads_of_64": (dict(heads=4, kv_heads=2, dim=64, vdim=64, rot=32), 96),
     "heads_of_128": (dict(heads=2, kv_heads=2, dim=128, vdim=128, rot=64), 96),
-    "keys_of_64_values_of_48": (dict(heads=4, kv_heads=1, dim=64, vdim=48, rot=4), 64),
+    "keys_of_64_values_of_80": (dict(heads=3, kv_heads=1, dim=64, vdim=80, rot=4), 64),
 }
 
 
