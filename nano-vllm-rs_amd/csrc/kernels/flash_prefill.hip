@@ -43,8 +43,9 @@ struct FlashParams {
     float *part_o, *part_ml;
     const int32_t *srows, *scount;     // optional: only the rows srows[0 .. *scount) of the batch share the prefix (row srows[0] names its blocks)
     const float *r1, *r2, *sink; int64_t ldo;   // PEN instantiations: distance penalty and sink per head (FlashArgs); ldo: output row stride in elements
-    int32_t window;                              // PEN instantiations: > 0, a query sees only the keys less than `window` positions back
+    int32_t window, keep_first;                  // PEN and DIFF instantiations: > 0, a query sees only the keys less than `window` positions back (and the first keep_first keys)
     const float *gate_bias; float softcap; int32_t chunk;   // GATE instantiations (FlashArgs): sigmoid weights with a bias per head, capped scores, chunks of positions
+    const float *lambda; float out_scale, eps; const half_t *head_gate; int64_t ldhg;   // DIFF instantiations (FlashArgs)
 };
 
 
@@ -126,7 +127,10 @@ constexpr int FLASH_WAVES = NVR_FLASH_WAVES;     // waves per workgroup: 32 quer
 // by attn_merge_kernel.
 // GATE: no softmax — a visible key's weight is sigmoid(cap tanh(score / cap) + bias of the head), not normalised; a query sees the keys of its own chunk of
 // p.chunk positions (chunks count from position 0) up to itself; the steps start at the chunk of the tile's first query.
-template <int D, int G, bool PAGED, bool UB = false, bool SHARED = false, bool PEN = false, bool GATE = false>
+// DIFF: differential attention.  A wave's two query tiles are the two maps of ONE head at the same 16 positions: map t multiplies its half of the K fragments, both use
+// every V fragment, and the difference, its norm and the gate are formed from the accumulators (the maps' outputs of a query sit in the same lanes).
+// A window with kept first keys (PEN, DIFF): the steps over the kept keys come first, then those from the window's first key on.
+template <int D, int G, bool PAGED, bool UB = false, bool SHARED = false, bool PEN = false, bool GATE = false, bool DIFF = false>
 __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefill_kernel(FlashParams p) {   // 2 waves per SIMD: <= 256 registers per lane
     constexpr int NT = 64 * FLASH_WAVES;         // threads
     constexpr int KT = NVR_FLASH_KT;             // keys per step
@@ -150,17 +154,21 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
     const int r = lane & 15, g4 = lane >> 4;
     // SHARED: blockIdx.y cuts the shared keys into partitions of shared_len tokens (more workgroups than 8 per kv head at 512 sequences)
     // (a window: the first step is the one that holds the first key the tile's first query sees)
-    const int kv_start = SHARED ? (int)blockIdx.y * p.shared_len : ((PEN && p.window > 0) ? max(tile.pos0 - p.window + 1, 0) / KT * KT :
+    const int kv_start = SHARED ? (int)blockIdx.y * p.shared_len : (((PEN || DIFF) && p.window > 0) ? max(tile.pos0 - p.window + 1, 0) / KT * KT :
                                                                     (GATE && p.chunk > 0) ? tile.pos0 / p.chunk * p.chunk / KT * KT : 0);
     const int kv_end = SHARED ? kv_start + p.shared_len : tile.pos0 + tile.nq;
+    const int nkept = ((PEN || DIFF) && p.window > 0) ? min((p.keep_first + KT - 1) / KT, kv_start / KT) : 0;      // steps over the kept first keys
+    auto first_key = [&](int it) { return ((PEN || DIFF) && it < nkept) ? it * KT : kv_start + (it - nkept) * KT; };
 
     // the wave's two query tiles: head and position block
     int qi[NQT], head[NQT], qpos[NQT], qrow[NQT]; bool qvalid[NQT];
-    half8_t qf[NQT][NKS];
+    constexpr int NQS = DIFF ? NKS / 2 : NKS;    // query fragments per tile
+    half8_t qf[NQT][NQS];
 #pragma unroll
     for (int t = 0; t < NQT; ++t) {
         int pblk;
-        if (G == 1) { head[t] = g; pblk = wave * 2 + t; }
+        if (DIFF) { head[t] = g * G + (G == 1 ? 0 : G == 2 ? (wave & 1) : wave); pblk = G == 1 ? wave : G == 2 ? (wave >> 1) : 0; }
+        else if (G == 1) { head[t] = g; pblk = wave * 2 + t; }
         else if (G == 2) { head[t] = g * 2 + t; pblk = wave; }
         else { head[t] = g * 4 + (wave & 1) * 2 + t; pblk = wave >> 1; }
         qi[t] = pblk * 16 + r;
@@ -168,14 +176,14 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
         const int qc = qvalid[t] ? qi[t] : tile.nq - 1;
         qpos[t] = SHARED ? 0x3fffffff : tile.pos0 + qc;           // absolute position = last visible key
         qrow[t] = (SHARED && p.srows) ? p.srows[tile.q_row0 + qc] : tile.q_row0 + qc;
-        const half_t *qptr = p.q + (int64_t)qrow[t] * p.ldq + (int64_t)head[t] * D + g4 * 8;
+        const half_t *qptr = p.q + (int64_t)qrow[t] * p.ldq + (int64_t)head[t] * D + (DIFF ? t * (D / 2) : 0) + g4 * 8;
 #pragma unroll
-        for (int ks = 0; ks < NKS; ++ks) qf[t][ks] = *reinterpret_cast<const half8_t *>(qptr + ks * 32);
+        for (int ks = 0; ks < NQS; ++ks) qf[t][ks] = *reinterpret_cast<const half8_t *>(qptr + ks * 32);
     }
 
     // last key any lane of this wave may attend to: a step that starts beyond it does no arithmetic in this wave
     const int wave_last = SHARED ? kv_end - 1
-        : __builtin_amdgcn_readfirstlane(tile.pos0 + min(tile.nq - 1, (G == 1 ? wave * 2 + 1 : (G == 2 ? wave : (wave >> 1))) * 16 + 15));
+        : __builtin_amdgcn_readfirstlane(tile.pos0 + min(tile.nq - 1, (DIFF ? (G == 1 ? wave : G == 2 ? (wave >> 1) : 0) : G == 1 ? wave * 2 + 1 : (G == 2 ? wave : (wave >> 1))) * 16 + 15));
     int bt_reg = 0, bt_chunk = -1;                                    // UB: register copy of 64 block-table entries
     // The chunk is fetched by an inline-asm load that waits for itself: a compiler-visible load inside the step loop (the reload of a
     // context longer than 64 blocks) makes hipcc put s_waitcnt vmcnt(0) in front of EVERY v_readlane of bt_reg, i.e. into every step —
@@ -212,7 +220,7 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
 #pragma unroll
     for (int t = 0; t < NQT; ++t)
 #pragma unroll
-        for (int ks = 0; ks < NKS; ++ks) asm volatile("" :: "v"(qf[t][ks]));
+        for (int ks = 0; ks < NQS; ++ks) asm volatile("" :: "v"(qf[t][ks]));
     auto stage = [&](int buf, int kt) {
         const half_t *src[2 * PIECES];
         const bool whole = kt + KT <= kv_end;                             // uniform: no key of this step is clamped
@@ -278,6 +286,8 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
     for (int t = 0; t < NQT; ++t) {
         pr1[t] = (PEN && p.r1) ? p.r1[head[t]] * (lin ? 1.44269504088896340736f : 1.0f) : 0.f; pr2[t] = (PEN && p.r2) ? p.r2[head[t]] : 0.f;
         if (PEN && p.sink) { m[t] = p.sink[head[t]] * 1.44269504088896340736f; ol[t] = (float4_t){1.f, 1.f, 1.f, 1.f}; }
+        else if (!GATE && !DIFF && p.sink) { m[t] = p.sink[head[t]] / p.scale; ol[t] = (float4_t){1.f, 1.f, 1.f, 1.f}; }      // (raw scores: the sink in their unit)
+        if (DIFF) m[t] = -1e30f;                                // (a step of a window may hold no visible key of a query: a finite maximum keeps the differences finite)
     }
     half8_t ones;
 #pragma unroll
@@ -287,15 +297,15 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
     for (int t = 0; t < NQT; ++t) { gbias[t] = GATE ? p.gate_bias[head[t]] : 0.f; qcs[t] = (GATE && p.chunk > 0) ? qpos[t] / p.chunk * p.chunk : 0; }
     if (GATE && p.softcap > 0.f) gcap2 = 2.0f * 1.44269504088896340736f / p.softcap;
 
-    const int nsteps = (kv_end - kv_start + KT - 1) / KT;
+    const int nsteps = nkept + (kv_end - kv_start + KT - 1) / KT;
     // step `it` computes on ring slot it % NBUF while tile it+NBUF-1 is requested into the slot step it-1 just released;
     // before its closing barrier every wave waits until only the loads of tiles it+2.. are outstanding, so tile it+1 has
     // landed for all waves after the barrier and the global loads never drain inside the stream.
     auto step = [&](auto cur_c, int it) {
         constexpr int cur = decltype(cur_c)::value;
-        const int kt = kv_start + it * KT;
+        const int kt = first_key(it);
         const bool more = it + NBUF - 1 < nsteps;
-        if (more) stage((cur + NBUF - 1) % NBUF, kt + (NBUF - 1) * KT);
+        if (more) stage((cur + NBUF - 1) % NBUF, first_key(it + NBUF - 1));
         const char *kl = smem + cur * STAGE, *vl = kl + KT * D * 2;
         if (kt <= wave_last) {
 
@@ -318,9 +328,9 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
 #pragma unroll
             for (int t = 0; t < NQT; ++t) s[t][mt] = (float4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int ks = 0; ks < NKS; ++ks)
+            for (int ks = 0; ks < NQS; ++ks)
 #pragma unroll
-                for (int t = 0; t < NQT; ++t) s[t][mt] = mfma16(kf[mt & 1][ks], qf[t][ks], s[t][mt]);
+                for (int t = 0; t < NQT; ++t) s[t][mt] = mfma16(kf[mt & 1][(DIFF ? t * NQS : 0) + ks], qf[t][ks], s[t][mt]);
             __builtin_amdgcn_sched_barrier(0);
         }
         half8_t pf[NQT][NK2];
@@ -348,7 +358,19 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
                         const int di = max(qpos[t] - (kt + mt * 16 + g4 * 4 + e), 0);
                         const float dist = (float)di;
                         const float v = fmaf(s[t][mt][e], c2, lin ? -pr1[t] * dist : -pr1[t] * __builtin_amdgcn_logf(fmaf(pr2[t], dist, 1.0f)));
-                        s[t][mt][e] = (p.window > 0 && di >= p.window) ? -INFINITY : v;
+                        s[t][mt][e] = (p.window > 0 && di >= p.window && kt + mt * 16 + g4 * 4 + e >= p.keep_first) ? -INFINITY : v;
+                    }
+        }
+        // DIFF: the window's far edge only on steps that hold a key out of some query's window
+        if (DIFF && p.window > 0 && tile.pos0 + tile.nq - 1 - kt >= p.window && kt + KT > p.keep_first) {
+#pragma unroll
+            for (int t = 0; t < NQT; ++t)
+#pragma unroll
+                for (int mt = 0; mt < NMT; ++mt)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        const int j = kt + mt * 16 + g4 * 4 + e;
+                        if (qpos[t] - j >= p.window && j >= p.keep_first) s[t][mt][e] = -INFINITY;
                     }
         }
         // causal mask only on steps that reach past the tile's first query (keys kt + mt*16 + g4*4 + e)
@@ -422,7 +444,7 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
 
 #pragma unroll
     for (int b = 0; b < NBUF - 1; ++b)
-        if (b < nsteps) stage(b, kv_start + b * KT);
+        if (b < nsteps) stage(b, first_key(b));
     if (NBUF - 1 < nsteps) {
         if (NBUF == 2) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         else if (NBUF == 3) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(1 * 2 * PIECES) : "memory");
@@ -450,6 +472,26 @@ __global__ __launch_bounds__(64 * FLASH_WAVES, 8 / FLASH_WAVES) void flash_prefi
         }
         return;
     }
+    if (DIFF) {                                                 // (both tiles: one head, one query per lane; a query's value numbers are spread over its four lanes)
+        const float i0 = 1.0f / ol[0][0], i1 = *p.lambda / ol[1][0];
+        float ss = 0.f;
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { const float d = o[0][dt][e] * i0 - o[1][dt][e] * i1; o[0][dt][e] = d; ss += d * d; }
+        ss += __shfl_xor(ss, 16, 64); ss += __shfl_xor(ss, 32, 64);
+        if (qvalid[0]) {
+            float f = p.out_scale / sqrtf(ss / (float)D + p.eps);
+            if (p.head_gate) f /= 1.0f + __expf(-(float)p.head_gate[(int64_t)qrow[0] * p.ldhg + head[0]]);
+            half_t *orow = p.out + (int64_t)qrow[0] * p.ldo + (int64_t)head[0] * D + g4 * 4;
+#pragma unroll
+            for (int dt = 0; dt < NDT; ++dt) {
+                half4_t hv = {(half_t)(o[0][dt][0] * f), (half_t)(o[0][dt][1] * f), (half_t)(o[0][dt][2] * f), (half_t)(o[0][dt][3] * f)};
+                *reinterpret_cast<half4_t *>(orow + dt * 16) = hv;
+            }
+        }
+        return;
+    }
 #pragma unroll
     for (int t = 0; t < NQT; ++t) {
         if (qvalid[t]) {
@@ -471,6 +513,8 @@ bool flash_prefill_ok(int D, int H, int KVH) {
     return (D == 64 || D == 128) && (G == 1 || G == 2 || G == 4);
 }
 int flash_tile_positions(int H, int KVH) { return 32 * FLASH_WAVES / (H / KVH); }
+bool flash_diff_ok(int D, int H, int KVH) { return FLASH_WAVES == 4 && flash_prefill_ok(D, H, KVH); }
+int flash_diff_tile_positions(int H, int KVH) { return 16 * FLASH_WAVES / (H / KVH); }
 
 int flash_prefill(const FlashArgs &a, bool paged, hipStream_t s) {
     if (a.ntiles == 0) return 0;
@@ -480,19 +524,26 @@ int flash_prefill(const FlashArgs &a, bool paged, hipStream_t s) {
     p.block_tables = a.block_tables; p.max_blocks = a.max_blocks; p.block_size = a.block_size;
     p.bs_shift = (a.block_size > 0 && (a.block_size & (a.block_size - 1)) == 0) ? __builtin_ctz(a.block_size) : -1;
     p.tiles = a.tiles; p.H = a.H; p.KVH = a.KVH; p.scale = a.scale; p.out = (half_t *)a.out;
-    p.r1 = a.r1; p.r2 = a.r2; p.sink = a.sink; p.ldo = a.ldo ? a.ldo : (int64_t)a.H * a.D; p.window = a.window;
+    p.r1 = a.r1; p.r2 = a.r2; p.sink = a.sink; p.ldo = a.ldo ? a.ldo : (int64_t)a.H * a.D; p.window = a.window; p.keep_first = a.keep_first;
+    p.lambda = a.lambda; p.out_scale = a.out_scale; p.eps = a.eps; p.head_gate = (const half_t *)a.head_gate; p.ldhg = a.ldhg;
     p.gate_bias = a.gate_bias; p.softcap = a.softcap; p.chunk = a.chunk;
     const bool gate = a.gate_bias != nullptr;
     if (gate && (a.r1 || a.sink || a.window > 0 || !paged)) return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: gated weights take no penalty, sink or window and read K and V through block tables");
-    const bool pen = a.r1 || a.sink;
-    if (a.window > 0 && !a.sink) return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: a window needs the sink form (a step may hold no visible key)");
+    const bool diff = a.lambda != nullptr;
+    if (diff && (gate || a.r1 || a.sink || !paged || !flash_diff_ok(a.D, a.H, a.KVH)))
+        return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: differential attention takes no penalty, sink or gated weights and reads K and V through block tables");
+    const bool pen = a.r1 || (a.sink && a.window > 0);         // (a sink alone costs nothing in the plain form)
+    if (a.window > 0 && !a.sink && !diff) return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: a window needs the sink form (a step may hold no visible key)");
+    if (a.sink && !pen && !(a.scale > 0.f)) return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: a sink needs a positive scale");
     if (pen && !paged) return nvr::fail(NVR_ERR_UNSUPPORTED, "flash_prefill: the penalty / sink form reads K and V through block tables");
     const int G = a.H / a.KVH;
     dim3 grid((unsigned)((int64_t)a.ntiles * a.KVH)), block(64 * FLASH_WAVES);
     const bool ub = paged && p.bs_shift >= 0 && a.block_size % NVR_FLASH_KT == 0;
 #define NVR_FLASH(DD, GG)                                                                             \
     if (a.D == DD && G == GG) {                                                                       \
-        if (gate && ub) flash_prefill_kernel<DD, GG, true, true, false, false, true><<<grid, block, 0, s>>>(p);   \
+        if (diff && ub) flash_prefill_kernel<DD, GG, true, true, false, false, false, true><<<grid, block, 0, s>>>(p);   \
+        else if (diff) flash_prefill_kernel<DD, GG, true, false, false, false, false, true><<<grid, block, 0, s>>>(p);   \
+        else if (gate && ub) flash_prefill_kernel<DD, GG, true, true, false, false, true><<<grid, block, 0, s>>>(p);   \
         else if (gate) flash_prefill_kernel<DD, GG, true, false, false, false, true><<<grid, block, 0, s>>>(p);   \
         else if (pen && ub) flash_prefill_kernel<DD, GG, true, true, false, true><<<grid, block, 0, s>>>(p);   \
         else if (pen) flash_prefill_kernel<DD, GG, true, false, false, true><<<grid, block, 0, s>>>(p);   \

@@ -112,6 +112,7 @@ bool gemm256_silu_ok(int64_t T, int64_t K, int64_t I, int64_t ldx);
 bool gemm256_rope_ok(int64_t T, int64_t K, int64_t H, int64_t KVH, int64_t D, int64_t ldx);
 int gemm256(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s);
 int gemm256_relu2(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s);   // y = max(x . W^T, 0)^2
+int gemm256_gelu(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s);    // y = gelu(x . W^T), error function
 int gemm256_grouped(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s, const int32_t *rows_used = nullptr);
 int gemm256_grouped_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t w_stride, const int32_t *row_w, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s, const int32_t *rows_used = nullptr);
 int gemm256_resid(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *h, hipStream_t s);
@@ -131,6 +132,9 @@ int attention(const AttnArgs &a, bool paged, hipStream_t s);
 
 bool flash_prefill_ok(int D, int H, int KVH);
 int flash_tile_positions(int H, int KVH);
+// differential attention (FlashArgs::lambda): D is the size of a key row with both maps, also the value size
+bool flash_diff_ok(int D, int H, int KVH);
+int flash_diff_tile_positions(int H, int KVH);
 int flash_prefill(const FlashArgs &a, bool paged, hipStream_t s);
 int flash_shared_prefix(const half_bits *q, int64_t ldq, const half_bits *k_cache, const half_bits *v_cache, const int32_t *block_tables,
                         int32_t max_blocks, int32_t block_size, int32_t nq, int32_t H, int32_t KVH, int32_t D, float scale,

@@ -61,12 +61,18 @@ struct FlashArgs {
     // Optional (all zero: plain softmax attention).  A distance penalty and a sink per head: score = q.k * scale - r1[h] * ln(1 + r2[h] * (i - j)), and the
     // softmax denominator also holds exp(sink[h]) (a term with no key and no value).  r1 / r2 together, sink on its own, each [H] f32 on the device.
     // ldo: elements between the output rows of consecutive query rows (0: H * D)
-    // r1 without r2: a penalty linear in the distance, r1[h] * (i - j).  window > 0 (with a sink): a query sees only the keys less than `window` positions back.
+    // r1 without r2: a penalty linear in the distance, r1[h] * (i - j).  window > 0 (with r1 and a sink): a query sees only the keys less than `window` positions back.
     const float *r1, *r2, *sink; int64_t ldo;
     int32_t window;
     // gate_bias ([H] f32 on the device; paged K / V; no penalty, sink or window): no softmax — a visible key's weight is sigmoid(score + gate_bias[h]) with the scaled
     // score first capped, softcap * tanh(score / softcap) (softcap 0: not); chunk > 0: a query sees the keys j <= i with floor(j / chunk) == floor(i / chunk)
     const float *gate_bias; float softcap; int32_t chunk;
+    // with a window: the keys j < keep_first stay visible whatever their distance
+    int32_t keep_first;
+    // lambda (one f32 number on the device; paged K / V; no penalty, sink or gate_bias, window optional) not null: differential attention.  A key row holds the keys of two maps side by
+    // side (D / 2 numbers each), a query head the queries of both; each map is a softmax attention over the same values, and out = f (a1 - lambda a2) / sqrt(mean^2 + eps) over the
+    // head's D value numbers with f = out_scale * sigmoid(head_gate[row * ldhg + head]) (head_gate rows of the operand type; null: no gate)
+    const float *lambda; float out_scale, eps; const half_bits *head_gate; int64_t ldhg;
 };
 
 // Config.dtype = "float32": attention arguments of the f32 path (kernels/f32_path.hip)

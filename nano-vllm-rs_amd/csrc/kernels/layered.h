@@ -57,10 +57,15 @@ struct SinkAttnArgs {
     float softcap;                           // > 0: score <- softcap * tanh(score / softcap) (after the scale, before any bias)
     const float *gate_bias;                  // not null: no softmax — the weight of a visible key is sigmoid(score + gate_bias[h]), not normalised over the keys
                                              // (both forms; not together with a penalty or a sink)
+    int32_t keep_first;                      // with a window: the keys j < keep_first stay visible whatever their distance (the tiled form: not together with a penalty table)
+    // lambda (one number) not null: differential attention.  A key row holds the keys of two maps side by side (D / 2 numbers each), a query head the queries of both; each map is a
+    // softmax attention of its own over the same values, and out = f (a1 - lambda a2) / sqrt(mean^2 + eps) over the head's Dv numbers, f = out_scale * sigmoid(head_gate[t * ldhg + h])
+    // (head_gate rows of the operand type; null: no gate).  General form: the maps' outputs pass through maps_o ([T][H][2][Dv] f32).  Not together with penalties, sinks or gate_bias
+    const float *lambda; float out_scale, eps; const void *head_gate; int64_t ldhg; float *maps_o;
 };
 int sink_attention(const SinkAttnArgs &a, const Batch &b, bool bf16, hipStream_t s);     // any shape; a context that fits the LDS score buffer
-// The same on the matrix cores (bf16 operands, D % 32 == 0, Dv % 16 == 0, both <= 256, H / G <= 16).  tiles (device, built by the host): tile i covers the
-// rows row0 .. row0 + 64 / (H / G) - 1 of sequence seq's chunk, for all H / G query heads of a key/value head.  nsplit > 1 spreads a tile's keys over that many
+// The same on the matrix cores (bf16 operands, D and Dv multiples of 8 up to 256, at most 16 query heads per key/value head — a head of differential attention counts twice).  tiles
+// (device, built by the host): tile i covers the rows row0 .. row0 + 64 / g - 1 of sequence seq's chunk, for all g query heads of a key/value head.  nsplit > 1 spreads a tile's keys over that many
 // workgroups (decode-sized steps over long contexts) and merges their partials; workspace: sink_attention_workspace_bytes(ntiles * G * nsplit).
 struct AttnTile { int32_t seq, row0; };
 bool sink_attention_tiled_ok(const SinkAttnArgs &a, bool bf16, int block_size);   // (pages of a multiple of 8 tokens)
@@ -129,15 +134,15 @@ struct GroupNormArgs {
 int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s);
 
 // Latent attention caches ONE row per token: `rank` numbers of the latent (proj columns col ..., divided by their root mean square, times w) and `rot` numbers of a
-// key part shared by the heads, rotated in pairs (2i, 2i+1) by position * freq[i].  pages: [blocks][block_size][rank + rot] of the operand type; rows (may be null):
-// the same rows in step order, [T][rank + rot].
+// key part shared by the heads, rotated in pairs (2i, 2i+1), or (i, i + rot / 2) with halves, by position * freq[i] (cosines and sines times gain).  pages:
+// [blocks][block_size][rank + rot] of the operand type; rows (may be null): the same rows in step order, [T][rank + rot].
 int latent_store(const void *proj, int64_t ld, int64_t col, const Batch &b, int64_t rank, int64_t rot, float eps, const float *w, const float *freq, void *pages, void *rows,
-                 bool bf16, hipStream_t s);
+                 bool bf16, hipStream_t s, bool halves = false, float gain = 1.f);
 // y[t][c] *= sigmoid(g[t][c]) (c < N; rows of y / g with strides ldy / ldg)
 int sigmoid_gate(void *y, int64_t ldy, const void *g, int64_t ldg, int64_t T, int64_t N, bool bf16, hipStream_t s);
-// The rotated part of the queries: q[t][h * qstride + qcol ...] (rot numbers, pairs (2i, 2i+1)) -> out[t][h * ostride + ocol ...]
+// The rotated part of the queries: q[t][h * qstride + qcol ...] (rot numbers, pairs as in latent_store) -> out[t][h * ostride + ocol ...]
 int rotate_heads(const void *q, int64_t ldq, int64_t qstride, int64_t qcol, const Batch &b, int64_t H, int64_t rot, const float *freq, void *out, int64_t ldo, int64_t ostride,
-                 int64_t ocol, bool bf16, hipStream_t s);
+                 int64_t ocol, bool bf16, hipStream_t s, bool halves = false, float gain = 1.f);
 
 // y[t][h * hy + n] = sum_k a[t][h * ha + k] * w[h][n][k] (n < N, k < K; rows of a / y / gate with strides lda / ldy / ldg), times sigmoid(gate[t][h * hg + n]) when gate is not null.
 // One matrix per head: the key expansion folded into the queries (w[h] = Wuk_h^T), the value expansion of the attended latent (w[h] = Wuv_h).
@@ -154,6 +159,8 @@ int poly_norm(const void *z, int64_t ldz, int64_t T, int64_t F, float eps, const
 // out = silu(gate) * up, or gelu(gate) * up (the tanh form); gu: rows [2 F] (gate columns, then up columns)
 int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
+// out = gelu(z), the form with the error function (rows of F numbers, strides ldz / ldo)
+int gelu_erf(const void *z, int64_t ldz, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 
 // Router of a mixture of experts: logits wr h in f32 (wr: [E][W] f32), the top largest per token -> sel / score (= sigmoid of the logit) [T][top]; then the rows
 // grouped by expert: off [E + 1], order [T top] (place -> token * top + choice; not written with pad > 1), place_of (its inverse).  With pad > 1 every expert's rows start at a multiple of pad
@@ -290,8 +297,9 @@ struct StreamArgs {
 };
 int stream_step(const StreamArgs &a, bool bf16, hipStream_t s);
 
-// Queries, keys and values on their way from the projections to an attention over pages.  In row t of proj: q += bq, k += bk, v += bv (each may be null); the first `rot` numbers of
-// every q / k head turned by position * freq[i] — pairs: numbers (2i, 2i + 1), else (i, i + rot / 2) —; unit: every q / k head divided by sqrt(mean^2 + eps) behind the rotation;
+// Queries, keys and values on their way from the projections to an attention over pages.  In row t of proj: q += bq, k += bk, v += bv (each may be null); with wq / wk ([D] f32,
+// shared by the heads) every q / k head divided by sqrt(mean^2 + eps), times the weight; the first `rot` numbers of every q / k head turned by position * freq[i] — pairs: numbers
+// (2i, 2i + 1), else (i, i + rot / 2); cosines and sines times gain (0: 1) —; Gv: value heads (0: G; other numbers where keys of several maps belong to one value head); unit: every q / k head divided by sqrt(mean^2 + eps) behind the rotation;
 // q stays in proj, k -> the K page row of the position.  v_keep (may be null): this step's values as they are now, [T][G Dv]; v_first (may be null): v <- (1 - lambda) v + lambda v_first
 // with rows like v_keep's; v -> the V page row (layouts as kv_store).
 struct QkvRopeArgs {
@@ -299,6 +307,7 @@ struct QkvRopeArgs {
     const float *bq, *bk, *bv; bool unit; float eps;
     void *v_keep; const void *v_first; const float *lambda;
     void *kc, *vc; bool v_grouped;
+    const float *wq, *wk; float gain; int32_t Gv;
 };
 int qkv_rope_store(const QkvRopeArgs &a, const Batch &b, bool bf16, hipStream_t s);
 

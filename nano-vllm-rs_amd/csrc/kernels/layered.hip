@@ -216,31 +216,34 @@ __global__ __launch_bounds__(256) void sink_attn_rows_kernel(SinkAttnArgs a, Bat
     __shared__ float red[4];
     const int t = blockIdx.x, h = blockIdx.y, sq = b.row_seq[t];
     const int i = b.start[sq] + (t - b.cu[sq]), ctx = i + 1;
-    const int kvh = h / (a.H / a.G);
+    // (differential attention: blockIdx.y counts the maps of all heads; map h & 1 has its keys in that half of the key row)
+    const int maps = a.lambda ? 2 : 1, Dq = a.D / maps, kvh = h / (a.H * maps / a.G);
     float *qs = sm, *sc = sm + a.D;
-    const CT *q = (const CT *)a.q + (int64_t)t * a.ldq + (int64_t)h * a.D;
-    for (int d = threadIdx.x; d < a.D; d += 256) qs[d] = ld_f(q, d);
+    const CT *q = (const CT *)a.q + (int64_t)t * a.ldq + (int64_t)h * Dq;
+    for (int d = threadIdx.x; d < Dq; d += 256) qs[d] = ld_f(q, d);
     __syncthreads();
     const CT *kc = (const CT *)a.kc; const CT *vc = (const CT *)a.vc;
     const int32_t *bt = b.block_tables + (int64_t)sq * b.max_blocks;
     const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r2 ? a.r2[h] : 0.f, slope = a.slope ? a.slope[h] : 0.f;
-    int j0 = a.window > 0 ? max(0, ctx - a.window) : 0;            // first visible key; the score buffer holds the keys j0 .. ctx - 1
+    int j0 = a.window > 0 ? max(0, ctx - a.window) : 0;            // first visible key
     if (a.chunk > 0) j0 = max(j0, i / a.chunk * a.chunk);          // (chunks count from position 0 of the sequence)
+    const int kept = (a.window > 0 && a.keep_first > 0) ? min(a.keep_first, j0) : 0;
+    const int nk = kept + ctx - j0, skip = j0 - kept;              // the score buffer holds the kept first keys, then the keys j0 .. ctx - 1: slot x is key x, or x + skip behind the kept ones
     const bool gate = a.gate_bias != nullptr;                      // weights sigmoid(score + bias), not normalised
     const float gb = gate ? a.gate_bias[h] : 0.f;
-    sc -= j0;
     float mx = a.sink ? a.sink[h] : -INFINITY;
-    for (int j = j0 + threadIdx.x; j < ctx; j += 256) {
+    for (int x = threadIdx.x; x < nk; x += 256) {
+        const int j = x < kept ? x : x + skip;
         const int64_t row = (int64_t)bt[j / b.block_size] * b.block_size + j % b.block_size;
-        const int64_t base = (row * a.G + kvh) * a.D;
+        const int64_t base = (row * a.G + kvh) * a.D + (maps == 2 ? (h & 1) * Dq : 0);
         float dot = 0.f;
-        for (int d = 0; d < a.D; ++d) dot += qs[d] * ld_f(kc, base + d);
+        for (int d = 0; d < Dq; ++d) dot += qs[d] * ld_f(kc, base + d);
         float s = dot * a.scale;
         if (a.r1) s -= r1 * log1pf(r2 * (float)(i - j));
         if (a.slope) s -= slope * (float)(i - j);
         if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
         if (gate) s = 1.0f / (1.0f + expf(-(s + gb)));
-        sc[j] = s;
+        sc[x] = s;
         mx = fmaxf(mx, s);
     }
     float inv = 1.0f;
@@ -248,30 +251,47 @@ __global__ __launch_bounds__(256) void sink_attn_rows_kernel(SinkAttnArgs a, Bat
     else {
     mx = block_max<256>(mx, red);
     float sum = 0.f;
-    for (int j = j0 + threadIdx.x; j < ctx; j += 256) { const float e = expf(sc[j] - mx); sc[j] = e; sum += e; }
+    for (int x = threadIdx.x; x < nk; x += 256) { const float e = expf(sc[x] - mx); sc[x] = e; sum += e; }
     sum = block_sum<256>(sum, red);                     // (its barriers also publish the weights)
     if (a.sink) sum += expf(a.sink[h] - mx);
     inv = 1.0f / sum;
     }
     // values: column c by lanes, keys split over the 256 / CW groups
-    float *part = sc + ctx;                             // (behind the last score)
+    float *part = sc + nk;                              // (behind the last score)
     const int64_t vld = a.vld ? a.vld : a.Dv;           // (values inside the key rows: the latent of latent attention)
     for (int cb = 0; cb < a.Dv; cb += 64) {
         const int c = cb + (threadIdx.x & 63), grp = threadIdx.x >> 6;
         float acc = 0.f;
         if (c < a.Dv)
-            for (int j = j0 + grp; j < ctx; j += 4) {
+            for (int x = grp; x < nk; x += 4) {
+                const int j = x < kept ? x : x + skip;
                 const int64_t row = (int64_t)bt[j / b.block_size] * b.block_size + j % b.block_size;
-                acc += sc[j] * ld_f(vc, (row * a.G + kvh) * vld + c);
+                acc += sc[x] * ld_f(vc, (row * a.G + kvh) * vld + c);
             }
         part[threadIdx.x] = acc;
         __syncthreads();
         if (grp == 0 && c < a.Dv) {
             const float o = (part[threadIdx.x] + part[threadIdx.x + 64]) + (part[threadIdx.x + 128] + part[threadIdx.x + 192]);
-            st_f((CT *)a.out, (int64_t)t * a.ldo + (int64_t)h * a.Dv + c, o * inv);
+            if (maps == 2) a.maps_o[((int64_t)t * a.H * 2 + h) * a.Dv + c] = o * inv;
+            else st_f((CT *)a.out, (int64_t)t * a.ldo + (int64_t)h * a.Dv + c, o * inv);
         }
         __syncthreads();
     }
+}
+
+// The end of differential attention from the maps' outputs [T][H][2][Dv]: a wave per (row, head).
+template <class CT>
+__global__ __launch_bounds__(256) void diff_combine_kernel(SinkAttnArgs a, int64_t n) {
+    const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (i >= n) return;                                 // (a whole wave)
+    const int64_t t = i / a.H; const int h = (int)(i - t * a.H), lane = threadIdx.x & 63;
+    const float *o = a.maps_o + i * 2 * a.Dv;
+    const float lam = *a.lambda;
+    float ss = 0.f;
+    for (int c = lane; c < a.Dv; c += 64) { const float d = o[c] - lam * o[a.Dv + c]; ss += d * d; }
+    float f = a.out_scale / sqrtf(wave_sum(ss) / (float)a.Dv + a.eps);
+    if (a.head_gate) f /= 1.0f + expf(-ld_f((const CT *)a.head_gate, t * a.ldhg + h));
+    for (int c = lane; c < a.Dv; c += 64) st_f((CT *)a.out, t * a.ldo + (int64_t)h * a.Dv + c, (o[c] - lam * o[a.Dv + c]) * f);
 }
 
 // Matrix-core form (bf16 operands; D and Dv multiples of 32 / 16 up to the size class C).  A workgroup owns one tile — up to 64 / g consecutive
@@ -291,9 +311,12 @@ __global__ __launch_bounds__(256) void penalty_table_kernel(const float *__restr
     if (d < n) tab[(int64_t)h * n + d] = (r2 ? r1[h] * log1pf(r2[h] * (float)d) : r1[h] * (float)d) * kLog2e;      // (r2 null: linear in the distance)
 }
 
+// A window with kept first keys: the tiles over the kept keys come first, then those from the window's first key on.  DIFF: differential attention — the two maps of a head
+// are two query rows next to each other over the key row with both maps' keys, each zero in the other map's half; the difference of the rows, its norm and the gate are formed
+// from the accumulators (or in the merge kernel).
 // GATE: no softmax — the weight of a visible key is sigmoid(capped score + bias of the head), the tiles' products are summed as they are (a split's partial carries
 // m = 0 and the first split l = 1, so that the merge adds the partials up).  chunk > 0 (both forms): a row sees the keys from its chunk's first position on.
-template <int C, bool GATE = false>
+template <int C, bool GATE = false, bool DIFF = false>
 __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, Batch b, const AttnTile *__restrict__ tiles, int nsplit, float *__restrict__ part_o,
                                                              float *__restrict__ part_ml) {
     constexpr int KT = 64, KS = C + 8, VS = KT + 8, VG = C + 1, NCH = C / 32;   // NCH: 16-byte pieces of a K (or V) tile per thread
@@ -305,9 +328,9 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
     const int tile = blockIdx.x, kvh = blockIdx.y, z = blockIdx.z;
     const int sq = tiles[tile].seq, lr0 = tiles[tile].row0;
     const int c0 = b.cu[sq], n = b.cu[sq + 1] - c0, st = b.start[sq];
-    const int g = a.H / a.G, PW = 64 / g;
+    const int g = a.H * (DIFF ? 2 : 1) / a.G, PW = 64 / g;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lm = lane & 15, lq = lane >> 4;
-    const int D = a.D, Dv = a.Dv, d32 = D >> 5, dv16 = Dv >> 4;
+    const int D = a.D, Dv = a.Dv, d32 = (D + 31) >> 5, dv16 = (Dv + 15) >> 4;      // (numbers beyond D are zeros in LDS and registers, columns beyond Dv are not stored)
     const int npos = min(PW, n - lr0);                  // positions of this tile
     const bool wave_on = wave * 16 < npos * g;
     const bf16_t *kc = (const bf16_t *)a.kc, *vc = (const bf16_t *)a.vc;
@@ -318,9 +341,14 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
     bf16x8 qf[C / 32];
     {
         const int r = wave * 16 + lm, pi = min(r / g, npos - 1), hg = r % g;
-        const bf16_t *q = (const bf16_t *)a.q + (int64_t)(c0 + lr0 + pi) * a.ldq + (int64_t)(kvh * g + hg) * D + lq * 8;
+        const int Dq = DIFF ? D >> 1 : D, d0 = DIFF ? (hg & 1) * Dq : 0;         // this row's numbers meet d0 .. d0 + Dq - 1 of a key row
+        const bf16_t *q = (const bf16_t *)a.q + (int64_t)(c0 + lr0 + pi) * a.ldq + (int64_t)(kvh * g + hg) * Dq + lq * 8 - d0;
 #pragma unroll
-        for (int ks = 0; ks < C / 32; ++ks) if (ks < d32) qf[ks] = *reinterpret_cast<const bf16x8 *>(q + ks * 32);
+        for (int ks = 0; ks < C / 32; ++ks) {
+            const int d = ks * 32 + lq * 8;
+            qf[ks] = bf16x8{};
+            if (d >= d0 && d < d0 + Dq) qf[ks] = *reinterpret_cast<const bf16x8 *>(q + ks * 32);
+        }
     }
     int pos[4], hgi[4], cs[4]; float m[4], l[4], gb[4];
 #pragma unroll
@@ -342,6 +370,9 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
     const int ntl = (nkeys + KT - 1) / KT;
     int kt0 = a.window > 0 ? max(p0 - a.window + 1, 0) / KT : 0;            // first key tile the tile's first position can see
     if (a.chunk > 0) kt0 = max(kt0, p0 / a.chunk * a.chunk / KT);
+    const int kept = (a.window > 0 && a.keep_first > 0) ? min(kt0, (a.keep_first + KT - 1) / KT) : 0;      // tiles over the kept first keys
+    const int ntk = kept + ntl - kt0;
+    auto tile_key = [&](int x) { return (x < kept ? x : x - kept + kt0) * KT; };
     const int kch = D >> 3;
     uint4 kreg[NCH], vreg[NCH];
     // a thread's pieces: key skey, 16-byte pieces sch, sch + 4, ... of its row; key group vkg, columns vcl, vcl + 32, ... (one block-table lookup each per tile)
@@ -360,14 +391,14 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
             else if (jk < nkeys && sch + 4 * x < (Dv >> 3)) vreg[x] = *reinterpret_cast<const uint4 *>(vrow + (sch + 4 * x) * 8);
         }
     };
-    if (kt0 + z < ntl) request((kt0 + z) * KT);
-    for (int kt = kt0 + z; kt < ntl; kt += nsplit) {
-        const int k0 = kt * KT;
+    if (z < ntk) request(tile_key(z));
+    for (int kt = z; kt < ntk; kt += nsplit) {
+        const int k0 = tile_key(kt);
         const int dmin = max(p0 - (k0 + KT - 1), 0);    // smallest distance a visible key of this tile can have
         __syncthreads();
 #pragma unroll
         for (int x = 0; x < NCH; ++x) {
-            if (sch + 4 * x < kch) *reinterpret_cast<uint4 *>(Ks + skey * KS + (sch + 4 * x) * 8) = kreg[x];
+            if (sch + 4 * x < d32 * 4) *reinterpret_cast<uint4 *>(Ks + skey * KS + (sch + 4 * x) * 8) = kreg[x];
             if (a.v_grouped) { if (vcl + 32 * x < Dv) *reinterpret_cast<uint4 *>(Vg + (vkg * VG + vcl + 32 * x) * 8) = vreg[x]; }
             else if (sch + 4 * x < (Dv >> 3)) {                                  // 8 columns of one key: into the key-group layout, element by element
                 const bf16_t *e = reinterpret_cast<const bf16_t *>(&vreg[x]);
@@ -381,7 +412,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
                 pen[idx] = d < a.pen_n ? a.pen[(int64_t)(kvh * g + hg) * a.pen_n + d] : 0.f;
             }
         __syncthreads();
-        if (kt + nsplit < ntl) request((kt + nsplit) * KT);
+        if (kt + nsplit < ntk) request(tile_key(kt + nsplit));
         if (wave_on) {
             f32x4 s[4];
 #pragma unroll
@@ -418,7 +449,7 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
                     const int dist = pos[i] - j;
                     float v = s[nt][i] * scale2;
                     if (a.pen) v -= pen[(hgi[i] << 7) + min(max(dist - dmin, 0), 127)];
-                    v = (dist < 0 || (a.window > 0 && dist >= a.window) || j < cs[i]) ? -INFINITY : v;
+                    v = (dist < 0 || (a.window > 0 && dist >= a.window && j >= a.keep_first) || j < cs[i]) ? -INFINITY : v;
                     s[nt][i] = v;
                     mx[i] = fmaxf(mx[i], v);
                 }
@@ -462,17 +493,41 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
     for (int i = 0; i < 4; ++i) {
 #pragma unroll
         for (int o = 1; o < 16; o <<= 1) l[i] += __shfl_xor(l[i], o, 64);
+    }
+    if (DIFF && nsplit == 1) {
+        const float lam = *a.lambda;
+#pragma unroll
+        for (int i = 0; i < 4; i += 2) {                        // rows i, i + 1: the two maps of one head
+            const int r = wave * 16 + lq * 4 + i, pi = r / g, h = (kvh * g + r % g) >> 1;
+            const float i0 = 1.0f / l[i], i1 = lam / l[i + 1];
+            float ss = 0.f;
+#pragma unroll
+            for (int t = 0; t < C / 16; ++t) { const float d = acc[t][i] * i0 - acc[t][i + 1] * i1; acc[t][i] = d; if (t * 16 + lm < Dv) ss += d * d; }
+#pragma unroll
+            for (int o = 1; o < 16; o <<= 1) ss += __shfl_xor(ss, o, 64);
+            if (pi >= npos) continue;
+            const int64_t row = c0 + lr0 + pi;
+            float f = a.out_scale / sqrtf(ss / (float)Dv + a.eps);
+            if (a.head_gate) f /= 1.0f + expf(-ld_f((const bf16_t *)a.head_gate, row * a.ldhg + h));
+            bf16_t *o = (bf16_t *)a.out + row * a.ldo + (int64_t)h * Dv;
+#pragma unroll
+            for (int t = 0; t < C / 16; ++t) if (t * 16 + lm < Dv) st_f(o, t * 16 + lm, acc[t][i] * f);
+        }
+        return;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
         const int r = wave * 16 + lq * 4 + i, pi = r / g, hg = r % g;
         if (pi >= npos) continue;
         if (nsplit == 1) {
             const float inv = 1.0f / l[i];
             bf16_t *o = (bf16_t *)a.out + (int64_t)(c0 + lr0 + pi) * a.ldo + (int64_t)(kvh * g + hg) * Dv;
 #pragma unroll
-            for (int t = 0; t < C / 16; ++t) if (t < dv16) st_f(o, t * 16 + lm, acc[t][i] * inv);
+            for (int t = 0; t < C / 16; ++t) if (t * 16 + lm < Dv) st_f(o, t * 16 + lm, acc[t][i] * inv);
         } else {
             const int64_t pr = (((int64_t)tile * a.G + kvh) * nsplit + z) * 64 + r;
 #pragma unroll
-            for (int t = 0; t < C / 16; ++t) if (t < dv16) part_o[pr * Dv + t * 16 + lm] = acc[t][i];
+            for (int t = 0; t < C / 16; ++t) if (t * 16 + lm < Dv) part_o[pr * Dv + t * 16 + lm] = acc[t][i];
             if (lm == 0) { part_ml[pr * 2] = m[i]; part_ml[pr * 2 + 1] = l[i]; }
         }
     }
@@ -498,6 +553,44 @@ __global__ __launch_bounds__(64) void sink_attn_merge_kernel(SinkAttnArgs a, Bat
         for (int z = 0; z < nsplit; ++z) { const float mz = part_ml[((base + z) * 64 + r) * 2]; if (mz != -INFINITY) acc += part_o[((base + z) * 64 + r) * a.Dv + c] * exp2f(mz - m); }
         st_f(o, c, acc / l);
     }
+}
+
+// the same for differential attention: one wave per (tile, key/value head, head's pair of rows), Dv <= 256
+__global__ __launch_bounds__(64) void diff_attn_merge_kernel(SinkAttnArgs a, Batch b, const AttnTile *__restrict__ tiles, int nsplit, const float *__restrict__ part_o,
+                                                             const float *__restrict__ part_ml) {
+    const int tile = blockIdx.x, kvh = blockIdx.y, r = blockIdx.z * 2;
+    const int sq = tiles[tile].seq, lr0 = tiles[tile].row0;
+    const int c0 = b.cu[sq], n = b.cu[sq + 1] - c0;
+    const int g = 2 * a.H / a.G, PW = 64 / g, npos = min(PW, n - lr0);
+    const int pi = r / g, h = (kvh * g + r % g) >> 1;
+    if (pi >= npos) return;
+    const int64_t base = ((int64_t)tile * a.G + kvh) * nsplit;
+    float d[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+        float m = -INFINITY;
+        for (int z = 0; z < nsplit; ++z) m = fmaxf(m, part_ml[((base + z) * 64 + r + k) * 2]);
+        float l = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
+        for (int z = 0; z < nsplit; ++z) {
+            const float mz = part_ml[((base + z) * 64 + r + k) * 2];
+            if (mz == -INFINITY) continue;
+            const float e = exp2f(mz - m);
+            l += part_ml[((base + z) * 64 + r + k) * 2 + 1] * e;
+            const float *o = part_o + ((base + z) * 64 + r + k) * a.Dv;
+#pragma unroll
+            for (int x = 0; x < 4; ++x) if (threadIdx.x + 64 * x < a.Dv) acc[x] += o[threadIdx.x + 64 * x] * e;
+        }
+        const float f = k ? -*a.lambda / l : 1.0f / l;
+#pragma unroll
+        for (int x = 0; x < 4; ++x) d[x] += acc[x] * f;
+    }
+    const float ss = wave_sum((d[0] * d[0] + d[1] * d[1]) + (d[2] * d[2] + d[3] * d[3]));
+    const int64_t row = c0 + lr0 + pi;
+    float f = a.out_scale / sqrtf(ss / (float)a.Dv + a.eps);
+    if (a.head_gate) f /= 1.0f + expf(-ld_f((const bf16_t *)a.head_gate, row * a.ldhg + h));
+    bf16_t *o = (bf16_t *)a.out + row * a.ldo + (int64_t)h * a.Dv;
+#pragma unroll
+    for (int x = 0; x < 4; ++x) if (threadIdx.x + 64 * x < a.Dv) st_f(o, threadIdx.x + 64 * x, d[x] * f);
 }
 
 // ------------------------------------------------------------------------------------------------ retention, token by token
@@ -855,6 +948,9 @@ int prepare() {
     NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<64, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
     NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<128, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
     NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<256, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
+    NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<64, false, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
+    NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<128, false, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
+    NVR_HIP_CHECK(hipFuncSetAttribute((const void *)sink_attn_mfma_kernel<256, false, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
     NVR_HIP_CHECK(hipFuncSetAttribute((const void *)norm_canon_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
     NVR_HIP_CHECK(hipFuncSetAttribute((const void *)norm_canon_kernel<bf16_t>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kMaxLds));
     return 0;
@@ -900,14 +996,17 @@ int kv_store(const void *proj, int64_t ld, int64_t kcol, int64_t vcol, const Bat
 }
 
 bool sink_attention_tiled_ok(const SinkAttnArgs &a, bool bf16, int block_size) {
-    return bf16 && (block_size % 8 == 0 || !a.v_grouped) && a.G >= 1 && a.H % a.G == 0 && a.H / a.G <= 16 && a.D % 32 == 0 && a.Dv % 16 == 0 && a.D <= 256 && a.Dv <= 256 && a.ldq % 8 == 0 && a.vld % 8 == 0 && (!a.vld || !a.v_grouped) &&
-           ((uintptr_t)a.q % 16) == 0 && ((uintptr_t)a.kc % 16) == 0 && ((uintptr_t)a.vc % 16) == 0;
+    const int maps = a.lambda ? 2 : 1;
+    return bf16 && (block_size % 8 == 0 || !a.v_grouped) && a.G >= 1 && a.H % a.G == 0 && a.H * maps / a.G <= 16 && a.D % (8 * maps) == 0 && a.Dv % 8 == 0 && a.D <= 256 && a.Dv <= 256 && a.ldq % 8 == 0 && a.vld % 8 == 0 &&
+           (!a.vld || !a.v_grouped) && ((uintptr_t)a.q % 16) == 0 && ((uintptr_t)a.kc % 16) == 0 && ((uintptr_t)a.vc % 16) == 0;
 }
 size_t sink_attention_workspace_bytes(int max_workgroups) { return (size_t)max_workgroups * 64 * (256 + 2) * sizeof(float); }
 
 int sink_attention_tiled(const SinkAttnArgs &a, const Batch &b, const AttnTile *tiles, int ntiles, int nsplit, void *workspace, size_t workspace_bytes, hipStream_t s) {
     if (ntiles == 0) return 0;
     if (!sink_attention_tiled_ok(a, true, b.block_size) || (a.v_grouped && b.block_size % 8)) return nvr::fail(NVR_ERR_UNSUPPORTED, "sink_attention_tiled: shape outside the matrix-core kernel");
+    if (a.lambda && (a.r1 || a.r2 || a.slope || a.sink || a.pen || a.gate_bias)) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention_tiled: differential attention takes no penalty, sink or gated weights");
+    if (a.pen && a.keep_first > 0) return nvr::fail(NVR_ERR_UNSUPPORTED, "sink_attention_tiled: kept first keys together with a penalty table");
     if (nsplit < 1) nsplit = 1;
     float *po = nullptr, *pml = nullptr;
     if (nsplit > 1) {
@@ -916,20 +1015,25 @@ int sink_attention_tiled(const SinkAttnArgs &a, const Batch &b, const AttnTile *
         po = (float *)workspace; pml = po + rows * a.Dv;
     }
     const int C = std::max(a.D, a.Dv) <= 64 ? 64 : std::max(a.D, a.Dv) <= 128 ? 128 : 256;
-    const size_t lds = ((size_t)64 * (C + 8) + (size_t)8 * (C + 1) * 8 + (size_t)64 * 72) * 2 + (size_t)(a.H / a.G) * 128 * 4;
+    const size_t lds = ((size_t)64 * (C + 8) + (size_t)8 * (C + 1) * 8 + (size_t)64 * 72) * 2 + (a.pen ? (size_t)(a.H / a.G) * 128 * 4 : 0);
     const dim3 grid((unsigned)ntiles, (unsigned)a.G, (unsigned)nsplit);
     if (a.gate_bias) {
         if (a.r1 || a.r2 || a.slope || a.sink || a.pen) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention_tiled: gated weights take no penalty and no sink");
         if (C == 64) sink_attn_mfma_kernel<64, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
         else if (C == 128) sink_attn_mfma_kernel<128, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
         else sink_attn_mfma_kernel<256, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
+    } else if (a.lambda) {
+        if (C == 64) sink_attn_mfma_kernel<64, false, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
+        else if (C == 128) sink_attn_mfma_kernel<128, false, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
+        else sink_attn_mfma_kernel<256, false, true><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
     } else if (C == 64) sink_attn_mfma_kernel<64><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
     else if (C == 128) sink_attn_mfma_kernel<128><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
     else sink_attn_mfma_kernel<256><<<grid, dim3(256), lds, s>>>(a, b, tiles, nsplit, po, pml);
     if (int rc = launched("sink_attention_tiled")) return rc;
     if (nsplit > 1) {
-        const int g = a.H / a.G, rows = std::min(64, std::max(1, std::min(64 / g, (int)b.max_rows)) * g);      // rows a tile of this step can hold
-        sink_attn_merge_kernel<<<dim3((unsigned)ntiles, (unsigned)a.G, (unsigned)rows), dim3(64), 0, s>>>(a, b, tiles, nsplit, po, pml);
+        const int g = a.H * (a.lambda ? 2 : 1) / a.G, rows = std::min(64, std::max(1, std::min(64 / g, (int)b.max_rows)) * g);      // rows a tile of this step can hold
+        if (a.lambda) diff_attn_merge_kernel<<<dim3((unsigned)ntiles, (unsigned)a.G, (unsigned)(rows / 2)), dim3(64), 0, s>>>(a, b, tiles, nsplit, po, pml);
+        else sink_attn_merge_kernel<<<dim3((unsigned)ntiles, (unsigned)a.G, (unsigned)rows), dim3(64), 0, s>>>(a, b, tiles, nsplit, po, pml);
         return launched("sink_attention merge");
     }
     return 0;
@@ -950,14 +1054,20 @@ int sink_attention(const SinkAttnArgs &a, const Batch &b, bool bf16, hipStream_t
     if (b.T == 0) return 0;
     if (a.G < 1 || a.H % a.G) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention: %d heads over %d key/value heads", a.H, a.G);
     if ((a.r1 || a.r2) && a.slope) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention: a logarithmic and a linear penalty together");
-    size_t keys = a.window > 0 ? (size_t)std::min(b.max_ctx, a.window) : (size_t)b.max_ctx;
+    if (a.lambda && (a.r1 || a.r2 || a.slope || a.sink || a.gate_bias || a.D % 2 || !a.maps_o)) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention: differential attention takes no penalty, sink or gated weights and needs room for the maps' outputs");
+    size_t keys = a.window > 0 ? (size_t)std::min<int64_t>(b.max_ctx, (int64_t)a.window + std::max(a.keep_first, 0)) : (size_t)b.max_ctx;
     if (a.chunk > 0) keys = std::min(keys, (size_t)a.chunk);
     if (a.gate_bias && (a.r1 || a.r2 || a.slope || a.sink)) return nvr::fail(NVR_ERR_INVALID_ARG, "sink_attention: gated weights take no penalty and no sink");
     const size_t lds = ((size_t)a.D + keys + 256) * 4;
     if (lds > kMaxLds) return nvr::fail(NVR_ERR_UNSUPPORTED, "sink_attention: %zu visible keys do not fit the score buffer", keys);
-    const dim3 grid((unsigned)b.T, (unsigned)a.H);
+    const dim3 grid((unsigned)b.T, (unsigned)(a.H * (a.lambda ? 2 : 1)));
     if (bf16) sink_attn_rows_kernel<bf16_t><<<grid, dim3(256), lds, s>>>(a, b);
     else sink_attn_rows_kernel<float><<<grid, dim3(256), lds, s>>>(a, b);
+    if (a.lambda) {
+        const int64_t n = (int64_t)b.T * a.H;
+        if (bf16) diff_combine_kernel<bf16_t><<<dim3((unsigned)((n + 3) / 4)), dim3(256), 0, s>>>(a, n);
+        else diff_combine_kernel<float><<<dim3((unsigned)((n + 3) / 4)), dim3(256), 0, s>>>(a, n);
+    }
     return launched("sink_attention");
 }
 

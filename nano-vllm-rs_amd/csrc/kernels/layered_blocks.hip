@@ -38,6 +38,8 @@ __device__ __forceinline__ float block_sum256(float v, float *red) {       // re
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gelu_tanh_f(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
+__device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
 int launched(const char *what) {
     hipError_t e = hipGetLastError();
     if (e != hipSuccess) return nvr::fail(NVR_ERR_HIP, "%s launch failed: %s", what, hipGetErrorString(e));
@@ -82,7 +84,7 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const IT *__restrict__ 
 // divided by its root mean square times w, and the key part with coordinate pairs (2i, 2i+1) turned by position * freq[i].
 template <class CT>
 __global__ __launch_bounds__(64) void latent_store_kernel(const CT *__restrict__ proj, int64_t ld, int64_t col, Batch b, int rank, int rot, float eps,
-                                                          const float *__restrict__ w, const float *__restrict__ freq, CT *__restrict__ pages, CT *__restrict__ rows) {
+                                                          const float *__restrict__ w, const float *__restrict__ freq, CT *__restrict__ pages, CT *__restrict__ rows, int halves, float gain) {
     const int t = blockIdx.x, sq = b.row_seq[t], lane = threadIdx.x;
     const int p = b.start[sq] + (t - b.cu[sq]);
     const int blk = b.block_tables[(int64_t)sq * b.max_blocks + p / b.block_size];
@@ -94,27 +96,29 @@ __global__ __launch_bounds__(64) void latent_store_kernel(const CT *__restrict__
     CT *dst2 = rows ? rows + (int64_t)t * (rank + rot) : nullptr;      // the same row once more, in step order
     for (int c = lane; c < rank; c += 64) { const float v = ld_f(src, c) * inv * w[c]; st_f(dst, c, v); if (dst2) st_f(dst2, c, v); }
     for (int i = lane; i < rot / 2; i += 64) {
-        const float ang = (float)p * freq[i], cs = cosf(ang), sn = sinf(ang);
-        const float u = ld_f(src, rank + 2 * i), v = ld_f(src, rank + 2 * i + 1);
-        st_f(dst, rank + 2 * i, u * cs - v * sn); st_f(dst, rank + 2 * i + 1, v * cs + u * sn);
-        if (dst2) { st_f(dst2, rank + 2 * i, u * cs - v * sn); st_f(dst2, rank + 2 * i + 1, v * cs + u * sn); }
+        const float ang = (float)p * freq[i], cs = gain * cosf(ang), sn = gain * sinf(ang);
+        const int cu = rank + (halves ? i : 2 * i), cv = rank + (halves ? i + rot / 2 : 2 * i + 1);
+        const float u = ld_f(src, cu), v = ld_f(src, cv);
+        st_f(dst, cu, u * cs - v * sn); st_f(dst, cv, v * cs + u * sn);
+        if (dst2) { st_f(dst2, cu, u * cs - v * sn); st_f(dst2, cv, v * cs + u * sn); }
     }
 }
 
 // q rows [H][D + rot]: the last rot numbers of every head, rotated like the key part, go to out rows [H][ldh] at column ocol
 template <class CT>
 __global__ __launch_bounds__(256) void rotate_heads_kernel(const CT *__restrict__ q, int64_t ldq, int qstride, int qcol, Batch b, int H, int rot, const float *__restrict__ freq,
-                                                           CT *__restrict__ out, int64_t ldo, int ostride, int ocol) {
+                                                           CT *__restrict__ out, int64_t ldo, int ostride, int ocol, int halves, float gain) {
     const int t = blockIdx.x, sq = b.row_seq[t];
     const int p = b.start[sq] + (t - b.cu[sq]);
     const int half = rot / 2;
     for (int idx = threadIdx.x; idx < H * half; idx += 256) {
         const int h = idx / half, i = idx - h * half;
-        const float ang = (float)p * freq[i], cs = cosf(ang), sn = sinf(ang);
+        const float ang = (float)p * freq[i], cs = gain * cosf(ang), sn = gain * sinf(ang);
+        const int cu = halves ? i : 2 * i, cv = halves ? i + half : 2 * i + 1;
         const CT *src = q + (int64_t)t * ldq + (int64_t)h * qstride + qcol;
-        const float u = ld_f(src, 2 * i), v = ld_f(src, 2 * i + 1);
+        const float u = ld_f(src, cu), v = ld_f(src, cv);
         CT *dst = out + (int64_t)t * ldo + (int64_t)h * ostride + ocol;
-        st_f(dst, 2 * i, u * cs - v * sn); st_f(dst, 2 * i + 1, v * cs + u * sn);
+        st_f(dst, cu, u * cs - v * sn); st_f(dst, cv, v * cs + u * sn);
     }
 }
 
@@ -809,6 +813,77 @@ __global__ __launch_bounds__(256) void moe_combine8_kernel(const bf16_t *__restr
     *reinterpret_cast<uint4 *>(out + t * W + c) = o;
 }
 
+// out = z Phi(z) (rows of F numbers)
+template <class CT>
+__global__ __launch_bounds__(256) void gelu_erf_kernel(const CT *__restrict__ z, int64_t ldz, int64_t T, int64_t F, CT *__restrict__ out, int64_t ldo) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= T * F) return;
+    const int64_t t = i / F, c = i - t * F;
+    st_f(out, t * ldo + c, gelu_erf_f(ld_f(z, t * ldz + c)));
+}
+
+// the same for 16-bit rows, 8 numbers per thread (F and both strides multiples of 8, 16-byte aligned rows)
+__global__ __launch_bounds__(256) void gelu_erf8_kernel(const bf16_t *__restrict__ z, int64_t ldz, int64_t T, int64_t F8, bf16_t *__restrict__ out, int64_t ldo) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= T * F8) return;
+    const int64_t t = i / F8, c = (i - t * F8) * 8;
+    uint4 v = *reinterpret_cast<const uint4 *>(z + t * ldz + c);
+    bf16_t *e = reinterpret_cast<bf16_t *>(&v);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) st_f(e, k, gelu_erf_f(ld_f(e, k)));
+    *reinterpret_cast<uint4 *>(out + t * ldo + c) = v;
+}
+
+// ------------------------------------------------------------------------------------------------ a normed row joins the stream
+// x += y / rms(y) * wb; then, where asked for, out = x / rms(x) * wn, or (plain) x itself in the operand type.  16-bit rows, widths that are multiples of 4, one norm group: NT threads
+// per row (64: a wave, four rows per workgroup, no barrier; 256: the workgroup), the row in registers.
+template <int NT, int NV>
+__global__ __launch_bounds__(256) void norm_join4_kernel(float *__restrict__ x, const bf16_t *__restrict__ y, int64_t ldy, int64_t T, int W, float eps, const float *__restrict__ wb,
+                                                         const float *__restrict__ wn, int plain, bf16_t *__restrict__ out, int64_t ldo) {
+    __shared__ float red[4];
+    const int W4 = W >> 2, l = threadIdx.x & (NT - 1);
+    const int64_t t = (int64_t)blockIdx.x * (256 / NT) + threadIdx.x / NT;
+    if (NT == 64 && t >= T) return;                     // (a whole wave: nobody waits for it)
+    float *xr = x + t * W;
+    float4 xs[NV], ys[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = l + k * NT;
+        xs[k] = ys[k] = float4{0.f, 0.f, 0.f, 0.f};
+        if (c4 < W4) {
+            xs[k] = *reinterpret_cast<const float4 *>(xr + c4 * 4);
+            const uint2 v = *reinterpret_cast<const uint2 *>(y + t * ldy + c4 * 4);
+            ys[k] = float4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)};
+        }
+        ss += (ys[k].x * ys[k].x + ys[k].y * ys[k].y) + (ys[k].z * ys[k].z + ys[k].w * ys[k].w);
+    }
+    const float f = 1.0f / sqrtf((NT == 64 ? wave_sum(ss) : block_sum256(ss, red)) / (float)W + eps);
+    float s2 = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = l + k * NT;
+        if (c4 < W4) {
+            const float4 w = *reinterpret_cast<const float4 *>(wb + c4 * 4);
+            xs[k].x += ys[k].x * f * w.x; xs[k].y += ys[k].y * f * w.y; xs[k].z += ys[k].z * f * w.z; xs[k].w += ys[k].w * f * w.w;
+            *reinterpret_cast<float4 *>(xr + c4 * 4) = xs[k];
+            s2 += (xs[k].x * xs[k].x + xs[k].y * xs[k].y) + (xs[k].z * xs[k].z + xs[k].w * xs[k].w);
+        }
+    }
+    if (!wn && !plain) return;
+    const float f2 = wn ? 1.0f / sqrtf((NT == 64 ? wave_sum(s2) : block_sum256(s2, red)) / (float)W + eps) : 1.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = l + k * NT;
+        if (c4 < W4) {
+            const float4 w = wn ? *reinterpret_cast<const float4 *>(wn + c4 * 4) : float4{1.f, 1.f, 1.f, 1.f};
+            bf16_t h[4];
+            st_f(h, 0, xs[k].x * f2 * w.x); st_f(h, 1, xs[k].y * f2 * w.y); st_f(h, 2, xs[k].z * f2 * w.z); st_f(h, 3, xs[k].w * f2 * w.w);
+            *reinterpret_cast<uint2 *>(out + t * ldo + c4 * 4) = uint2{(uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16)};
+        }
+    }
+}
+
 // ------------------------------------------------------------------------------------------------ end of a layer
 // Per row: (1) the token input's last step: x += y / rms(y) * wn for the projected rows y (side_y); (2) X_(i+1) = x goes to its
 // place among the kept streams and x becomes sum_j mix[j] X_j over the nx kept streams (X_0 the embedding output ... X_(nx-1) this layer's); (3) with wnext the next layer's
@@ -911,9 +986,27 @@ int embed_keep(const void *E, bool bf16, const int64_t *ids, int64_t T, int64_t 
     return launched("embed_keep");
 }
 
+static bool aligned16(const void *p) { return ((uintptr_t)p & 15) == 0; }
+
+static bool norm_join4_ok(int64_t W, const float *x, const void *y, int64_t ldy, const float *wb, const float *wn, const void *out, int64_t ldo) {
+    return W % 4 == 0 && W <= 8192 && ldy % 4 == 0 && ldo % 4 == 0 && aligned16(x) && aligned16(y) && aligned16(wb) && aligned16(wn) && aligned16(out);
+}
+static int norm_join4(float *x, const void *y, int64_t ldy, int64_t T, int64_t W, float eps, const float *wb, const float *wn, bool plain, void *out, int64_t ldo, hipStream_t s) {
+    const int64_t W4 = W / 4;
+    const bool wave = T >= 1024 && W4 <= 256;           // many rows: a wave per row up to 1024 numbers; few rows: a workgroup per row
+    const dim3 grid((unsigned)(wave ? (T + 3) / 4 : T)), blk(256);
+#define NVR_NJ(NT_, NV_) norm_join4_kernel<NT_, NV_><<<grid, blk, 0, s>>>(x, (const bf16_t *)y, ldy, T, (int)W, eps, wb, wn, plain ? 1 : 0, (bf16_t *)out, ldo)
+    if (wave) { if (W4 <= 64) NVR_NJ(64, 1); else if (W4 <= 128) NVR_NJ(64, 2); else NVR_NJ(64, 4); }
+    else if (W4 <= 256) NVR_NJ(256, 1); else if (W4 <= 512) NVR_NJ(256, 2); else if (W4 <= 1024) NVR_NJ(256, 4); else NVR_NJ(256, 8);
+#undef NVR_NJ
+    return launched("norm_join4");
+}
+
 int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s) {
     if (a.rows_n == 0) return 0;
     if (a.groups < 1 || a.W % a.groups) return nvr::fail(NVR_ERR_INVALID_ARG, "group_norm: %ld columns in %d groups", (long)a.W, a.groups);
+    if (bf16 && a.xres && a.groups == 1 && !a.in_f32 && !a.rows && !(a.w2 && a.out_plain) && norm_join4_ok(a.W, a.xres, a.in, a.ldi, a.w, a.w2, a.out, a.ldo))
+        return norm_join4(a.xres, a.in, a.ldi, a.rows_n, a.W, a.eps, a.w, a.w2, a.out_plain, a.out, a.ldo, s);
     if (a.out_plain && (a.w2 || !a.xres)) return nvr::fail(NVR_ERR_INVALID_ARG, "group_norm: a plain copy leaves only with the residual sum, instead of the next norm");
     const dim3 grid((unsigned)a.rows_n), blk(256);
     const int W = (int)a.W;
@@ -931,24 +1024,22 @@ int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s) {
 }
 
 int latent_store(const void *proj, int64_t ld, int64_t col, const Batch &b, int64_t rank, int64_t rot, float eps, const float *w, const float *freq, void *pages, void *rows,
-                 bool bf16, hipStream_t s) {
+                 bool bf16, hipStream_t s, bool halves, float gain) {
     if (b.T == 0) return 0;
     if (rot % 2) return nvr::fail(NVR_ERR_INVALID_ARG, "latent_store: %ld rotated coordinates", (long)rot);
-    if (bf16) latent_store_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const bf16_t *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (bf16_t *)pages, (bf16_t *)rows);
-    else latent_store_kernel<float><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const float *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (float *)pages, (float *)rows);
+    if (bf16) latent_store_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const bf16_t *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (bf16_t *)pages, (bf16_t *)rows, halves ? 1 : 0, gain);
+    else latent_store_kernel<float><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const float *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (float *)pages, (float *)rows, halves ? 1 : 0, gain);
     return launched("latent_store");
 }
 
 int rotate_heads(const void *q, int64_t ldq, int64_t qstride, int64_t qcol, const Batch &b, int64_t H, int64_t rot, const float *freq, void *out, int64_t ldo, int64_t ostride,
-                 int64_t ocol, bool bf16, hipStream_t s) {
+                 int64_t ocol, bool bf16, hipStream_t s, bool halves, float gain) {
     if (b.T == 0 || rot == 0) return 0;
     if (rot % 2) return nvr::fail(NVR_ERR_INVALID_ARG, "rotate_heads: %ld rotated coordinates", (long)rot);
-    if (bf16) rotate_heads_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const bf16_t *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (bf16_t *)out, ldo, (int)ostride, (int)ocol);
-    else rotate_heads_kernel<float><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const float *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (float *)out, ldo, (int)ostride, (int)ocol);
+    if (bf16) rotate_heads_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const bf16_t *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (bf16_t *)out, ldo, (int)ostride, (int)ocol, halves ? 1 : 0, gain);
+    else rotate_heads_kernel<float><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const float *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (float *)out, ldo, (int)ostride, (int)ocol, halves ? 1 : 0, gain);
     return launched("rotate_heads");
 }
-
-static bool aligned16(const void *p) { return ((uintptr_t)p & 15) == 0; }
 
 int head_linear(const HeadLinearArgs &a, bool bf16, hipStream_t s) {
     if (a.T == 0 || a.N == 0 || a.H == 0) return 0;
@@ -999,6 +1090,18 @@ static int gated_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ld
 }
 int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) { return gated_mul<false>(gu, T, F, out, ldo, bf16, s); }
 int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) { return gated_mul<true>(gu, T, F, out, ldo, bf16, s); }
+
+int gelu_erf(const void *z, int64_t ldz, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s) {
+    if (T * F == 0) return 0;
+    if (bf16 && F % 8 == 0 && ldz % 8 == 0 && ldo % 8 == 0 && aligned16(z) && aligned16(out)) {
+        gelu_erf8_kernel<<<dim3((unsigned)((T * (F / 8) + 255) / 256)), dim3(256), 0, s>>>((const bf16_t *)z, ldz, T, F / 8, (bf16_t *)out, ldo);
+        return launched("gelu_erf");
+    }
+    const dim3 grid((unsigned)((T * F + 255) / 256));
+    if (bf16) gelu_erf_kernel<bf16_t><<<grid, dim3(256), 0, s>>>((const bf16_t *)z, ldz, T, F, (bf16_t *)out, ldo);
+    else gelu_erf_kernel<float><<<grid, dim3(256), 0, s>>>((const float *)z, ldz, T, F, (float *)out, ldo);
+    return launched("gelu_erf");
+}
 
 int moe_route(const void *h, int64_t ldh, int64_t T, int64_t W, const float *wr, int64_t E, int64_t top, int32_t *sel, float *score, int32_t *off, int32_t *order,
               int32_t *place_of, int64_t pad, int32_t *row_w, int64_t nblocks, bool bf16, hipStream_t s, bool softmax, int64_t extra, float *extra_out,
@@ -1076,6 +1179,8 @@ int side_gate(const void *z, const int64_t *ids, const void *E, int64_t lde, int
 
 int layer_tail(const LayerTailArgs &a, bool bf16, hipStream_t s) {
     if (a.T == 0) return 0;
+    if (bf16 && a.side_y && !a.kept && (!a.wnext || a.groups == 1) && norm_join4_ok(a.W, a.x, a.side_y, a.W, a.side_norm, a.wnext, a.out, a.W))
+        return norm_join4(a.x, a.side_y, a.W, a.T, a.W, a.eps, a.side_norm, a.wnext, false, a.out, a.W, s);
     const size_t lds = (size_t)2 * a.W * 4;
     if (lds > kMaxLds) return nvr::fail(NVR_ERR_UNSUPPORTED, "layer_tail: rows of %d numbers do not fit LDS", a.W);
     if (a.wnext && (a.groups < 1 || a.W % a.groups)) return nvr::fail(NVR_ERR_INVALID_ARG, "layer_tail: %d columns in %d groups", a.W, a.groups);

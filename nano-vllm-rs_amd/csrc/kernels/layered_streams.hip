@@ -191,17 +191,25 @@ __global__ __launch_bounds__(256) void qkv_rope_kernel(QkvRopeArgs a, Batch b) {
     CT *pr = (CT *)a.proj + (int64_t)t * a.ld;
     const int D = a.D, half = a.rot / 2, np = (D + 1) / 2;
     float *cs = sm, *sn = sm + half;
-    for (int i = threadIdx.x; i < half; i += 256) { const float ang = (float)p * a.freq[i]; cs[i] = cosf(ang); sn[i] = sinf(ang); }
+    const float gain = a.gain == 0.f ? 1.f : a.gain;
+    for (int i = threadIdx.x; i < half; i += 256) { const float ang = (float)p * a.freq[i]; cs[i] = gain * cosf(ang); sn[i] = gain * sinf(ang); }
     __syncthreads();
     for (int hd = threadIdx.x >> 6; hd < a.H + a.G; hd += 4) {
         const bool isq = hd < a.H;
         const int h = isq ? hd : hd - a.H;
         CT *src = pr + (isq ? a.qcol : a.kcol) + (int64_t)h * D;
-        const float *bias = isq ? a.bq : a.bk;
+        const float *bias = isq ? a.bq : a.bk, *wn = isq ? a.wq : a.wk;
         CT *dst = isq ? src : (CT *)a.kc + (row * a.G + h) * D;
+        auto raw = [&](int c) { return c < D ? ld_f(src, c) + (bias ? bias[(int64_t)h * D + c] : 0.f) : 0.f; };
+        float pre = 1.f;
+        if (wn) {
+            float ss = 0.f;
+            for (int c = lane; c < D; c += 64) { const float v = raw(c); ss += v * v; }
+            pre = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
+        }
         auto turned = [&](int i, int ca, int cb, float &u, float &v) {
-            u = ld_f(src, ca) + (bias ? bias[(int64_t)h * D + ca] : 0.f);
-            v = cb < D ? ld_f(src, cb) + (bias ? bias[(int64_t)h * D + cb] : 0.f) : 0.f;
+            u = raw(ca); v = raw(cb);
+            if (wn) { u *= pre * wn[ca]; v *= cb < D ? pre * wn[cb] : 0.f; }
             if (i < half) { const float c = cs[i], s = sn[i], u0 = u; u = u0 * c - v * s; v = v * c + u0 * s; }
         };
         float f = 1.f;
@@ -216,7 +224,7 @@ __global__ __launch_bounds__(256) void qkv_rope_kernel(QkvRopeArgs a, Batch b) {
             st_f(dst, ca, u * f); if (cb < D) st_f(dst, cb, v * f);
         }
     }
-    const int GV = a.G * a.Dv;
+    const int GV = (a.Gv > 0 ? a.Gv : a.G) * a.Dv;
     CT *vc = (CT *)a.vc;
     const int64_t grp = ((int64_t)blk * (b.block_size >> 3) + (jj >> 3)) * GV;        // grouped value pages: [block][block_size / 8][G][Dv][8 keys]
     const float lam = a.v_first ? *a.lambda : 0.f;
@@ -228,16 +236,16 @@ __global__ __launch_bounds__(256) void qkv_rope_kernel(QkvRopeArgs a, Batch b) {
     }
 }
 
-// 16-bit rows, rotated pairs, all parts multiples of 8 numbers: LP lanes with 8 numbers each per head (16-byte loads and stores, pairs inside a lane, the sum of squares by
-// shuffles), 64 / LP heads per wave at a time; RB rows per workgroup (1: the four waves share a row's heads; 4: a wave per row), cosines and sines once per row.
-template <int LP, int RB>
+// 16-bit rows, all parts multiples of 8 numbers: LP lanes with 8 numbers each per head (16-byte loads and stores, pairs inside a lane — with HALVES the partner's 8 numbers come
+// from the lane half / 8 further —, the sums of squares by shuffles), 64 / LP heads per wave at a time; RB rows per workgroup (1: the four waves share a row's heads; 4: a wave per row), cosines and sines once per row.
+template <int LP, int RB, bool HALVES>
 __global__ __launch_bounds__(256) void qkv_rope8_kernel(QkvRopeArgs a, Batch b) {
     extern __shared__ float2 tab[];                     // [RB][half] (cosine, sine)
     constexpr int WR = 4 / RB, HW = 64 / LP;            // waves per row, heads per wave and pass
     const int half = a.rot / 2, r0 = blockIdx.x * RB;
     for (int idx = threadIdx.x; idx < RB * half; idx += 256) {
         const int rr = RB == 1 ? 0 : idx / half, i = idx - rr * half, t = r0 + rr;
-        if (t < b.T) { const int sq = b.row_seq[t]; const float ang = (float)(b.start[sq] + (t - b.cu[sq])) * a.freq[i]; tab[idx] = float2{cosf(ang), sinf(ang)}; }
+        if (t < b.T) { const int sq = b.row_seq[t]; const float ang = (float)(b.start[sq] + (t - b.cu[sq])) * a.freq[i], gain = a.gain == 0.f ? 1.f : a.gain; tab[idx] = float2{gain * cosf(ang), gain * sinf(ang)}; }
     }
     __syncthreads();
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, rr = wave / WR, wv = wave % WR, t = r0 + rr;
@@ -252,7 +260,7 @@ __global__ __launch_bounds__(256) void qkv_rope8_kernel(QkvRopeArgs a, Batch b) 
         const int hd = hd0 + sub;
         const bool on = hd < a.H + a.G && l * 8 < D, isq = hd < a.H;
         const int h = isq ? hd : hd - a.H;
-        float e[8];
+        float e[8] = {};
         float ss = 0.f;
         bf16_t *src = pr + (isq ? a.qcol : a.kcol) + (int64_t)h * D + l * 8;
         if (on) {
@@ -264,6 +272,34 @@ __global__ __launch_bounds__(256) void qkv_rope8_kernel(QkvRopeArgs a, Batch b) 
                 const float4 b0 = *reinterpret_cast<const float4 *>(bias + (int64_t)h * D + l * 8), b1 = *reinterpret_cast<const float4 *>(bias + (int64_t)h * D + l * 8 + 4);
                 e[0] += b0.x; e[1] += b0.y; e[2] += b0.z; e[3] += b0.w; e[4] += b1.x; e[5] += b1.y; e[6] += b1.z; e[7] += b1.w;
             }
+        }
+        const float *wn = isq ? a.wq : a.wk;
+        if (a.wq || a.wk) {                                 // (every lane of the wave: q and k heads may share a pass)
+            float sw = 0.f;
+            if (on)
+#pragma unroll
+                for (int k = 0; k < 8; ++k) sw += e[k] * e[k];
+#pragma unroll
+            for (int o = LP / 2; o > 0; o >>= 1) sw += __shfl_xor(sw, o, 64);
+            if (on && wn) {
+                const float pre = 1.0f / sqrtf(sw / (float)D + a.eps);
+                const float4 w0 = *reinterpret_cast<const float4 *>(wn + l * 8), w1 = *reinterpret_cast<const float4 *>(wn + l * 8 + 4);
+                e[0] *= pre * w0.x; e[1] *= pre * w0.y; e[2] *= pre * w0.z; e[3] *= pre * w0.w; e[4] *= pre * w1.x; e[5] *= pre * w1.y; e[6] *= pre * w1.z; e[7] *= pre * w1.w;
+            }
+        }
+        if (HALVES) {
+            const int hl = half >> 3, i0 = l < hl ? l : l - hl;
+            const bool turn = on && l < 2 * hl;
+            const int other = (lane & ~(LP - 1)) + (l < 2 * hl ? (l < hl ? l + hl : l - hl) : l);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) {
+                const float v2 = __shfl(e[k], other, 64);
+                if (turn) { const float2 q = ct[i0 * 8 + k]; e[k] = l < hl ? e[k] * q.x - v2 * q.y : e[k] * q.x + v2 * q.y; }
+            }
+            if (on)
+#pragma unroll
+                for (int k = 0; k < 8; ++k) ss += e[k] * e[k];
+        } else if (on) {
 #pragma unroll
             for (int k = 0; k < 4; ++k) {
                 const int i = l * 4 + k;
@@ -282,7 +318,7 @@ __global__ __launch_bounds__(256) void qkv_rope8_kernel(QkvRopeArgs a, Batch b) 
             *reinterpret_cast<uint4 *>(isq ? src : (bf16_t *)a.kc + (row * a.G + h) * D + l * 8) = o;
         }
     }
-    const int GV = a.G * a.Dv;
+    const int GV = (a.Gv > 0 ? a.Gv : a.G) * a.Dv;
     bf16_t *vc = (bf16_t *)a.vc;
     const int64_t grp = ((int64_t)blk * (b.block_size >> 3) + (jj >> 3)) * GV;
     const float lam = a.v_first ? *a.lambda : 0.f;
@@ -330,11 +366,11 @@ void step4(const StreamArgs &a, hipStream_t s) {
     else stream_step4_kernel<S, 256, 8, KIND><<<grid, dim3(256), 0, s>>>(a);
 }
 
-template <int LP>
+template <int LP, bool HALVES>
 void rope8(const QkvRopeArgs &a, const Batch &b, hipStream_t s) {
     const size_t lds = (size_t)std::max(a.rot / 2, 1) * sizeof(float2);
-    if (b.T >= 1024) qkv_rope8_kernel<LP, 4><<<dim3((unsigned)((b.T + 3) / 4)), dim3(256), 4 * lds, s>>>(a, b);
-    else qkv_rope8_kernel<LP, 1><<<dim3((unsigned)b.T), dim3(256), lds, s>>>(a, b);
+    if (b.T >= 1024) qkv_rope8_kernel<LP, 4, HALVES><<<dim3((unsigned)((b.T + 3) / 4)), dim3(256), 4 * lds, s>>>(a, b);
+    else qkv_rope8_kernel<LP, 1, HALVES><<<dim3((unsigned)b.T), dim3(256), lds, s>>>(a, b);
 }
 
 }  // namespace
@@ -372,10 +408,12 @@ int qkv_rope_store(const QkvRopeArgs &a, const Batch &b, bool bf16, hipStream_t 
     if (a.v_grouped && b.block_size % 8) return nvr::fail(NVR_ERR_INVALID_ARG, "qkv_rope_store: grouped value pages need pages of a multiple of 8 tokens");
     if (a.v_first && !a.lambda) return nvr::fail(NVR_ERR_INVALID_ARG, "qkv_rope_store: values to mix without their share");
     if ((size_t)a.rot * 4 > 60000) return nvr::fail(NVR_ERR_UNSUPPORTED, "qkv_rope_store: %d rotated coordinates", a.rot);
-    const bool vec = bf16 && a.pairs && a.D % 8 == 0 && a.Dv % 8 == 0 && a.D <= 512 && a.ld % 8 == 0 && ((a.qcol | a.kcol | a.vcol) & 7) == 0 && a.rot <= 1024 &&
-                     aligned16(a.proj) && aligned16(a.kc) && aligned16(a.vc) && aligned16(a.bq) && aligned16(a.bk) && aligned16(a.bv) && aligned16(a.v_first) && aligned16(a.v_keep);
+    const bool vec = bf16 && (a.pairs || a.rot % 16 == 0) && a.D % 8 == 0 && a.Dv % 8 == 0 && a.D <= 512 && a.ld % 8 == 0 && ((a.qcol | a.kcol | a.vcol) & 7) == 0 && a.rot <= 1024 &&
+                     aligned16(a.proj) && aligned16(a.kc) && aligned16(a.vc) && aligned16(a.bq) && aligned16(a.bk) && aligned16(a.bv) && aligned16(a.v_first) && aligned16(a.v_keep) && aligned16(a.wq) && aligned16(a.wk);
     if (vec) {
-        if (a.D <= 32) rope8<4>(a, b, s); else if (a.D <= 64) rope8<8>(a, b, s); else if (a.D <= 128) rope8<16>(a, b, s); else if (a.D <= 256) rope8<32>(a, b, s); else rope8<64>(a, b, s);
+#define NVR_ROPE8(LP_) do { if (a.pairs) rope8<LP_, false>(a, b, s); else rope8<LP_, true>(a, b, s); } while (0)
+        if (a.D <= 32) NVR_ROPE8(4); else if (a.D <= 64) NVR_ROPE8(8); else if (a.D <= 128) NVR_ROPE8(16); else if (a.D <= 256) NVR_ROPE8(32); else NVR_ROPE8(64);
+#undef NVR_ROPE8
         return launched("qkv_rope_store");
     }
     const size_t lds = (size_t)std::max(a.rot, 2) * 4;

@@ -49,7 +49,7 @@ int LayeredModel::init_joint(nvr_model_runner &r) {
             if (std::find(attn_groups.begin(), attn_groups.end(), L.heads / L.kv_heads) == attn_groups.end()) attn_groups.push_back(L.heads / L.kv_heads);
             // prompts and portions on the dense graph's flash kernel in its gated form (row-major value pages)
             w.flash = bf16 && L.dim == L.vdim && nvr::kb::flash_prefill_ok((int)L.dim, (int)L.heads, (int)L.kv_heads) && hv % 8 == 0;
-            if (w.flash && std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) == flash_groups.end()) flash_groups.push_back(L.heads / L.kv_heads);
+            if (w.flash) flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
             max_cat = std::max(max_cat, hv); max_ro = std::max(max_ro, tn); max_t4 = std::max(max_t4, 4 * tn); max_tn = std::max(max_tn, tn);
         } else return fail(NVR_ERR_UNSUPPORTED, "layer %zu: this mixer does not belong to the joint layout", i);
         RC(named(&w.mix, (size_t)(w.nmix * W * esz)));         // (freed by name with the model)
@@ -258,7 +258,7 @@ int LayeredModel::forward_joint(nvr_model_runner &r, const StepPlan &p) {
             ra.rot = (int32_t)L.rot_dims; ra.freq = w.rfreq; ra.kc = st.kc; ra.vc = st.vc; ra.v_grouped = tiled && !w.flash;
             RC(kl::rope_store(ra, b, bf16, s));
             if (w.flash && !p.decode_sized) {
-                const size_t gi = (size_t)(std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) - flash_groups.begin());
+                const size_t gi = flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
                 nvr::kt::FlashArgs f{};
                 f.q = (const uint16_t *)a.q; f.ldq = w.nmix; f.k = (const uint16_t *)st.kc; f.v = (const uint16_t *)st.vc; f.ldkv = 0;
                 f.block_tables = b.block_tables; f.max_blocks = b.max_blocks; f.block_size = b.block_size;

@@ -36,7 +36,45 @@ inline float f16_to_f(uint16_t h) {
 inline float src_at(int dtype, const void *src, size_t i) {
     return dtype == 2 ? ((const float *)src)[i] : dtype == 1 ? bf16_to_f(((const uint16_t *)src)[i]) : f16_to_f(((const uint16_t *)src)[i]);
 }
+inline int64_t pad16(int64_t n) { return (n + 15) / 16 * 16; }
 }  // namespace
+
+// Stretch by wavelength: kept for wavelengths below original / high, divided by factor above original / low, blended linearly in original / wavelength between.  Stretch by index:
+// the index where a wavelength fits the original length `turns` times is dims ln(original / (2 pi turns)) / (2 ln base); kept up to the one for `fast`, divided by factor from the
+// one for `slow` on (both rounded outwards), blended linearly in the index between.
+std::vector<float> rotation_frequencies(const LayeredSpec::Layer &L, float *gain) {
+    std::vector<float> f((size_t)std::max<int64_t>(L.rot_dims / 2, 1));
+    const bool by_index = L.rot_original > 0 && L.rot_fast > 0;
+    double lo = 0, hi = 0;
+    if (by_index) {
+        auto index = [&](double turns) { return (double)L.rot_dims * std::log(L.rot_original / (2.0 * M_PI * turns)) / (2.0 * std::log(L.rot_base)); };
+        lo = std::max(std::floor(index(L.rot_fast)), 0.0); hi = std::min(std::ceil(index(L.rot_slow)), (double)L.rot_dims - 1.0);
+    }
+    for (int64_t j = 0; j < L.rot_dims / 2; ++j) {
+        double v = std::pow(L.rot_base, -2.0 * (double)j / (double)L.rot_dims);
+        if (by_index) {
+            const double ramp = std::min(std::max(((double)j - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            v = v / L.rot_factor * ramp + v * (1.0 - ramp);
+        } else if (L.rot_original > 0) {
+            const double wave = 2.0 * M_PI / v;
+            if (wave > L.rot_original / L.rot_low) v /= L.rot_factor;
+            else if (!(wave < L.rot_original / L.rot_high)) {
+                const double s = L.rot_high > L.rot_low ? (L.rot_original / wave - L.rot_low) / (L.rot_high - L.rot_low) : 1.0;
+                v = (1.0 - s) * v / L.rot_factor + s * v;
+            }
+        }
+        f[(size_t)j] = (float)v;
+    }
+    if (gain) *gain = by_index ? (float)(0.1 * std::log(L.rot_factor) + 1.0) : 1.f;
+    return f;
+}
+
+size_t LayeredModel::flash_kind(int64_t positions, bool rows) {
+    const FlashKind k{positions, rows};
+    const size_t i = (size_t)(std::find(flash_kinds.begin(), flash_kinds.end(), k) - flash_kinds.begin());
+    if (i == flash_kinds.size()) flash_kinds.push_back(k);
+    return i;
+}
 
 LayeredModel::~LayeredModel() {
     for (auto &g : graphs) if (g.second) (void)hipGraphExecDestroy(g.second);
@@ -96,7 +134,7 @@ int LayeredModel::init(nvr_model_runner &r) {
         if (L.mixer == LayeredSpec::ATTENTION) {
             if (std::find(attn_groups.begin(), attn_groups.end(), L.heads / L.kv_heads) == attn_groups.end()) attn_groups.push_back(L.heads / L.kv_heads);
             w.flash = bf16 && L.dim == L.vdim && nvr::kb::flash_prefill_ok((int)L.dim, (int)L.heads, (int)L.kv_heads) && w.nmix % 8 == 0 && w.kcat % 4 == 0;
-            if (w.flash && std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) == flash_groups.end()) flash_groups.push_back(L.heads / L.kv_heads);
+            if (w.flash) flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
             for (float **p : {&w.r1, &w.r2, &w.sink}) { RC(dmalloc(p, (size_t)L.heads * 4)); NVR_HIP_CHECK(hipMemset(*p, 0, (size_t)L.heads * 4)); }
         } else {
             std::vector<float> d(L.heads);
@@ -165,7 +203,7 @@ int LayeredModel::init(nvr_model_runner &r) {
 
     // step inputs: ids | row_seq | want | cu | start | slot | par | context lengths | block tables
     in_bytes = (size_t)(MT * 8 + MT * 4 * 2 + (r.max_seqs + 1) * 4 + r.max_seqs * 4 * 4 + r.max_seqs * r.max_blocks_per_seq * 4 + 256) +
-               (attn_groups.size() + 2 * flash_groups.size()) * (size_t)((MT + r.max_seqs) * sizeof(kl::AttnTile) + 16);
+               (attn_groups.size() + 2 * flash_kinds.size()) * (size_t)((MT + r.max_seqs) * sizeof(kl::AttnTile) + 16);
     attn_ws_bytes = kl::sink_attention_workspace_bytes(4 * r.num_cus);
     NVR_HIP_CHECK(hipMalloc(&attn_ws, attn_ws_bytes));
     NVR_HIP_CHECK(hipHostMalloc((void **)&in_host, in_bytes, hipHostMallocDefault));
@@ -300,21 +338,21 @@ int LayeredModel::execute(nvr_model_runner &r, nvr_seq *const *seqs, size_t nseq
         for (size_t i = 0; i < nseq; ++i) cnt += (seqs[i]->chunk_len + (size_t)pw - 1) / (size_t)pw;
         o_tiles[gi] = carve(cnt * sizeof(kl::AttnTile)); n_tiles[gi] = (int32_t)cnt;
     }
-    std::vector<size_t> o_ftiles(flash_groups.size()); std::vector<int32_t> n_ftiles(flash_groups.size(), 0);
-    for (size_t gi = 0; gi < flash_groups.size(); ++gi) {
-        const int64_t pw = nvr::kb::flash_tile_positions((int)flash_groups[gi], 1);
+    std::vector<size_t> o_ftiles(flash_kinds.size()); std::vector<int32_t> n_ftiles(flash_kinds.size(), 0);
+    for (size_t k = 0; k < flash_kinds.size(); ++k) {
+        const int64_t pw = flash_kinds[k].positions;
         size_t cnt = 0;
         for (size_t i = 0; i < nseq; ++i) cnt += (seqs[i]->chunk_len + (size_t)pw - 1) / (size_t)pw;
-        o_ftiles[gi] = carve(cnt * sizeof(nvr::kt::FlashTile)); n_ftiles[gi] = (int32_t)cnt;
+        o_ftiles[k] = carve(cnt * sizeof(nvr::kt::FlashTile)); n_ftiles[k] = (int32_t)cnt;
     }
     if (off > in_bytes) return fail(NVR_ERR_INVARIANT, "execute_model: step inputs of %zu bytes exceed the arena", off);
-    for (size_t gi = 0; gi < flash_groups.size(); ++gi) {
-        const int64_t pw = nvr::kb::flash_tile_positions((int)flash_groups[gi], 1);
-        nvr::kt::FlashTile *tl = (nvr::kt::FlashTile *)(in_host + o_ftiles[gi]);
+    for (size_t k = 0; k < flash_kinds.size(); ++k) {
+        const int64_t pw = flash_kinds[k].positions;
+        nvr::kt::FlashTile *tl = (nvr::kt::FlashTile *)(in_host + o_ftiles[k]);
         int64_t row = 0;
         for (size_t i = 0; i < nseq; ++i) {
             for (int64_t r0 = 0; r0 < (int64_t)seqs[i]->chunk_len; r0 += pw)
-                *tl++ = nvr::kt::FlashTile{(int32_t)(row + r0), (int32_t)std::min<int64_t>(pw, (int64_t)seqs[i]->chunk_len - r0), (int32_t)((int64_t)seqs[i]->chunk_start + r0), flash_contiguous ? (int32_t)row : (int32_t)i};
+                *tl++ = nvr::kt::FlashTile{(int32_t)(row + r0), (int32_t)std::min<int64_t>(pw, (int64_t)seqs[i]->chunk_len - r0), (int32_t)((int64_t)seqs[i]->chunk_start + r0), flash_kinds[k].rows ? (int32_t)row : (int32_t)i};
             row += (int64_t)seqs[i]->chunk_len;
         }
     }
@@ -419,7 +457,7 @@ int LayeredModel::forward(nvr_model_runner &r, const StepPlan &p) {
             RC(kl::kv_store(proj, w.nmix, w.kcol, w.vcol, b, L.kv_heads, L.dim, L.vdim, st.kc, st.vc, bf16, tiled && !w.flash, s));
             if (w.flash && !p.decode_sized) {
                 // prompts and portions: the dense graph's flash kernel in its penalty / sink form (K and V through the block tables, the step's own rows included)
-                const size_t gi = (size_t)(std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) - flash_groups.begin());
+                const size_t gi = flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
                 nvr::kt::FlashArgs f{};
                 f.q = (const uint16_t *)a.q; f.ldq = w.nmix; f.k = (const uint16_t *)st.kc; f.v = (const uint16_t *)st.vc; f.ldkv = 0;
                 f.block_tables = b.block_tables; f.max_blocks = b.max_blocks; f.block_size = b.block_size;
@@ -463,7 +501,7 @@ int LayeredModel::forward(nvr_model_runner &r, const StepPlan &p) {
 }
 
 // ===================================================================================================================================================
-// Sequential layout: x <- x + nb(mixer(n(x))); x <- x + nb(ff(n(x))); token input; weighted average over depth.
+// Sequential layout: x <- x + nb(mixer(n(x))); x <- x + nb(ff(n(x))); token input; where the design has one, a weighted average over depth.
 
 int LayeredModel::init_sequential(nvr_model_runner &r) {
     const int64_t W = spec.width, V = spec.vocab, MT = r.max_tokens, nL = (int64_t)spec.layers.size();
@@ -473,7 +511,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
         return (int)NVR_OK;
     };
     lw.resize(spec.layers.size());
-    int64_t max_kvx = 0, max_experts = 0, max_f = 0;
+    int64_t max_kvx = 0, max_experts = 0, max_f = 0, max_maps = 0;
     int64_t max_nmix = 0, max_q2 = 0, max_qabs = 0, max_ctx = 0, max_hv = 0, max_qlat = 0, max_hd = 0, max_ff = 0, max_rows_e = 0, max_e2f = 0, max_ef = 0;
     size_t block_bytes = 0;
     for (size_t i = 0; i < spec.layers.size(); ++i) {
@@ -483,18 +521,18 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
         if (L.has_mlp) for (float **p : {&w.n2, &w.n2b}) RC(own(p, (size_t)W * 4));
         if (L.mixer == LayeredSpec::LATENT) {
             const int64_t R = L.rot_dim, own_kv = L.kv_from < 0 ? L.kv_rank + R : 0;
-            // mix rows: queries (or their latent), the output gate's rows, the cached row's source
-            w.qcol = 0; const int64_t qn = L.q_rank ? L.q_rank : hd;
-            w.gcol = qn; w.dcol = qn + (L.out_gate ? hv : 0); w.nmix = w.dcol + own_kv;
+            // mix rows: queries (or their latent), the output gate's rows, the cached row's source; segments at multiples of 16 rows
+            w.qcol = 0; const int64_t qn = L.q_rank ? L.q_rank : L.heads * (L.dim + R);
+            w.gcol = pad16(qn); w.dcol = w.gcol + (L.out_gate ? pad16(hv) : 0); w.nmix = w.dcol + pad16(own_kv);
+            if (L.sink) RC(named((void **)&w.sink, (size_t)L.heads * 4));
             if (L.q_rank) { RC(own(&w.uq, (size_t)(L.heads * (L.dim + R) * L.q_rank * esz))); RC(own(&w.dqn, (size_t)L.q_rank * 4)); max_q2 = std::max(max_q2, L.heads * (L.dim + R)); max_qlat = std::max(max_qlat, L.q_rank); }
             if (own_kv) { RC(own(&w.dkvn, (size_t)L.kv_rank * 4)); block_bytes += (size_t)(r.block_size * own_kv * esz); }
             RC(own(&w.ukt, (size_t)(L.heads * L.kv_rank * L.dim * esz))); RC(own(&w.uv, (size_t)(hv * L.kv_rank * esz)));
-            std::vector<float> f((size_t)std::max<int64_t>(R / 2, 1));
-            for (int64_t j = 0; j < R / 2; ++j) f[(size_t)j] = (float)std::pow(L.rot_base, -2.0 * (double)j / (double)L.rot_dims);
+            const std::vector<float> f = rotation_frequencies(L, &w.rot_gain);
             RC(own(&w.rfreq, f.size() * 4)); NVR_HIP_CHECK(hipMemcpy(w.rfreq, f.data(), f.size() * 4, hipMemcpyHostToDevice));
             max_qabs = std::max(max_qabs, L.heads * (L.kv_rank + R)); max_ctx = std::max(max_ctx, L.heads * L.kv_rank);
             // whole prompts (every key is a row of the step): keys and values expanded by one product and the dense graph's flash kernel, one key/value head per query head
-            w.flash = bf16 && L.dim + R == L.vdim && nvr::kb::flash_prefill_ok((int)L.vdim, (int)L.heads, (int)L.heads) && (L.kv_rank + R) % 32 == 0 && (2 * hv) % 16 == 0 &&
+            w.flash = bf16 && L.window == 0 && L.scale > 0 && L.dim + R == L.vdim && nvr::kb::flash_prefill_ok((int)L.vdim, (int)L.heads, (int)L.heads) && (L.kv_rank + R) % 32 == 0 && (2 * hv) % 16 == 0 &&
                       w.nmix % 8 == 0 && (L.heads * (L.dim + R)) % 8 == 0;
             if (w.flash) {
                 RC(own(&w.wx, (size_t)(2 * hv * (L.kv_rank + R) * esz)));
@@ -502,8 +540,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
                 for (int64_t h = 0; h < L.heads; ++h)           // the shared rotated key part is copied into every head's keys by rows of the identity
                     for (int64_t j = 0; j < R; ++j)
                         NVR_HIP_CHECK(hipMemcpy((char *)w.wx + (size_t)(((h * L.vdim + L.dim + j) * (L.kv_rank + R) + L.kv_rank + j) * esz), one.data(), 2, hipMemcpyHostToDevice));
-                if (std::find(flash_groups.begin(), flash_groups.end(), (int64_t)1) == flash_groups.end()) flash_groups.push_back(1);
-                flash_contiguous = true;
+                flash_kind(nvr::kb::flash_tile_positions(1, 1), true);
                 max_kvx = std::max(max_kvx, 2 * hv);
             }
             // the matrix-core attention takes up to 16 query heads per key/value row: the heads go in equal shares of the largest divisor of H up to 16
@@ -515,10 +552,29 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             w.qcol = 0; w.kcol = hd; w.vcol = 2 * hd; w.gcol = 2 * hd + hv; w.nmix = 2 * hd + 2 * hv;
             RC(own(&w.a2b, (size_t)hd * 4)); RC(own(&w.hnorm, (size_t)L.vdim * 4));
             max_hd = std::max(max_hd, hd);
+        } else if (L.mixer == LayeredSpec::ATTN_DIFF) {
+            // mix rows: queries [H][2][D], keys [G][2][D], values [G][Dv], one gate number per head; a key row of the pages holds both maps' keys
+            const int64_t kn = L.kv_heads * 2 * L.dim, vn = L.kv_heads * L.vdim;
+            w.qcol = 0; w.kcol = pad16(2 * hd); w.vcol = w.kcol + pad16(kn); w.gcol = w.vcol + pad16(vn); w.nmix = w.gcol + pad16(L.heads);
+            RC(own(&w.qn, (size_t)L.dim * 4)); RC(own(&w.kn, (size_t)L.dim * 4)); RC(own(&w.lambda, 4));
+            for (auto &v : w.lam) v.assign((size_t)L.dim, 0.f);
+            RC(diff_share(w, L));
+            const std::vector<float> f = rotation_frequencies(L, &w.rot_gain);
+            RC(own(&w.rfreq, f.size() * 4)); NVR_HIP_CHECK(hipMemcpy(w.rfreq, f.data(), f.size() * 4, hipMemcpyHostToDevice));
+            block_bytes += (size_t)(r.block_size * L.kv_heads * (2 * L.dim + L.vdim) * esz);
+            const int64_t g = 2 * L.heads / L.kv_heads;
+            if (std::find(attn_groups.begin(), attn_groups.end(), g) == attn_groups.end()) attn_groups.push_back(g);
+            // prompts and portions with values twice the size of a map's keys, key rows of 64 / 128 numbers: the flash kernel in its differential form
+            w.flash = bf16 && 2 * L.dim == L.vdim && L.scale > 0 && hv % 8 == 0 && nvr::kb::flash_diff_ok((int)L.vdim, (int)L.heads, (int)L.kv_heads);
+            if (w.flash) flash_kind(nvr::kb::flash_diff_tile_positions((int)L.heads, (int)L.kv_heads));
+            if (!kl::sink_attention_tiled_ok(diff_args(w, L), bf16, (int)r.block_size)) max_maps = std::max(max_maps, L.heads * 2 * L.vdim);
         } else return fail(NVR_ERR_UNSUPPORTED, "layer %zu: this mixer does not belong to the sequential layout", i);
         RC(named(&w.mix, (size_t)(w.nmix * W * esz))); RC(own(&w.wo, (size_t)(W * hv * esz)));
         if (L.ff_kind == LayeredSpec::FF_POLY) {
             RC(own(&w.up, (size_t)(L.ff * W * esz))); RC(own(&w.down, (size_t)(W * L.ff * esz))); RC(own(&w.act, 16));
+            max_ff = std::max(max_ff, L.ff);
+        } else if (L.ff_kind == LayeredSpec::FF_GELU) {
+            RC(own(&w.up, (size_t)(L.ff * W * esz))); RC(own(&w.down, (size_t)(W * L.ff * esz)));
             max_ff = std::max(max_ff, L.ff);
         } else if (L.ff_kind == LayeredSpec::FF_MOE) {
             const int64_t f = L.expert_ff, fs = L.shared_ff;
@@ -528,20 +584,25 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             max_ff = std::max(max_ff, 2 * fs); max_rows_e = std::max(max_rows_e, L.top); max_e2f = std::max(max_e2f, L.top * 2 * f); max_ef = std::max(max_ef, L.top * f); max_experts = std::max(max_experts, L.experts); max_f = std::max(max_f, f);
         } else if (L.has_mlp) return fail(NVR_ERR_UNSUPPORTED, "layer %zu: this feed-forward does not belong to the sequential layout", i);
         if (spec.side_dim) { RC(own(&w.sgate, (size_t)(spec.side_dim * W * esz))); RC(own(&w.sproj, (size_t)(W * spec.side_dim * esz))); RC(own(&w.snorm, (size_t)W * 4)); }
-        RC(own(&w.dwa, (size_t)(i + 2) * 4));                   // (until loaded: the layer's own output passes)
-        { const float one = 1.f; NVR_HIP_CHECK(hipMemcpy(w.dwa + i + 1, &one, 4, hipMemcpyHostToDevice)); }
+        if (spec.depth_average) {
+            RC(own(&w.dwa, (size_t)(i + 2) * 4));               // (until loaded: the layer's own output passes)
+            const float one = 1.f;
+            NVR_HIP_CHECK(hipMemcpy(w.dwa + i + 1, &one, 4, hipMemcpyHostToDevice));
+        }
         max_nmix = std::max(max_nmix, w.nmix); max_hv = std::max(max_hv, hv);
     }
     RC(named(&embed, (size_t)(V * W * esz))); RC(named(&head, (size_t)(V * W * esz))); RC(own(&wfinal, (size_t)W * 4));
+    if (spec.max_positions) RC(own(&pos, (size_t)(spec.max_positions * W * esz)));
     if (spec.side_dim) RC(own(&side_embed, (size_t)(V * nL * spec.side_dim * esz)));
 
-    // pages: one row of kv_rank + rot_dim numbers per token for every latent-attention layer with a latent of its own; state per slot for gated linear attention
+    // pages: one row of kv_rank + rot_dim numbers per token for every latent-attention layer with a latent of its own, keys and values for every differential attention; state per
+    // slot for gated linear attention
     if (r.cfg.num_kvcache_blocks >= 0) r.num_blocks = r.cfg.num_kvcache_blocks;
     else if (r.cfg.num_kvcache_blocks == -1) r.num_blocks = 1000;
     else {
         size_t free_b = 0, total_b = 0;
         NVR_HIP_CHECK(hipMemGetInfo(&free_b, &total_b));
-        const double budget = (double)free_b - (1.0 - r.cfg.gpu_memory_utilization) * (double)total_b - (double)((nL + 8) * MT * W * 4);
+        const double budget = (double)free_b - (1.0 - r.cfg.gpu_memory_utilization) * (double)total_b - (double)(((spec.depth_average ? nL : 0) + 8) * MT * W * 4) - (double)(MT * (max_nmix + 2 * max_ff + max_qabs + max_ctx + max_kvx + 2 * max_maps) * esz);
         const int64_t nb = block_bytes ? (int64_t)(budget * 0.9 / (double)block_bytes) : 1000;
         if (nb < 1) return fail(NVR_ERR_HIP, "not enough free HBM for one KV block");
         r.num_blocks = nb;
@@ -553,6 +614,9 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             RC(named(&rs[i].kc, (size_t)(r.num_blocks * r.block_size * (L.kv_rank + L.rot_dim) * esz)));
             RC(own(&rs[i].rows, (size_t)(MT * (L.kv_rank + L.rot_dim) * esz)));                 // the step's own cached rows, in step order
         }
+        else if (L.mixer == LayeredSpec::ATTN_DIFF) {
+            RC(named(&rs[i].kc, (size_t)(r.num_blocks * r.block_size * L.kv_heads * 2 * L.dim * esz))); RC(named(&rs[i].vc, (size_t)(r.num_blocks * r.block_size * L.kv_heads * L.vdim * esz)));
+        }
         else if (L.mixer == LayeredSpec::GLA) RC(named((void **)&rs[i].state, (size_t)(slots * L.heads * L.dim * L.vdim * 4)));
     }
     for (size_t i = 0; i < spec.layers.size(); ++i) {                           // a layer without a latent of its own reads its source's pages
@@ -561,7 +625,9 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
     }
 
     // activations
-    RC(named((void **)&x, (size_t)(MT * W * 4))); RC(own(&kept, (size_t)((nL + 1) * MT * W * 4)));
+    RC(named((void **)&x, (size_t)(MT * W * 4)));
+    if (spec.depth_average) RC(own(&kept, (size_t)((nL + 1) * MT * W * 4)));
+    if (max_maps) RC(own(&maps_o, (size_t)(MT * max_maps * 4)));
     RC(named(&a1, (size_t)(MT * W * esz))); RC(named(&a2, (size_t)(MT * W * esz))); RC(named(&tmp, (size_t)(MT * W * esz)));
     RC(named(&proj, (size_t)(MT * max_nmix * esz))); RC(named(&cat, (size_t)(MT * max_hv * esz)));
     RC(own(&qlat, (size_t)(MT * max_qlat * esz))); RC(own(&q2, (size_t)(MT * max_q2 * esz))); RC(own(&qabs, (size_t)(MT * max_qabs * esz))); RC(own(&ctx, (size_t)(MT * max_ctx * esz)));
@@ -576,8 +642,26 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
     return NVR_OK;
 }
 
-// Tensors by the names of the checkpoint: "embed", "head", "final.norm" [W], "side.embed" [vocab][layers * side]; per layer i "l<i>.norm1" / "norm1b" / "norm2" / "norm2b" [W],
-// "l<i>.mix.*" (latent attention: q | dq, dq.norm, uq; dkv, dkv.norm; uk, uv; g; o — gated linear attention: q, k, v, g, o, norm, a1, a2, a2.b), "l<i>.mlp.*" (dense: up, down,
+// The share of differential attention's second map: exp(lq1 . lk1) - exp(lq2 . lk2) + the layer's fixed part.
+int LayeredModel::diff_share(LayerW &w, const LayeredSpec::Layer &L) {
+    double d1 = 0, d2 = 0;
+    for (size_t k = 0; k < w.lam[0].size(); ++k) { d1 += (double)w.lam[0][k] * w.lam[1][k]; d2 += (double)w.lam[2][k] * w.lam[3][k]; }
+    const float v = (float)(std::exp(d1) - std::exp(d2) + L.diff);
+    NVR_HIP_CHECK(hipMemcpy(w.lambda, &v, 4, hipMemcpyHostToDevice));
+    return NVR_OK;
+}
+
+// What a differential attention's launches have in common, without the step's pointers.
+kl::SinkAttnArgs LayeredModel::diff_args(const LayerW &w, const LayeredSpec::Layer &L) const {
+    kl::SinkAttnArgs a{};
+    a.ldq = w.nmix; a.H = (int32_t)L.heads; a.G = (int32_t)L.kv_heads; a.D = (int32_t)(2 * L.dim); a.Dv = (int32_t)L.vdim; a.scale = (float)L.scale; a.ldo = L.heads * L.vdim;
+    a.window = (int32_t)L.window; a.keep_first = (int32_t)L.keep_first; a.v_grouped = w.flash ? 0 : 1;      // (a property of the layer: the pages keep one layout)
+    a.lambda = w.lambda; a.out_scale = (float)(1.0 - L.diff); a.eps = (float)spec.eps; a.ldhg = w.nmix;
+    return a;
+}
+
+// Tensors by the names of the checkpoint: "embed", "head", "final.norm" [W], "pos" [positions][W], "side.embed" [vocab][layers * side]; per layer i "l<i>.norm1" / "norm1b" / "norm2" / "norm2b" [W],
+// "l<i>.mix.*" (latent attention: q | dq, dq.norm, uq; dkv, dkv.norm; uk, uv; sink; g; o — differential attention: q, k, v, g, o, q.norm, k.norm, lq1, lk1, lq2, lk2 — gated linear attention: q, k, v, g, o, norm, a1, a2, a2.b), "l<i>.mlp.*" (dense: up, down,
 // act — experts: router, e<j>.{gate,up,down}, shared.{gate,up,down}), "l<i>.side.{gate,proj,norm}", "l<i>.dwa" [i + 2].  Linear weights are [out][in].
 int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data) {
     const int64_t W = spec.width, V = spec.vocab, nL = (int64_t)spec.layers.size();
@@ -591,6 +675,7 @@ int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, 
     if (name == "embed") return mat(embed, W, V, W);
     if (name == "head") return mat(head, W, V, W);
     if (name == "final.norm") return vec(wfinal, W);
+    if (name == "pos" && spec.max_positions) return mat(pos, W, spec.max_positions, W);
     if (name == "side.embed") return spec.side_dim ? mat(side_embed, nL * spec.side_dim, V, nL * spec.side_dim) : unknown();
     size_t dot = name.find('.');
     if (name.size() < 3 || name[0] != 'l' || dot == std::string::npos || dot < 2) return unknown();
@@ -604,7 +689,7 @@ int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, 
     if (rest == "norm1b") return vec(w.n1b, W);
     if (rest == "norm2") return L.has_mlp ? vec(w.n2, W) : unknown();
     if (rest == "norm2b") return L.has_mlp ? vec(w.n2b, W) : unknown();
-    if (rest == "dwa") return vec(w.dwa, li + 2);
+    if (rest == "dwa" && spec.depth_average) return vec(w.dwa, li + 2);
     if (spec.side_dim) {
         if (rest == "side.gate") return mat(w.sgate, W, spec.side_dim, W);
         if (rest == "side.proj") return mat(w.sproj, spec.side_dim, W, spec.side_dim);
@@ -612,7 +697,8 @@ int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, 
     }
     if (rest == "mix.o") return mat(w.wo, hv, W, hv);
     if (L.mixer == LayeredSpec::LATENT) {
-        if (rest == "mix.q" && !L.q_rank) return mat(w.mix, W, hd, W);
+        if (rest == "mix.q" && !L.q_rank) return mat(w.mix, W, L.heads * (L.dim + R), W);
+        if (rest == "mix.sink" && L.sink) return vec(w.sink, L.heads);
         if (rest == "mix.dq" && L.q_rank) return mat(w.mix, W, L.q_rank, W);
         if (rest == "mix.dq.norm" && L.q_rank) return vec(w.dqn, L.q_rank);
         if (rest == "mix.uq" && L.q_rank) return mat(w.uq, L.q_rank, L.heads * (L.dim + R), L.q_rank);
@@ -635,6 +721,22 @@ int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, 
                            (const char *)data + (size_t)(h * L.dim * L.kv_rank) * (dtype == 2 ? 4 : 2), true));
             return put(r, w.ukt, L.dim, L.heads * L.kv_rank, L.dim, 2, t.data(), true);
         }
+    } else if (L.mixer == LayeredSpec::ATTN_DIFF) {
+        const int64_t D = L.dim;
+        if (rest == "mix.q") return mat(rows_at(w.mix, w.qcol, W), W, 2 * hd, W);
+        if (rest == "mix.k") return mat(rows_at(w.mix, w.kcol, W), W, L.kv_heads * 2 * D, W);
+        if (rest == "mix.v") return mat(rows_at(w.mix, w.vcol, W), W, L.kv_heads * L.vdim, W);
+        if (rest == "mix.g") return mat(rows_at(w.mix, w.gcol, W), W, L.heads, W);
+        if (rest == "mix.q.norm") return vec(w.qn, D);
+        if (rest == "mix.k.norm") return vec(w.kn, D);
+        static const char *const parts[4] = {"mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"};
+        for (int k = 0; k < 4; ++k)
+            if (rest == parts[k]) {
+                if (ndim != 1 || shape[0] != D) return bad();
+                for (int64_t d = 0; d < D; ++d) w.lam[k][(size_t)d] = src_at(dtype, data, (size_t)d);
+                NVR_HIP_CHECK(hipSetDevice(r.device));
+                return diff_share(w, L);
+            }
     } else {
         if (rest == "mix.q") return mat(rows_at(w.mix, w.qcol, W), W, hd, W);
         if (rest == "mix.k") return mat(rows_at(w.mix, w.kcol, W), W, hd, W);
@@ -660,6 +762,9 @@ int LayeredModel::load_sequential(nvr_model_runner &r, const std::string &name, 
         if (rest == "mlp.up") return mat(w.up, W, L.ff, W);
         if (rest == "mlp.down") return mat(w.down, L.ff, W, L.ff);
         if (rest == "mlp.act") return vec(w.act, 4);
+    } else if (L.ff_kind == LayeredSpec::FF_GELU) {
+        if (rest == "mlp.up") return mat(w.up, W, L.ff, W);
+        if (rest == "mlp.down") return mat(w.down, L.ff, W, L.ff);
     } else if (L.ff_kind == LayeredSpec::FF_MOE) {
         const int64_t f = L.expert_ff, fs = L.shared_ff;
         if (rest == "mlp.router") return (is2(L.experts, W)) ? put(r, w.router, W, L.experts, W, dtype, data, false) : bad();
@@ -687,7 +792,8 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
     const float eps = (float)spec.eps; const int groups = (int)spec.norm_groups;
     hipStream_t s = r.stream;
     auto at = [&](void *base, int64_t col) { return (void *)((char *)base + (size_t)(col * esz)); };
-    RC(kl::embed_keep(embed, bf16, b.ids, T, W, x, kept, s));
+    if (pos) RC(kl::embed_pos(embed, pos, bf16, b, W, (float)spec.embedding_scale, x, s));
+    else RC(kl::embed_keep(embed, bf16, b.ids, T, W, x, kept, s));
     {   // the first layer's input; every later one leaves the end of the layer before it
         kl::GroupNormArgs n{}; n.in = x; n.ldi = W; n.in_f32 = true; n.rows_n = T; n.W = W; n.groups = groups; n.eps = eps; n.w = lw[0].n1; n.out = a1; n.ldo = W;
         RC(kl::group_norm(n, bf16, s));
@@ -698,23 +804,23 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
         RC(gemm(r, a1, W, w.mix, T, W, w.nmix, proj));
         if (L.mixer == LayeredSpec::LATENT) {
             const int64_t Rr = L.rot_dim, rank = L.kv_rank, Dq = rank + Rr;
-            const void *qsrc = proj; int64_t ldq = w.nmix, qstride = L.dim;
+            const void *qsrc = proj; int64_t ldq = w.nmix, qstride = L.dim + Rr;
             if (L.q_rank) {                                 // queries through their own normed latent
                 kl::GroupNormArgs n{}; n.in = proj; n.ldi = w.nmix; n.rows_n = T; n.W = L.q_rank; n.groups = 1; n.eps = eps; n.w = w.dqn; n.out = qlat; n.ldo = L.q_rank;
                 RC(kl::group_norm(n, bf16, s));
                 RC(gemm(r, qlat, L.q_rank, w.uq, T, L.q_rank, L.heads * (L.dim + Rr), q2));
                 qsrc = q2; ldq = L.heads * (L.dim + Rr); qstride = L.dim + Rr;
             }
-            if (L.kv_from < 0) RC(kl::latent_store(proj, w.nmix, w.dcol, b, rank, Rr, eps, w.dkvn, w.rfreq, st.kc, st.rows, bf16, s));
+            if (L.kv_from < 0) RC(kl::latent_store(proj, w.nmix, w.dcol, b, rank, Rr, eps, w.dkvn, w.rfreq, st.kc, st.rows, bf16, s, L.rot_halves, w.rot_gain));
             if (w.flash && p.whole_prompts) {
                 // every key is a row of this step: K (with the rotated part) and V of all heads by one product from the step's cached rows, then the flash kernel
-                RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, (void *)qsrc, ldq, qstride, L.dim, bf16, s));   // (in place: a thread reads a pair, then writes it)
+                RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, (void *)qsrc, ldq, qstride, L.dim, bf16, s, L.rot_halves, w.rot_gain));   // (in place: a thread reads a pair, then writes it)
                 RC(gemm(r, st.rows, Dq, w.wx, T, Dq, 2 * hv, kvx));
-                const size_t gi = (size_t)(std::find(flash_groups.begin(), flash_groups.end(), (int64_t)1) - flash_groups.begin());
+                const size_t gi = flash_kind(nvr::kb::flash_tile_positions(1, 1), true);
                 nvr::kt::FlashArgs f{};
                 f.q = (const uint16_t *)qsrc; f.ldq = ldq; f.k = (const uint16_t *)kvx; f.v = (const uint16_t *)kvx + hv; f.ldkv = 2 * hv;
                 f.tiles = (const nvr::kt::FlashTile *)(in_dev + p.o_ftiles[gi]); f.ntiles = p.n_ftiles[gi];
-                f.H = (int32_t)L.heads; f.KVH = (int32_t)L.heads; f.D = (int32_t)L.vdim; f.scale = (float)L.scale; f.out = (uint16_t *)cat; f.ldo = hv;
+                f.H = (int32_t)L.heads; f.KVH = (int32_t)L.heads; f.D = (int32_t)L.vdim; f.scale = (float)L.scale; f.out = (uint16_t *)cat; f.ldo = hv; f.sink = w.sink;
                 RC(nvr::kb::flash_prefill(f, false, s));
                 if (L.out_gate) RC(kl::sigmoid_gate(cat, hv, at(proj, w.gcol), w.nmix, T, hv, bf16, s));
             } else {
@@ -722,10 +828,10 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             kl::HeadLinearArgs ha{}; ha.a = qsrc; ha.lda = ldq; ha.ha = qstride; ha.w = w.ukt; ha.y = qabs; ha.ldy = L.heads * Dq; ha.hy = Dq;
             ha.T = (int32_t)T; ha.H = (int32_t)L.heads; ha.K = (int32_t)L.dim; ha.N = (int32_t)rank;
             RC(kl::head_linear(ha, bf16, s));
-            RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, qabs, L.heads * Dq, Dq, rank, bf16, s));
+            RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, qabs, L.heads * Dq, Dq, rank, bf16, s, L.rot_halves, w.rot_gain));
             kl::SinkAttnArgs a{};
             a.q = qabs; a.ldq = L.heads * Dq; a.kc = st.kc; a.vc = st.kc; a.vld = Dq; a.H = (int32_t)L.heads; a.G = 1; a.D = (int32_t)Dq; a.Dv = (int32_t)rank;
-            a.scale = (float)L.scale; a.out = ctx; a.ldo = L.heads * rank;
+            a.scale = (float)L.scale; a.out = ctx; a.ldo = L.heads * rank; a.sink = w.sink; a.window = (int32_t)L.window; a.keep_first = (int32_t)L.keep_first;
             kl::SinkAttnArgs a1s = a; a1s.H = (int32_t)w.head_share;
             if (kl::sink_attention_tiled_ok(a1s, bf16, (int)r.block_size)) {
                 const size_t gi = (size_t)(std::find(attn_groups.begin(), attn_groups.end(), w.head_share) - attn_groups.begin());
@@ -736,6 +842,7 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
                 for (int64_t h0 = 0; h0 < L.heads; h0 += w.head_share) {       // one launch per share of the heads, all on the same cached rows
                     kl::SinkAttnArgs as = a1s;
                     as.q = (const char *)qabs + (size_t)(h0 * Dq * esz); as.out = (char *)ctx + (size_t)(h0 * rank * esz);
+                    if (w.sink) as.sink = w.sink + h0;
                     RC(kl::sink_attention_tiled(as, b, (const kl::AttnTile *)(in_dev + p.o_tiles[gi]), p.n_tiles[gi], (int)nsplit, (char *)attn_ws + (size_t)(h0 / w.head_share) * share_ws, share_ws, s));
                 }
             } else
@@ -746,6 +853,32 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             if (L.out_gate) { hu.gate = at(proj, w.gcol); hu.ldg = w.nmix; hu.hg = L.vdim; }
             RC(kl::head_linear(hu, bf16, s));
             }
+        } else if (L.mixer == LayeredSpec::ATTN_DIFF) {
+            kl::SinkAttnArgs a = diff_args(w, L);
+            a.q = at(proj, w.qcol); a.kc = st.kc; a.vc = st.vc; a.out = cat; a.head_gate = at(proj, w.gcol); a.maps_o = maps_o;
+            const bool tiled = kl::sink_attention_tiled_ok(a, bf16, (int)r.block_size);
+            kl::QkvRopeArgs qa{};                           // (a map counts as a head)
+            qa.proj = proj; qa.ld = w.nmix; qa.qcol = w.qcol; qa.kcol = w.kcol; qa.vcol = w.vcol; qa.H = 2 * a.H; qa.G = 2 * a.G; qa.D = (int32_t)L.dim; qa.Dv = a.Dv; qa.Gv = a.G;
+            qa.rot = (int32_t)L.rot_dims; qa.freq = w.rfreq; qa.pairs = !L.rot_halves; qa.gain = w.rot_gain; qa.wq = w.qn; qa.wk = w.kn; qa.eps = eps;
+            qa.kc = st.kc; qa.vc = st.vc; qa.v_grouped = tiled && !w.flash;
+            RC(kl::qkv_rope_store(qa, b, bf16, s));
+            if (w.flash && !p.decode_sized) {
+                const size_t gi = flash_kind(nvr::kb::flash_diff_tile_positions((int)L.heads, (int)L.kv_heads));
+                nvr::kt::FlashArgs f{};
+                f.q = (const uint16_t *)a.q; f.ldq = w.nmix; f.k = (const uint16_t *)st.kc; f.v = (const uint16_t *)st.vc; f.ldkv = 0;
+                f.block_tables = b.block_tables; f.max_blocks = b.max_blocks; f.block_size = b.block_size;
+                f.tiles = (const nvr::kt::FlashTile *)(in_dev + p.o_ftiles[gi]); f.ntiles = p.n_ftiles[gi];
+                f.H = a.H; f.KVH = a.G; f.D = a.Dv; f.scale = a.scale; f.out = (uint16_t *)cat; f.ldo = hv; f.window = a.window; f.keep_first = a.keep_first;
+                f.lambda = a.lambda; f.out_scale = a.out_scale; f.eps = a.eps; f.head_gate = (const uint16_t *)a.head_gate; f.ldhg = a.ldhg;
+                RC(nvr::kb::flash_prefill(f, true, s));
+            } else if (tiled) {
+                const size_t gi = (size_t)(std::find(attn_groups.begin(), attn_groups.end(), 2 * L.heads / L.kv_heads) - attn_groups.begin());
+                const int64_t wgs = (int64_t)p.n_tiles[gi] * L.kv_heads, keys = L.window > 0 ? std::min<int64_t>(p.max_ctx, L.window + L.keep_first + 64) : p.max_ctx;
+                int64_t nsplit = 1;
+                if (wgs < r.num_cus && keys >= 512) nsplit = std::max<int64_t>(1, std::min<int64_t>({(2 * r.num_cus) / wgs, (keys + 255) / 256, 16}));
+                RC(kl::sink_attention_tiled(a, b, (const kl::AttnTile *)(in_dev + p.o_tiles[gi]), p.n_tiles[gi], (int)nsplit, attn_ws, attn_ws_bytes, s));
+            } else
+                RC(kl::sink_attention(a, b, bf16, s));
         } else {
             if (!w.wa1 || !w.wa2) return fail(NVR_ERR_NOT_ALLOCATED, "layer %ld: the decay projections were not loaded", (long)i);
             RC(gemm(r, a1, W, w.wa1, T, W, w.a_rank, alow));
@@ -767,6 +900,13 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
         if (L.ff_kind == LayeredSpec::FF_POLY) {
             RC(gemm(r, a2, W, w.up, T, W, L.ff, gu));
             RC(kl::poly_norm(gu, L.ff, T, L.ff, eps, w.act, act, L.ff, bf16, s));
+            RC(gemm(r, act, L.ff, w.down, T, L.ff, W, tmp));
+        } else if (L.ff_kind == LayeredSpec::FF_GELU) {
+            if (bf16 && nvr::kb::gemm256_preferred(T, W, L.ff, W)) RC(nvr::kb::gemm256_gelu((const uint16_t *)a2, W, (const uint16_t *)w.up, T, W, L.ff, (uint16_t *)act, s));   // (GELU in the product's epilogue)
+            else {
+                RC(gemm(r, a2, W, w.up, T, W, L.ff, gu));
+                RC(kl::gelu_erf(gu, L.ff, T, L.ff, act, L.ff, bf16, s));
+            }
             RC(gemm(r, act, L.ff, w.down, T, L.ff, W, tmp));
         } else if (L.ff_kind == LayeredSpec::FF_MOE) {
             const int64_t f = L.expert_ff, fs = L.shared_ff, n = T * L.top;
@@ -809,7 +949,7 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             RC(gemm(r, side_g, spec.side_dim, w.sproj, T, spec.side_dim, W, tmp));
             t.side_y = tmp; t.side_norm = w.snorm;
         }
-        t.kept = kept; t.kept_rows = MT; t.nx = (int32_t)(i + 2); t.mix = w.dwa;
+        if (spec.depth_average) { t.kept = kept; t.kept_rows = MT; t.nx = (int32_t)(i + 2); t.mix = w.dwa; }
         if (i + 1 < nL) { t.wnext = lw[(size_t)(i + 1)].n1; t.groups = groups; t.out = a1; }
         RC(kl::layer_tail(t, bf16, s));
     }
@@ -821,8 +961,6 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
 // ===================================================================================================================================================
 // Scaled layout: x <- x + ls1 * mixer(n1(x)); x <- x + ls2 * ff(n2(x)); learned positions; a layer run uses the weights of layer spec.runs[run] and a
 // cache / state of its own.
-
-namespace { inline int64_t pad16(int64_t n) { return (n + 15) / 16 * 16; } }
 
 int LayeredModel::init_scaled(nvr_model_runner &r) {
     const int64_t W = spec.width, V = spec.vocab, MT = r.max_tokens;
@@ -860,7 +998,7 @@ int LayeredModel::init_scaled(nvr_model_runner &r) {
             RC(own(&w.slope, sl.size() * 4)); NVR_HIP_CHECK(hipMemcpy(w.slope, sl.data(), sl.size() * 4, hipMemcpyHostToDevice));
             if (std::find(attn_groups.begin(), attn_groups.end(), L.heads / L.kv_heads) == attn_groups.end()) attn_groups.push_back(L.heads / L.kv_heads);
             w.flash = bf16 && L.dim == L.vdim && nvr::kb::flash_prefill_ok((int)L.dim, (int)L.heads, (int)L.kv_heads) && hv % 8 == 0;
-            if (w.flash && std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) == flash_groups.end()) flash_groups.push_back(L.heads / L.kv_heads);
+            if (w.flash) flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
             if (bf16) {                                     // the matrix-core attention takes the slopes as its table of penalties by distance (the window bounds the distance)
                 const int64_t n = std::min<int64_t>(r.max_pos, L.window) + 1;
                 RC(dmalloc(&w.pen, (size_t)(L.heads * n * 4)));
@@ -1020,7 +1158,7 @@ int LayeredModel::forward_scaled(nvr_model_runner &r, const StepPlan &p) {
             RC(kl::qkv_norm_store(qa, b, bf16, s));
             if (w.flash && !p.decode_sized) {
                 // prompts and portions: the dense graph's flash kernel in its penalty / sink form, linear in the distance and windowed
-                const size_t gi = (size_t)(std::find(flash_groups.begin(), flash_groups.end(), L.heads / L.kv_heads) - flash_groups.begin());
+                const size_t gi = flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
                 nvr::kt::FlashArgs f{};
                 f.q = (const uint16_t *)a.q; f.ldq = w.nmix; f.k = (const uint16_t *)st.kc; f.v = (const uint16_t *)st.vc; f.ldkv = 0;
                 f.block_tables = b.block_tables; f.max_blocks = b.max_blocks; f.block_size = b.block_size;

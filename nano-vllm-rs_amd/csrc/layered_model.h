@@ -7,7 +7,11 @@
 //   sequential (Pusunex) — x <- x + nb(mixer(n(x))), then x <- x + nb(ff(n(x))) with RMS norms in groups before and after each sublayer; the mixer is latent
 //                          attention (one cached latent row per token, optionally shared with an earlier layer, optionally with a rotated key part and a
 //                          latent for the queries) or gated linear attention; the feed-forward is dense with a polynomial-norm activation or a mixture of
-//                          experts; a per-layer token input and a weighted average over the outputs of all earlier layers close the layer.
+//                          experts; a per-layer token input and a weighted average over the outputs of all earlier layers close the layer;
+//   sequential (Kiduvik) — the same layer without the average over depth, on an embedding with learned positions; the mixer is latent attention with a sink (queries
+//                          straight from the input, every layer with a rotated key part in halves, rows shared with an earlier layer or not) or differential
+//                          attention (two softmax maps per head over the same values, the second subtracted with a learned share, the difference normed; normed and
+//                          rotated queries and keys, a window with kept first tokens, a gate per head); the feed-forward is dense with the exact GELU.
 //   scaled (Sosutar)     — x <- x + ls1 * mixer(n1(x)), then x <- x + ls2 * ff(n2(x)): RMS norms in front, a learned scale per channel behind each sublayer, learned
 //                          positions added to the embedding; the mixer is an exponentially gated matrix memory (mLSTM), or a windowed attention (normed queries, keys
 //                          and values, query temperature, linear distance penalty, sink, output gate) side by side with an elementwise gated recurrence (minGRU),
@@ -44,8 +48,8 @@ struct nvr_model_runner;
 namespace nvr {
 
 struct LayeredSpec {
-    enum Mixer { ATTENTION = 0, RETENTION = 1, LATENT = 2, GLA = 3, MLSTM = 4, ATTN_GRU = 5, SSM = 6, ATTN_TMIX = 7, ATTN_UNIT = 8 };
-    enum Ff { FF_NONE = 0, FF_CLAMPED_GLU = 1, FF_POLY = 2, FF_MOE = 3, FF_RELU2 = 4, FF_MOE_GLU = 5, FF_GEGLU = 6, FF_MOE_IDENT = 7 };
+    enum Mixer { ATTENTION = 0, RETENTION = 1, LATENT = 2, GLA = 3, MLSTM = 4, ATTN_GRU = 5, SSM = 6, ATTN_TMIX = 7, ATTN_UNIT = 8, ATTN_DIFF = 9 };
+    enum Ff { FF_NONE = 0, FF_CLAMPED_GLU = 1, FF_POLY = 2, FF_MOE = 3, FF_RELU2 = 4, FF_MOE_GLU = 5, FF_GEGLU = 6, FF_MOE_IDENT = 7, FF_GELU = 8 };
     enum Layout { PARALLEL = 0, SEQUENTIAL = 1, SCALED = 2, JOINT = 3, STREAMS = 4 };
     struct Layer {
         int mixer = ATTENTION;
@@ -75,10 +79,17 @@ struct LayeredSpec {
         // streams layout: the rotation's frequencies stretched by wavelength (rot_original 0: not) — kept below rot_original / rot_high, divided by rot_factor above
         // rot_original / rot_low, blended between —, values mixed with the first v_mix layer's, experts without a matrix behind the `experts` others
         double rot_low = 1.0, rot_high = 1.0, rot_original = 0.0; bool v_mix = false; int64_t identity = 0;
+        // rotation frequencies stretched by index (rot_original 0: not): kept where the wavelength fits rot_original at least rot_fast times, divided by rot_factor where at most
+        // rot_slow times, blended between; cosines and sines times 0.1 ln(rot_factor) + 1.  rot_halves: number i pairs with i + rot_dims / 2 (else 2i with 2i + 1)
+        double rot_fast = 0.0, rot_slow = 0.0; bool rot_halves = false;
+        bool sink = false;                                  // latent attention: exp(sink of the head) in the softmax denominator
+        int64_t keep_first = 0;                             // windowed attention: the first keys of a sequence stay visible
+        double diff = 0.0;                                  // differential attention: the fixed part of the second map's share
         int64_t t_heads = 0, t_dim = 0;                     // the time-mixing recurrence beside the attention: heads of t_dim x t_dim states
     };
     int layout = PARALLEL;
     int64_t norm_groups = 1;                                // sequential layout: RMS norms over this many equal parts of a row
+    bool depth_average = false;                             // sequential layout: every layer ends in a weighted average over the outputs of all layers so far
     int64_t side_dim = 0;                                   // per-layer token input: numbers per layer and token (0: none)
     int64_t vocab = 0, width = 0;
     double embedding_scale = 1.0, eps = 1e-5, residual_mult = 1.0;
@@ -96,7 +107,12 @@ struct LayeredSpec {
     static int parse_sosutar(const Json &cfg, LayeredSpec *out);
     static int parse_sokalorn(const Json &cfg, LayeredSpec *out);
     static int parse_negunex(const Json &cfg, LayeredSpec *out);
+    static int parse_kiduvik(const Json &cfg, LayeredSpec *out);
 };
+
+// A layer's rotation frequencies [rot_dims / 2], base^(-2i / rot_dims) with whichever stretch the layer names (by wavelength or by index), and the factor that goes with
+// them on cosines and sines (1 but for the stretch by index).
+std::vector<float> rotation_frequencies(const LayeredSpec::Layer &L, float *gain = nullptr);
 
 class LayeredModel {
 public:
@@ -137,6 +153,9 @@ public:
         void *w4 = nullptr, *w1 = nullptr, *w2 = nullptr; int64_t t_rank = 0;         // time mixing: r / k / v / g stacked [4][Ht Dt][W]; decay projections [rank][W], [Ht Dt][rank]
         float *w0 = nullptr, *bonus = nullptr, *tnorm = nullptr;                      // [Ht Dt] each
         void *router_op = nullptr;                                                   // [E + 1, padded to 16][W] operand type: the router's rows, then the shared expert's gate
+        // differential attention: the heads' norms [dim] (in qn, kn), the four vectors the share of the second map is made of (host copies) and the share (one number)
+        std::vector<float> lam[4]; float *lambda = nullptr;
+        float rot_gain = 1.f;                                                        // factor on cosines and sines
         // streams layout: what a sublayer reads from the streams [S], writes into them [S], and their mixing matrix [S][S] (from, to); projection biases; the share of the first
         // layer's values; the experts' choice correction
         float *hin[2] = {nullptr, nullptr}, *hout[2] = {nullptr, nullptr}, *hmix[2] = {nullptr, nullptr};
@@ -151,7 +170,8 @@ public:
     float *wfinal = nullptr; void *side_embed = nullptr;                    // [W]; [vocab][layers * side_dim]
     float *kept = nullptr;                                                  // the embedding output and every layer's output: [layers + 1][max tokens][W] f32
     void *qlat = nullptr, *q2 = nullptr, *qabs = nullptr, *ctx = nullptr, *alow = nullptr, *az = nullptr, *act = nullptr, *shared_y = nullptr;
-    bool flash_contiguous = false; void *kvx = nullptr;                      // flash tiles refer to rows of the step (not to block tables); expanded keys | values of a step
+    void *kvx = nullptr;                                                    // expanded keys | values of a step
+    float *maps_o = nullptr;                                                // differential attention outside the matrix-core kernels: both maps' outputs [max tokens][2 H Dv]
     int64_t alow_cap = 0; void *side_z = nullptr, *side_g = nullptr;
     // scaled layout
     void *pos = nullptr; void *tmp2 = nullptr, *gy = nullptr; float *gpre = nullptr, *tokg = nullptr, *gfloor = nullptr;   // [positions][W]; second branch's output, the recurrence's output; gates
@@ -170,7 +190,11 @@ public:
     float *x = nullptr, *ret_o = nullptr;                                  // residual stream, retention outputs: f32
     void *proj = nullptr, *gu = nullptr, *tmp = nullptr, *a1 = nullptr, *a2 = nullptr, *cat = nullptr, *xsel = nullptr;   // operand type
     int64_t slots = 0; std::vector<int32_t> slot_par;
-    std::vector<int64_t> flash_groups;                      // distinct H / G of the layers whose prompts take the flash kernel: one FlashTile list per value and step
+    // query tiles of the flash kernel: one list per step for every kind the layers need — query positions per tile, and whether the tiles refer to rows of the step (keys
+    // and values expanded for it) or to block tables
+    struct FlashKind { int64_t positions; bool rows; bool operator==(const FlashKind &o) const { return positions == o.positions && rows == o.rows; } };
+    std::vector<FlashKind> flash_kinds;
+    size_t flash_kind(int64_t positions, bool rows = false);                // index of a kind's list, added where it is new (at init)
     std::vector<int64_t> attn_groups;                       // distinct H / G of the attention layers: one list of query tiles per value and step
     void *attn_ws = nullptr; size_t attn_ws_bytes = 0;      // split-key partials of decode-sized steps
     // step inputs
@@ -195,6 +219,8 @@ private:
     int init_sequential(nvr_model_runner &r);
     int load_sequential(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
     int forward_sequential(nvr_model_runner &r, const StepPlan &p);
+    int diff_share(LayerW &w, const LayeredSpec::Layer &L);
+    kl::SinkAttnArgs diff_args(const LayerW &w, const LayeredSpec::Layer &L) const;
     int init_scaled(nvr_model_runner &r);
     int load_scaled(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
     int forward_scaled(nvr_model_runner &r, const StepPlan &p);

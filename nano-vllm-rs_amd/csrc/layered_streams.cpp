@@ -16,23 +16,6 @@ namespace nvr {
 namespace {
 inline int64_t pad16(int64_t n) { return (n + 15) / 16 * 16; }
 
-// base^(-2i / dims); with a stretch: kept for wavelengths below original / high, divided by factor above original / low, blended linearly in original / wavelength between
-std::vector<float> rotation_frequencies(const LayeredSpec::Layer &L) {
-    std::vector<float> f((size_t)std::max<int64_t>(L.rot_dims / 2, 1));
-    for (int64_t j = 0; j < L.rot_dims / 2; ++j) {
-        double v = std::pow(L.rot_base, -2.0 * (double)j / (double)L.rot_dims);
-        if (L.rot_original > 0) {
-            const double wave = 2.0 * M_PI / v;
-            if (wave > L.rot_original / L.rot_low) v /= L.rot_factor;
-            else if (!(wave < L.rot_original / L.rot_high)) {
-                const double s = L.rot_high > L.rot_low ? (L.rot_original / wave - L.rot_low) / (L.rot_high - L.rot_low) : 1.0;
-                v = (1.0 - s) * v / L.rot_factor + s * v;
-            }
-        }
-        f[(size_t)j] = (float)v;
-    }
-    return f;
-}
 template <class V, class T> void add_once(V &v, T x) { if (std::find(v.begin(), v.end(), x) == v.end()) v.push_back(x); }
 template <class V, class T> size_t index_of(const V &v, T x) { return (size_t)(std::find(v.begin(), v.end(), x) - v.begin()); }
 }
@@ -63,7 +46,7 @@ int LayeredModel::init_streams(nvr_model_runner &r) {
         // plain causal softmax: equal key and value sizes of 64 / 128 take the dense graph's kernels, prompts and portions its flash kernel, decoded tokens its split decode attention
         w.flash = bf16 && L.dim == L.vdim && nvr::kb::flash_prefill_ok((int)L.dim, (int)L.heads, (int)L.kv_heads);
         if (w.flash) {
-            add_once(flash_groups, g);
+            flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
             dec_ws_bytes = std::max(dec_ws_bytes, nvr::kb::attn_workspace_bytes(r.max_seqs, L.heads, L.dim, (r.max_pos + 255) / 256 * 256));
             max_pairs = std::max(max_pairs, r.max_seqs * L.kv_heads);
         }
@@ -228,7 +211,7 @@ int LayeredModel::forward_streams(nvr_model_runner &r, const StepPlan &p) {
             d.scale = a.scale; d.max_ctx = (int32_t)p.max_ctx; d.out = (uint16_t *)cat; d.workspace = dec_ws; d.workspace_bytes = dec_ws_bytes; d.tickets = dec_tickets;
             RC(nvr::kb::attention(d, true, s));
         } else if (w.flash) {
-            const size_t gi = index_of(flash_groups, g);
+            const size_t gi = flash_kind(nvr::kb::flash_tile_positions((int)L.heads, (int)L.kv_heads));
             nvr::kt::FlashArgs f{};
             f.q = (const uint16_t *)a.q; f.ldq = w.nmix; f.k = (const uint16_t *)rst.kc; f.v = (const uint16_t *)rst.vc; f.ldkv = 0;
             f.block_tables = b.block_tables; f.max_blocks = b.max_blocks; f.block_size = b.block_size;

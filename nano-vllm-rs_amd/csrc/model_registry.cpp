@@ -75,6 +75,11 @@ int parse_negunex_spec(const Json &c, nvr_model_spec *out) {
     return LayeredSpec::parse_negunex(c, &out->layered);
 }
 
+int parse_kiduvik_spec(const Json &c, nvr_model_spec *out) {
+    out->family = 1;
+    return LayeredSpec::parse_kiduvik(c, &out->layered);
+}
+
 struct Entry { const char *name; int (*parse)(const Json &, nvr_model_spec *); };
 const Entry kRegistry[] = {
     {"Qwen3ForCausalLM", parse_qwen3},
@@ -83,6 +88,7 @@ const Entry kRegistry[] = {
     {"Sosutar", parse_sosutar_spec},
     {"Sokalorn", parse_sokalorn_spec},
     {"Negunex", parse_negunex_spec},
+    {"Kiduvik", parse_kiduvik_spec},
 };
 
 }  // namespace
@@ -156,7 +162,7 @@ int LayeredSpec::parse_rugudra(const Json &c, LayeredSpec *s) {
 // (polynomial-norm activation) or 'moe' (sigmoid router, top-k, shared expert); a per-layer token input ('token_side') and a weighted average over depth.
 int LayeredSpec::parse_pusunex(const Json &c, LayeredSpec *s) {
     Reader rd;
-    s->layout = SEQUENTIAL; s->taps = 1; s->embedding_scale = 1.0; s->residual_mult = 1.0;
+    s->layout = SEQUENTIAL; s->taps = 1; s->embedding_scale = 1.0; s->residual_mult = 1.0; s->depth_average = true;
     s->vocab = rd.integer(c, "vocab", ""); s->width = rd.integer(c, "width", "");
     if (const Json *n = rd.need(c, "norm", "")) { s->eps = rd.num(*n, "eps", "norm."); s->norm_groups = rd.integer(*n, "groups", "norm."); }
     const Json *side = c.get("token_side");
@@ -454,6 +460,86 @@ int LayeredSpec::parse_negunex(const Json &c, LayeredSpec *s) {
             else if (s->layers[(size_t)first_mix].kv_heads * s->layers[(size_t)first_mix].vdim != L.kv_heads * L.vdim)
                 return fail(NVR_ERR_INVALID_ARG, "config: '%sv_mix' mixes values of other sizes than layer %ld's", wm.c_str(), (long)first_mix);
         }
+        s->layers.push_back(L); s->runs.push_back((int)i);
+    }
+    return NVR_OK;
+}
+
+// Kiduvik: the sequential layer (norms before and after each sublayer, per-layer token input) on an embedding with learned positions.  Mixers 'latent_attention'
+// (mixer.{heads, dim, rot_dim, vdim, kv_rank, scale, rot.{dims, base}}, optional kv_from, optional mask; a sink per head) and 'attention' (differential: mixer.{heads, kv_heads,
+// dim, vdim, scale, diff}, optional rot.{dims, base, scaling.{factor, original, fast, slow}}, optional mask.{size, keep_first}); feed-forward 'dense' (exact GELU) or none.
+int LayeredSpec::parse_kiduvik(const Json &c, LayeredSpec *s) {
+    Reader rd;
+    s->layout = SEQUENTIAL; s->taps = 1; s->embedding_scale = 1.0; s->residual_mult = 1.0; s->norm_groups = 1; s->depth_average = false;
+    s->vocab = rd.integer(c, "vocab", ""); s->width = rd.integer(c, "width", ""); s->max_positions = rd.integer(c, "max_positions", "");
+    if (const Json *n = rd.need(c, "norm", "")) s->eps = rd.num(*n, "eps", "norm.");
+    const Json *side = c.get("token_side");
+    s->side_dim = (side && !side->is_null()) ? rd.integer(*side, "dim", "token_side.") : 0;
+    const Json *layers = rd.need(c, "layers", "");
+    if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+    if (layers->kind != Json::Arr || layers->arr.empty()) return fail(NVR_ERR_INVALID_ARG, "config: 'layers' is not a list of layers");
+    if (s->vocab < 1 || s->width < 1 || s->max_positions < 1 || s->side_dim < 0) return fail(NVR_ERR_INVALID_ARG, "config: vocab, width and max_positions must be positive");
+    s->layers.clear(); s->runs.clear();
+    for (size_t i = 0; i < layers->arr.size(); ++i) {
+        const Json &lj = layers->arr[i];
+        const std::string w = "layers[" + std::to_string(i) + "].", wm = w + "mixer.";
+        Layer L;
+        const Json *type = rd.need(lj, "type", w), *mx = rd.need(lj, "mixer", w);
+        if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+        if (type->kind != Json::Str) return fail(NVR_ERR_INVALID_ARG, "config: '%stype' is not a string", w.c_str());
+        const bool latent = type->str == "latent_attention";
+        if (!latent && type->str != "attention") return fail(NVR_ERR_UNSUPPORTED, "config: layer type '%s' (attention or latent_attention)", type->str.c_str());
+        L.heads = rd.integer(*mx, "heads", wm); L.dim = rd.integer(*mx, "dim", wm); L.vdim = rd.integer(*mx, "vdim", wm); L.scale = rd.num(*mx, "scale", wm);
+        L.rot_halves = true;
+        const Json *rot = mx->get("rot");
+        if (rot && !rot->is_null()) {
+            L.rot_dims = rd.integer(*rot, "dims", wm + "rot."); L.rot_base = rd.num(*rot, "base", wm + "rot.");
+            const Json *sc = rot->get("scaling");
+            if (sc && !sc->is_null()) {
+                const std::string ws = wm + "rot.scaling.";
+                L.rot_factor = rd.num(*sc, "factor", ws); L.rot_original = rd.num(*sc, "original", ws); L.rot_fast = rd.num(*sc, "fast", ws); L.rot_slow = rd.num(*sc, "slow", ws);
+                if (rd.err.empty() && !(L.rot_factor > 0 && L.rot_original > 0 && L.rot_fast > 0 && L.rot_slow > 0 && L.rot_base > 1))
+                    return fail(NVR_ERR_INVALID_ARG, "config: %s factor, original, fast and slow must be positive (and rot.base above 1)", ws.c_str());
+            }
+        }
+        const Json *mask = mx->get("mask");
+        if (mask && !mask->is_null()) {
+            L.window = rd.integer(*mask, "size", wm + "mask.");
+            const Json *kf = mask->get("keep_first");
+            if (kf && !kf->is_null()) L.keep_first = rd.integer(*mask, "keep_first", wm + "mask.");
+            if (rd.err.empty() && (L.window < 1 || L.keep_first < 0)) return fail(NVR_ERR_INVALID_ARG, "config: '%smask' needs a positive size and keep_first >= 0", wm.c_str());
+        }
+        if (latent) {
+            L.mixer = LATENT; L.kv_heads = 1; L.sink = true;
+            L.kv_rank = rd.integer(*mx, "kv_rank", wm);
+            const Json *rdim = mx->get("rot_dim");
+            if (rdim && !rdim->is_null()) L.rot_dim = rd.integer(*mx, "rot_dim", wm);
+            if (rd.err.empty() && (L.kv_rank < 1 || L.rot_dim < 0 || L.rot_dim % 2 || L.rot_dims != L.rot_dim || !(L.rot_base > 0)))
+                return fail(NVR_ERR_INVALID_ARG, "config: %s needs a positive kv_rank and rotates rot.dims = rot_dim coordinates, an even number", wm.c_str());
+            const Json *from = mx->get("kv_from");
+            if (from && !from->is_null()) {
+                L.kv_from = rd.integer(*mx, "kv_from", wm);
+                if (L.kv_from < 0 || L.kv_from >= (int64_t)i) return fail(NVR_ERR_INVALID_ARG, "config: '%skv_from' must name an earlier layer", wm.c_str());
+                const Layer &src = s->layers[(size_t)L.kv_from];
+                if (src.mixer != LATENT || src.kv_from >= 0 || src.kv_rank != L.kv_rank || src.rot_dim != L.rot_dim)
+                    return fail(NVR_ERR_INVALID_ARG, "config: '%skv_from' must name a latent-attention layer with a latent of its own and the same kv_rank and rot_dim", wm.c_str());
+            }
+        } else {
+            L.mixer = ATTN_DIFF; L.out_gate = true;
+            L.kv_heads = rd.integer(*mx, "kv_heads", wm); L.diff = rd.num(*mx, "diff", wm);
+            if (rd.err.empty() && (L.rot_dims < 0 || L.rot_dims % 2 || L.rot_dims > L.dim || !(L.rot_base > 0)))
+                return fail(NVR_ERR_INVALID_ARG, "config: %s needs an even rot.dims <= dim and a positive base", wm.c_str());
+        }
+        const Json *mlp = lj.get("mlp");
+        if (mlp && !mlp->is_null()) {
+            const Json *kind = rd.need(*mlp, "kind", w + "mlp.");
+            if (kind && !(kind->kind == Json::Str && kind->str == "dense")) return fail(NVR_ERR_UNSUPPORTED, "config: '%smlp.kind' (dense)", w.c_str());
+            L.has_mlp = true; L.ff_kind = FF_GELU; L.ff = rd.integer(*mlp, "ff", w + "mlp.");
+            if (rd.err.empty() && L.ff < 1) return fail(NVR_ERR_INVALID_ARG, "config: '%smlp.ff' must be positive", w.c_str());
+        }
+        if (!rd.err.empty()) return fail(NVR_ERR_INVALID_ARG, "%s", rd.err.c_str());
+        if (L.heads < 1 || L.dim < 1 || L.vdim < 1 || L.kv_heads < 1 || L.heads % L.kv_heads)
+            return fail(NVR_ERR_INVALID_ARG, "config: %s %ld heads over %ld key/value heads of %ld / %ld", wm.c_str(), (long)L.heads, (long)L.kv_heads, (long)L.dim, (long)L.vdim);
         s->layers.push_back(L); s->runs.push_back((int)i);
     }
     return NVR_OK;
