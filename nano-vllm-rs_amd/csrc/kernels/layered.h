@@ -64,7 +64,8 @@ struct SinkAttnArgs {
     const float *lambda; float out_scale, eps; const void *head_gate; int64_t ldhg; float *maps_o;
 };
 int sink_attention(const SinkAttnArgs &a, const Batch &b, bool bf16, hipStream_t s);     // any shape; a context that fits the LDS score buffer
-// The same on the matrix cores (bf16 operands, D and Dv multiples of 8 up to 256, at most 16 query heads per key/value head — a head of differential attention counts twice).  tiles
+// The same on the matrix cores (bf16 operands, D % 32 == 0 and Dv % 16 == 0, with two maps D % 16 == 0 and Dv % 8 == 0, both <= 256, at most 16 query heads per key/value head — a head with
+// two maps counts twice).  tiles
 // (device, built by the host): tile i covers the rows row0 .. row0 + 64 / g - 1 of sequence seq's chunk, for all g query heads of a key/value head.  nsplit > 1 spreads a tile's keys over that many
 // workgroups (decode-sized steps over long contexts) and merges their partials; workspace: sink_attention_workspace_bytes(ntiles * G * nsplit).
 struct AttnTile { int32_t seq, row0; };
@@ -133,17 +134,18 @@ struct GroupNormArgs {
 };
 int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s);
 
-// Latent attention caches ONE row per token: `rank` numbers of the latent (proj columns col ..., divided by their root mean square, times w) and `rot` numbers of a
-// key part shared by the heads, rotated in pairs (2i, 2i+1), or (i, i + rot / 2) with halves, by position * freq[i] (cosines and sines times gain).  pages:
-// [blocks][block_size][rank + rot] of the operand type; rows (may be null): the same rows in step order, [T][rank + rot].
-int latent_store(const void *proj, int64_t ld, int64_t col, const Batch &b, int64_t rank, int64_t rot, float eps, const float *w, const float *freq, void *pages, void *rows,
-                 bool bf16, hipStream_t s, bool halves = false, float gain = 1.f);
+// What latent attention does between its projections and its products, each part optional (null pointers).  pages: the ONE cached row per token, `rank` numbers of the latent (proj
+// columns col ..., divided by their root mean square, times w) and `rot` numbers of a key part shared by the heads, rotated by position * freq[i] in pairs (2i, 2i+1), or
+// (i, i + rot / 2) with halves (cosines and sines times gain); [blocks][block_size][rank + rot] of the operand type; rows (may be null): the same rows in step order, [T][rank + rot].
+// q: the rotated part of the queries, q[t][h * qstride + qcol ...] -> out[t][h * ostride + ocol ...] (may be the same place).
+struct LatentRopeArgs {
+    const void *proj; int64_t ld, col; int32_t rank; float eps; const float *w; void *pages, *rows;
+    const void *q; int64_t ldq, qstride, qcol; int32_t H; void *out; int64_t ldo, ostride, ocol;
+    int32_t rot; const float *freq; bool halves; float gain;
+};
+int latent_rope(const LatentRopeArgs &a, const Batch &b, bool bf16, hipStream_t s);
 // y[t][c] *= sigmoid(g[t][c]) (c < N; rows of y / g with strides ldy / ldg)
 int sigmoid_gate(void *y, int64_t ldy, const void *g, int64_t ldg, int64_t T, int64_t N, bool bf16, hipStream_t s);
-// The rotated part of the queries: q[t][h * qstride + qcol ...] (rot numbers, pairs as in latent_store) -> out[t][h * ostride + ocol ...]
-int rotate_heads(const void *q, int64_t ldq, int64_t qstride, int64_t qcol, const Batch &b, int64_t H, int64_t rot, const float *freq, void *out, int64_t ldo, int64_t ostride,
-                 int64_t ocol, bool bf16, hipStream_t s, bool halves = false, float gain = 1.f);
-
 // y[t][h * hy + n] = sum_k a[t][h * ha + k] * w[h][n][k] (n < N, k < K; rows of a / y / gate with strides lda / ldy / ldg), times sigmoid(gate[t][h * hg + n]) when gate is not null.
 // One matrix per head: the key expansion folded into the queries (w[h] = Wuk_h^T), the value expansion of the attended latent (w[h] = Wuv_h).
 struct HeadLinearArgs { const void *a; int64_t lda, ha; const void *w; void *y; int64_t ldy, hy; const void *gate; int64_t ldg, hg; int32_t T, H, K, N; };

@@ -533,7 +533,16 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
     }
 }
 
-// one wave per (tile, key/value head, row): out = sum_z o_z 2^(m_z - m) / sum_z l_z 2^(m_z - m)
+// Of a row's partials (at most 64 splits), lane z holds split z's weight 2^(m_z - m) / sum_z l_z 2^(m_z - m).  (A split that saw no visible key has m = -inf and weight 0; what it left is zero.)
+__device__ __forceinline__ float split_weight(const float *__restrict__ part_ml, int64_t base, int r, int nsplit) {
+    const int z = threadIdx.x & 63;
+    float m = -INFINITY, l = 0.f;
+    if (z < nsplit) { const float2 v = *reinterpret_cast<const float2 *>(part_ml + ((base + z) * 64 + r) * 2); m = v.x; l = v.y; }
+    const float mx = wave_max(m), e = m == -INFINITY ? 0.f : exp2f(m - mx);
+    return e / wave_sum(l * e);
+}
+
+// one wave per (tile, key/value head, row): out = sum_z o_z weight_z
 __global__ __launch_bounds__(64) void sink_attn_merge_kernel(SinkAttnArgs a, Batch b, const AttnTile *__restrict__ tiles, int nsplit, const float *__restrict__ part_o,
                                                              const float *__restrict__ part_ml) {
     const int tile = blockIdx.x, kvh = blockIdx.y, r = blockIdx.z;
@@ -543,15 +552,14 @@ __global__ __launch_bounds__(64) void sink_attn_merge_kernel(SinkAttnArgs a, Bat
     const int pi = r / g, hg = r % g;
     if (pi >= npos) return;
     const int64_t base = ((int64_t)tile * a.G + kvh) * nsplit;
-    float m = -INFINITY;
-    for (int z = 0; z < nsplit; ++z) m = fmaxf(m, part_ml[((base + z) * 64 + r) * 2]);
-    float l = 0.f;
-    for (int z = 0; z < nsplit; ++z) { const float mz = part_ml[((base + z) * 64 + r) * 2]; if (mz != -INFINITY) l += part_ml[((base + z) * 64 + r) * 2 + 1] * exp2f(mz - m); }
+    const float wz = split_weight(part_ml, base, r, nsplit);
     bf16_t *o = (bf16_t *)a.out + (int64_t)(c0 + lr0 + pi) * a.ldo + (int64_t)(kvh * g + hg) * a.Dv;
-    for (int c = threadIdx.x; c < a.Dv; c += 64) {
+    for (int cb = 0; cb < a.Dv; cb += 64) {              // (every lane takes part in the shuffles)
+        const int c = cb + threadIdx.x, cc = min(c, a.Dv - 1);
         float acc = 0.f;
-        for (int z = 0; z < nsplit; ++z) { const float mz = part_ml[((base + z) * 64 + r) * 2]; if (mz != -INFINITY) acc += part_o[((base + z) * 64 + r) * a.Dv + c] * exp2f(mz - m); }
-        st_f(o, c, acc / l);
+#pragma unroll 8
+        for (int z = 0; z < nsplit; ++z) acc += part_o[((base + z) * 64 + r) * a.Dv + cc] * __shfl(wz, z, 64);
+        if (c < a.Dv) st_f(o, c, acc);
     }
 }
 
@@ -568,21 +576,13 @@ __global__ __launch_bounds__(64) void diff_attn_merge_kernel(SinkAttnArgs a, Bat
     float d[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < 2; ++k) {
-        float m = -INFINITY;
-        for (int z = 0; z < nsplit; ++z) m = fmaxf(m, part_ml[((base + z) * 64 + r + k) * 2]);
-        float l = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
+        const float wz = split_weight(part_ml, base, r + k, nsplit) * (k ? -*a.lambda : 1.0f);
+#pragma unroll 4
         for (int z = 0; z < nsplit; ++z) {
-            const float mz = part_ml[((base + z) * 64 + r + k) * 2];
-            if (mz == -INFINITY) continue;
-            const float e = exp2f(mz - m);
-            l += part_ml[((base + z) * 64 + r + k) * 2 + 1] * e;
-            const float *o = part_o + ((base + z) * 64 + r + k) * a.Dv;
+            const float e = __shfl(wz, z, 64), *o = part_o + ((base + z) * 64 + r + k) * a.Dv;
 #pragma unroll
-            for (int x = 0; x < 4; ++x) if (threadIdx.x + 64 * x < a.Dv) acc[x] += o[threadIdx.x + 64 * x] * e;
+            for (int x = 0; x < 4; ++x) if (threadIdx.x + 64 * x < a.Dv) d[x] += o[threadIdx.x + 64 * x] * e;
         }
-        const float f = k ? -*a.lambda / l : 1.0f / l;
-#pragma unroll
-        for (int x = 0; x < 4; ++x) d[x] += acc[x] * f;
     }
     const float ss = wave_sum((d[0] * d[0] + d[1] * d[1]) + (d[2] * d[2] + d[3] * d[3]));
     const int64_t row = c0 + lr0 + pi;
@@ -997,7 +997,8 @@ int kv_store(const void *proj, int64_t ld, int64_t kcol, int64_t vcol, const Bat
 
 bool sink_attention_tiled_ok(const SinkAttnArgs &a, bool bf16, int block_size) {
     const int maps = a.lambda ? 2 : 1;
-    return bf16 && (block_size % 8 == 0 || !a.v_grouped) && a.G >= 1 && a.H % a.G == 0 && a.H * maps / a.G <= 16 && a.D % (8 * maps) == 0 && a.Dv % 8 == 0 && a.D <= 256 && a.Dv <= 256 && a.ldq % 8 == 0 && a.vld % 8 == 0 &&
+    const bool sizes = a.lambda ? a.D % 16 == 0 && a.Dv % 8 == 0 : a.D % 32 == 0 && a.Dv % 16 == 0;      // (one map: the sizes that fill the tiles)
+    return bf16 && sizes && (block_size % 8 == 0 || !a.v_grouped) && a.G >= 1 && a.H % a.G == 0 && a.H * maps / a.G <= 16 && a.D <= 256 && a.Dv <= 256 && a.ldq % 8 == 0 && a.vld % 8 == 0 &&
            (!a.vld || !a.v_grouped) && ((uintptr_t)a.q % 16) == 0 && ((uintptr_t)a.kc % 16) == 0 && ((uintptr_t)a.vc % 16) == 0;
 }
 size_t sink_attention_workspace_bytes(int max_workgroups) { return (size_t)max_workgroups * 64 * (256 + 2) * sizeof(float); }

@@ -81,7 +81,7 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const IT *__restrict__ 
 
 // ------------------------------------------------------------------------------------------------ the cached row of latent attention
 // Row t of proj holds, from column col, `rank` latent numbers and `rot` numbers of the shared key part.  The page row of the token's position receives the latent
-// divided by its root mean square times w, and the key part with coordinate pairs (2i, 2i+1) turned by position * freq[i].
+// divided by its root mean square times w, and the key part with coordinate pairs (2i, 2i+1), or halves (i, i + rot / 2), turned by position * freq[i].
 template <class CT>
 __global__ __launch_bounds__(64) void latent_store_kernel(const CT *__restrict__ proj, int64_t ld, int64_t col, Batch b, int rank, int rot, float eps,
                                                           const float *__restrict__ w, const float *__restrict__ freq, CT *__restrict__ pages, CT *__restrict__ rows, int halves, float gain) {
@@ -120,6 +120,73 @@ __global__ __launch_bounds__(256) void rotate_heads_kernel(const CT *__restrict_
         CT *dst = out + (int64_t)t * ldo + (int64_t)h * ostride + ocol;
         st_f(dst, cu, u * cs - v * sn); st_f(dst, cv, v * cs + u * sn);
     }
+}
+
+// Both at once for 16-bit rows whose parts are multiples of 8 numbers (halves: a rotated part of a multiple of 16): 16-byte loads and stores, cosines and sines once per row.  RB rows
+// per workgroup: 4, a wave each; or 1, its queries by all four waves.
+template <int RB>
+__global__ __launch_bounds__(256) void latent_rope8_kernel(LatentRopeArgs a, Batch b) {
+    extern __shared__ float2 tab[];                     // [RB][half] (cosine, sine)
+    const int half = a.rot >> 1, r0 = blockIdx.x * RB;
+    for (int idx = threadIdx.x; idx < RB * half; idx += 256) {
+        const int rr = RB == 1 ? 0 : idx / half, i = idx - rr * half, t = r0 + rr;
+        if (t < b.T) { const int sq = b.row_seq[t]; const float ang = (float)(b.start[sq] + (t - b.cu[sq])) * a.freq[i]; tab[idx] = float2{a.gain * cosf(ang), a.gain * sinf(ang)}; }
+    }
+    __syncthreads();
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, rr = RB == 1 ? 0 : wave, t = r0 + rr;
+    if (t >= b.T) return;
+    const float2 *ct = tab + rr * half;
+    const int nch = a.halves ? half >> 3 : a.rot >> 3;  // pieces of a rotated part: 8 numbers of each half, or 4 pairs
+    auto turn = [&](const bf16_t *src, bf16_t *d1, bf16_t *d2, int i) {       // piece i of the part at src -> the same place behind d1 and d2 (d2 may be null)
+        if (a.halves) {
+            const uint4 x = *reinterpret_cast<const uint4 *>(src + i * 8), y = *reinterpret_cast<const uint4 *>(src + half + i * 8);
+            const bf16_t *xe = reinterpret_cast<const bf16_t *>(&x), *ye = reinterpret_cast<const bf16_t *>(&y);
+            uint4 o1, o2; bf16_t *e1 = reinterpret_cast<bf16_t *>(&o1), *e2 = reinterpret_cast<bf16_t *>(&o2);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) {
+                const float2 c = ct[i * 8 + k]; const float u = ld_f(xe, k), v = ld_f(ye, k);
+                st_f(e1, k, u * c.x - v * c.y); st_f(e2, k, v * c.x + u * c.y);
+            }
+            *reinterpret_cast<uint4 *>(d1 + i * 8) = o1; *reinterpret_cast<uint4 *>(d1 + half + i * 8) = o2;
+            if (d2) { *reinterpret_cast<uint4 *>(d2 + i * 8) = o1; *reinterpret_cast<uint4 *>(d2 + half + i * 8) = o2; }
+        } else {
+            const uint4 x = *reinterpret_cast<const uint4 *>(src + i * 8); const bf16_t *xe = reinterpret_cast<const bf16_t *>(&x);
+            uint4 o; bf16_t *e = reinterpret_cast<bf16_t *>(&o);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const float2 c = ct[i * 4 + k]; const float u = ld_f(xe, 2 * k), v = ld_f(xe, 2 * k + 1);
+                st_f(e, 2 * k, u * c.x - v * c.y); st_f(e, 2 * k + 1, v * c.x + u * c.y);
+            }
+            *reinterpret_cast<uint4 *>(d1 + i * 8) = o;
+            if (d2) *reinterpret_cast<uint4 *>(d2 + i * 8) = o;
+        }
+    };
+    if (a.pages && (RB > 1 || wave == 0)) {
+        const int sq = b.row_seq[t], p = b.start[sq] + (t - b.cu[sq]), blk = b.block_tables[(int64_t)sq * b.max_blocks + p / b.block_size];
+        bf16_t *d1 = (bf16_t *)a.pages + ((int64_t)blk * b.block_size + p % b.block_size) * (a.rank + a.rot), *d2 = a.rows ? (bf16_t *)a.rows + (int64_t)t * (a.rank + a.rot) : nullptr;
+        const bf16_t *src = (const bf16_t *)a.proj + (int64_t)t * a.ld + a.col;
+        float ss = 0.f;
+        for (int c = lane * 8; c < a.rank; c += 512) {
+            const uint4 x = *reinterpret_cast<const uint4 *>(src + c); const bf16_t *xe = reinterpret_cast<const bf16_t *>(&x);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) { const float v = ld_f(xe, k); ss += v * v; }
+        }
+        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.rank + a.eps);
+        for (int c = lane * 8; c < a.rank; c += 512) {
+            const uint4 x = *reinterpret_cast<const uint4 *>(src + c); const bf16_t *xe = reinterpret_cast<const bf16_t *>(&x);
+            uint4 o; bf16_t *e = reinterpret_cast<bf16_t *>(&o);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) st_f(e, k, ld_f(xe, k) * inv * a.w[c + k]);
+            *reinterpret_cast<uint4 *>(d1 + c) = o;
+            if (d2) *reinterpret_cast<uint4 *>(d2 + c) = o;
+        }
+        for (int i = lane; i < nch; i += 64) turn(src + a.rank, d1 + a.rank, d2 ? d2 + a.rank : nullptr, i);
+    }
+    if (a.q)
+        for (int idx = RB == 1 ? threadIdx.x : lane; idx < a.H * nch; idx += RB == 1 ? 256 : 64) {
+            const int h = idx / nch, i = idx - h * nch;
+            turn((const bf16_t *)a.q + (int64_t)t * a.ldq + h * a.qstride + a.qcol, (bf16_t *)a.out + (int64_t)t * a.ldo + h * a.ostride + a.ocol, nullptr, i);
+        }
 }
 
 // ------------------------------------------------------------------------------------------------ one small matrix per head / per group of rows
@@ -1023,22 +1090,31 @@ int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s) {
     return launched("group_norm");
 }
 
-int latent_store(const void *proj, int64_t ld, int64_t col, const Batch &b, int64_t rank, int64_t rot, float eps, const float *w, const float *freq, void *pages, void *rows,
-                 bool bf16, hipStream_t s, bool halves, float gain) {
+int latent_rope(const LatentRopeArgs &a, const Batch &b, bool bf16, hipStream_t s) {
     if (b.T == 0) return 0;
-    if (rot % 2) return nvr::fail(NVR_ERR_INVALID_ARG, "latent_store: %ld rotated coordinates", (long)rot);
-    if (bf16) latent_store_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const bf16_t *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (bf16_t *)pages, (bf16_t *)rows, halves ? 1 : 0, gain);
-    else latent_store_kernel<float><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const float *)proj, ld, col, b, (int)rank, (int)rot, eps, w, freq, (float *)pages, (float *)rows, halves ? 1 : 0, gain);
-    return launched("latent_store");
-}
-
-int rotate_heads(const void *q, int64_t ldq, int64_t qstride, int64_t qcol, const Batch &b, int64_t H, int64_t rot, const float *freq, void *out, int64_t ldo, int64_t ostride,
-                 int64_t ocol, bool bf16, hipStream_t s, bool halves, float gain) {
-    if (b.T == 0 || rot == 0) return 0;
-    if (rot % 2) return nvr::fail(NVR_ERR_INVALID_ARG, "rotate_heads: %ld rotated coordinates", (long)rot);
-    if (bf16) rotate_heads_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const bf16_t *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (bf16_t *)out, ldo, (int)ostride, (int)ocol, halves ? 1 : 0, gain);
-    else rotate_heads_kernel<float><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const float *)q, ldq, (int)qstride, (int)qcol, b, (int)H, (int)rot, freq, (float *)out, ldo, (int)ostride, (int)ocol, halves ? 1 : 0, gain);
-    return launched("rotate_heads");
+    if (a.rot % 2) return nvr::fail(NVR_ERR_INVALID_ARG, "latent_rope: %d rotated coordinates", a.rot);
+    const bool turns = a.q && a.rot > 0;
+    if (!a.pages && !turns) return 0;
+    const bool vec = bf16 && a.rot % (a.halves ? 16 : 8) == 0 && a.rot <= 4096 && (!a.pages || (a.rank % 8 == 0 && a.ld % 8 == 0 && a.col % 8 == 0 && aligned16(a.proj) && aligned16(a.pages) && aligned16(a.rows))) &&
+                     (!turns || (((a.ldq | a.qstride | a.qcol | a.ldo | a.ostride | a.ocol) & 7) == 0 && aligned16(a.q) && aligned16(a.out)));
+    if (vec) {
+        LatentRopeArgs v = a;
+        if (!turns) v.q = nullptr;
+        const size_t lds = (size_t)std::max(a.rot / 2, 1) * sizeof(float2);
+        if (b.T >= 1024 && 4 * lds <= 60000) latent_rope8_kernel<4><<<dim3((unsigned)((b.T + 3) / 4)), dim3(256), 4 * lds, s>>>(v, b);
+        else latent_rope8_kernel<1><<<dim3((unsigned)b.T), dim3(256), lds, s>>>(v, b);
+        return launched("latent_rope");
+    }
+    const int hv = a.halves ? 1 : 0;
+    if (a.pages) {
+        if (bf16) latent_store_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const bf16_t *)a.proj, a.ld, a.col, b, a.rank, a.rot, a.eps, a.w, a.freq, (bf16_t *)a.pages, (bf16_t *)a.rows, hv, a.gain);
+        else latent_store_kernel<float><<<dim3((unsigned)b.T), dim3(64), 0, s>>>((const float *)a.proj, a.ld, a.col, b, a.rank, a.rot, a.eps, a.w, a.freq, (float *)a.pages, (float *)a.rows, hv, a.gain);
+    }
+    if (turns) {
+        if (bf16) rotate_heads_kernel<bf16_t><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const bf16_t *)a.q, a.ldq, (int)a.qstride, (int)a.qcol, b, a.H, a.rot, a.freq, (bf16_t *)a.out, a.ldo, (int)a.ostride, (int)a.ocol, hv, a.gain);
+        else rotate_heads_kernel<float><<<dim3((unsigned)b.T), dim3(256), 0, s>>>((const float *)a.q, a.ldq, (int)a.qstride, (int)a.qcol, b, a.H, a.rot, a.freq, (float *)a.out, a.ldo, (int)a.ostride, (int)a.ocol, hv, a.gain);
+    }
+    return launched("latent_rope");
 }
 
 int head_linear(const HeadLinearArgs &a, bool bf16, hipStream_t s) {

@@ -811,10 +811,16 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
                 RC(gemm(r, qlat, L.q_rank, w.uq, T, L.q_rank, L.heads * (L.dim + Rr), q2));
                 qsrc = q2; ldq = L.heads * (L.dim + Rr); qstride = L.dim + Rr;
             }
-            if (L.kv_from < 0) RC(kl::latent_store(proj, w.nmix, w.dcol, b, rank, Rr, eps, w.dkvn, w.rfreq, st.kc, st.rows, bf16, s, L.rot_halves, w.rot_gain));
-            if (w.flash && p.whole_prompts) {
+            const bool expanded = w.flash && p.whole_prompts;
+            kl::LatentRopeArgs lr{};
+            if (L.kv_from < 0) { lr.proj = proj; lr.ld = w.nmix; lr.col = w.dcol; lr.eps = eps; lr.w = w.dkvn; lr.pages = st.kc; lr.rows = st.rows; }
+            lr.rank = (int32_t)rank; lr.rot = (int32_t)Rr; lr.freq = w.rfreq; lr.halves = L.rot_halves; lr.gain = w.rot_gain;
+            lr.q = qsrc; lr.ldq = ldq; lr.qstride = qstride; lr.qcol = L.dim; lr.H = (int32_t)L.heads;
+            if (expanded) { lr.out = (void *)qsrc; lr.ldo = ldq; lr.ostride = qstride; lr.ocol = L.dim; }      // (in place: a thread reads its pairs, then writes them)
+            else { lr.out = qabs; lr.ldo = L.heads * Dq; lr.ostride = Dq; lr.ocol = rank; }
+            RC(kl::latent_rope(lr, b, bf16, s));
+            if (expanded) {
                 // every key is a row of this step: K (with the rotated part) and V of all heads by one product from the step's cached rows, then the flash kernel
-                RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, (void *)qsrc, ldq, qstride, L.dim, bf16, s, L.rot_halves, w.rot_gain));   // (in place: a thread reads a pair, then writes it)
                 RC(gemm(r, st.rows, Dq, w.wx, T, Dq, 2 * hv, kvx));
                 const size_t gi = flash_kind(nvr::kb::flash_tile_positions(1, 1), true);
                 nvr::kt::FlashArgs f{};
@@ -828,7 +834,6 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             kl::HeadLinearArgs ha{}; ha.a = qsrc; ha.lda = ldq; ha.ha = qstride; ha.w = w.ukt; ha.y = qabs; ha.ldy = L.heads * Dq; ha.hy = Dq;
             ha.T = (int32_t)T; ha.H = (int32_t)L.heads; ha.K = (int32_t)L.dim; ha.N = (int32_t)rank;
             RC(kl::head_linear(ha, bf16, s));
-            RC(kl::rotate_heads(qsrc, ldq, qstride, L.dim, b, L.heads, Rr, w.rfreq, qabs, L.heads * Dq, Dq, rank, bf16, s, L.rot_halves, w.rot_gain));
             kl::SinkAttnArgs a{};
             a.q = qabs; a.ldq = L.heads * Dq; a.kc = st.kc; a.vc = st.kc; a.vld = Dq; a.H = (int32_t)L.heads; a.G = 1; a.D = (int32_t)Dq; a.Dv = (int32_t)rank;
             a.scale = (float)L.scale; a.out = ctx; a.ldo = L.heads * rank; a.sink = w.sink; a.window = (int32_t)L.window; a.keep_first = (int32_t)L.keep_first;

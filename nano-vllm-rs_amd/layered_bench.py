@@ -1,4 +1,4 @@
-"""Prefill and decode throughput of the layer-list designs (Rugudra, Pusunex, Sosutar, Sokalorn, Negunex) beside the dense Qwen3 graph at equal sizes (bench.py --layered-compare).
+"""Prefill and decode throughput of the layer-list designs (Rugudra, Pusunex, Sosutar, Sokalorn, Negunex, Kiduvik) beside the dense Qwen3 graph at equal sizes (bench.py --layered-compare).
 
 Random weights, layer shapes that resemble a real model's; both models go through the same engine (scheduler, block manager, runner step).
 Per size one JSON object: tokens/s of one prefill step over BATCH prompts of PROMPT tokens and of the decode steps that follow, for both."""
@@ -271,8 +271,59 @@ def negunex_weights(cfg, seed=0):
     return out
 
 
+def kiduvik_config(s, window=512, keep=64):
+    """Layers in turn: differential attention with a window (two maps of half the head size over values of the full size: projections as large as a plain attention's), latent
+    attention with a latent of its own, latent attention on that layer's rows, differential attention; dense feed-forwards of ff."""
+    H, G, D, W = s["heads"], s["kv_heads"], s["dim"], s["width"]
+    layers, src = [], None
+    for i in range(s["layers"]):
+        if i % 4 in (0, 3):
+            m = {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "scale": (D // 2) ** -0.5, "diff": 0.5, "mask": {"size": window, "keep_first": keep},
+                 "rot": {"dims": D // 2, "base": 1000000.0, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            layers.append({"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}})
+        else:
+            m = {"heads": H, "dim": D - 64, "rot_dim": 64, "vdim": D, "kv_rank": 192, "rot": {"dims": 64, "base": 10000.0}, "scale": D ** -0.5}
+            if i % 4 == 2:
+                m["kv_from"] = src
+            else:
+                src = i
+            layers.append({"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}})
+    return {"architecture": "Kiduvik", "vocab": s["vocab"], "width": W, "max_positions": 4096, "norm": {"eps": 1e-5}, "token_side": {"dim": 64}, "layers": layers}
+
+
+def kiduvik_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    W, V, nL, side = cfg["width"], cfg["vocab"], len(cfg["layers"]), cfg["token_side"]["dim"]
+
+    def lin(o, i, g=1.0):
+        return (rng.standard_normal((o, i), dtype=np.float32) * (g / np.sqrt(i))).astype(np.float32)
+
+    def gains(n, mean=1.0):
+        return (mean * (1.0 + 0.1 * rng.standard_normal(n))).astype(np.float32)
+    out = {"embed": rng.standard_normal((V, W), dtype=np.float32), "pos": 0.5 * rng.standard_normal((cfg["max_positions"], W), dtype=np.float32), "head": lin(V, W), "final.norm": gains(W),
+           "side.embed": rng.standard_normal((V, nL * side), dtype=np.float32)}
+    for i, L in enumerate(cfg["layers"]):
+        m, p, F = L["mixer"], "l%d." % i, L["mlp"]["ff"]
+        q, H, D, Dv = p + "mix.", m["heads"], m["dim"], m["vdim"]
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            out[p + n] = gains(W)
+        if L["type"] == "attention":
+            G = m["kv_heads"]
+            out[q + "q"], out[q + "k"], out[q + "v"], out[q + "g"], out[q + "q.norm"], out[q + "k.norm"] = lin(2 * H * D, W), lin(2 * G * D, W), lin(G * Dv, W), lin(H, W), gains(D), gains(D)
+            for n in ("lq1", "lk1", "lq2", "lk2"):
+                out[q + n] = (0.5 * D ** -0.5 * rng.standard_normal(D)).astype(np.float32)
+        else:
+            rank, R = m["kv_rank"], m["rot_dim"]
+            out[q + "q"], out[q + "uk"], out[q + "uv"], out[q + "sink"] = lin(H * (D + R), W), lin(H * D, rank), lin(H * Dv, rank), rng.standard_normal(H).astype(np.float32)
+            if m.get("kv_from") is None:
+                out[q + "dkv"], out[q + "dkv.norm"] = lin(rank + R, W), gains(rank)
+        out[q + "o"], out[p + "mlp.up"], out[p + "mlp.down"] = lin(W, H * Dv), lin(F, W), lin(W, F)
+        out[p + "side.gate"], out[p + "side.proj"], out[p + "side.norm"] = lin(side, W), lin(W, side), gains(W, 0.3)
+    return out
+
+
 LAYERED = {"rugudra": (rugudra_config, random_weights), "pusunex": (pusunex_config, pusunex_weights), "sosutar": (sosutar_config, sosutar_weights),
-           "sokalorn": (sokalorn_config, sokalorn_weights), "negunex": (negunex_config, negunex_weights),
+           "sokalorn": (sokalorn_config, sokalorn_weights), "negunex": (negunex_config, negunex_weights), "kiduvik": (kiduvik_config, kiduvik_weights),
            "negunex4": (lambda s: negunex_config(s, streams=4), negunex_weights)}      # (four streams instead of two)
 
 
