@@ -76,6 +76,13 @@ int penalty_table(const float *r1, const float *r2, int64_t H, int64_t n, float 
 int linear_penalty_table(const float *slope, int64_t H, int64_t n, float *tab, hipStream_t s);
 size_t sink_attention_workspace_bytes(int max_workgroups);
 int sink_attention_tiled(const SinkAttnArgs &a, const Batch &b, const AttnTile *tiles, int ntiles, int nsplit, void *workspace, size_t workspace_bytes, hipStream_t s);
+// Decode-sized steps (one row per sequence) in one launch (layered_decode.hip): bf16 operands, D % 32 == 0, Dv % 16 == 0, both <= 256, row-major value pages or values inside the key
+// rows (vld = D, one key/value head); sink, window with kept keys and two maps as above, no penalties, gated weights or chunks.  The keys go to up to max_splits workgroups per group of up
+// to 16 query rows; tickets: num_tickets >= sequences * attention_decode_groups counters, zero before the first launch (every launch leaves them zero).
+int prepare_decode();                                   // LDS opt-ins (call once, outside captures)
+bool attention_decode_ok(const SinkAttnArgs &a, bool bf16);
+int attention_decode_groups(const SinkAttnArgs &a);
+int attention_decode(const SinkAttnArgs &a, const Batch &b, int max_splits, void *workspace, size_t workspace_bytes, unsigned int *tickets, int num_tickets, hipStream_t s);
 
 // Retention over the rows of a step: per head S <- decay[h] * S + k v^T, o = S^T q, with q and k rotated (first rot_dims coordinates, pairs (i, i + rot_dims/2),
 // angle = position * freq[i], cosines and sines from a table) and k scaled by kscale after the rotation.  state: [slots][H][D][Dv] f32, zero at position 0.  proj: rows of the operand type (stride ld) holding

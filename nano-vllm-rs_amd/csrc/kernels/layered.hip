@@ -488,30 +488,40 @@ __global__ __launch_bounds__(256, 2) void sink_attn_mfma_kernel(SinkAttnArgs a, 
             }
         }
     }
+    if (DIFF && nsplit == 1) __syncthreads();                   // (the key and value images give way to the rows)
     if (!wave_on) return;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
 #pragma unroll
         for (int o = 1; o < 16; o <<= 1) l[i] += __shfl_xor(l[i], o, 64);
     }
-    if (DIFF && nsplit == 1) {
+    if (DIFF && nsplit == 1) {                                  // a wave's 16 rows through LDS, then a pair of rows (the two maps of one head) at a time
+        float *rows = (float *)smem + (int64_t)wave * 16 * Dv;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float inv = 1.0f / l[i];
+#pragma unroll
+            for (int t = 0; t < C / 16; ++t) if (t * 16 + lm < Dv) rows[(lq * 4 + i) * Dv + t * 16 + lm] = acc[t][i] * inv;
+        }
+        __builtin_amdgcn_wave_barrier();
         const float lam = *a.lambda;
-#pragma unroll
-        for (int i = 0; i < 4; i += 2) {                        // rows i, i + 1: the two maps of one head
-            const int r = wave * 16 + lq * 4 + i, pi = r / g, h = (kvh * g + r % g) >> 1;
-            const float i0 = 1.0f / l[i], i1 = lam / l[i + 1];
-            float ss = 0.f;
-#pragma unroll
-            for (int t = 0; t < C / 16; ++t) { const float d = acc[t][i] * i0 - acc[t][i + 1] * i1; acc[t][i] = d; if (t * 16 + lm < Dv) ss += d * d; }
-#pragma unroll
-            for (int o = 1; o < 16; o <<= 1) ss += __shfl_xor(ss, o, 64);
-            if (pi >= npos) continue;
+        for (int i = 0; i < 16; i += 2) {
+            const int r = wave * 16 + i, pi = r / g, h = (kvh * g + r % g) >> 1;
+            if (pi >= npos) break;
+            const float *d1 = rows + i * Dv, *d2 = d1 + Dv;
             const int64_t row = c0 + lr0 + pi;
-            float f = a.out_scale / sqrtf(ss / (float)Dv + a.eps);
+            float d[C / 64], ss = 0.f;
+#pragma unroll
+            for (int x = 0; x < C / 64; ++x) {
+                const int c = lane + 64 * x;
+                d[x] = c < Dv ? d1[c] - lam * d2[c] : 0.f;
+                ss += d[x] * d[x];
+            }
+            float f = a.out_scale / sqrtf(wave_sum(ss) / (float)Dv + a.eps);
             if (a.head_gate) f /= 1.0f + expf(-ld_f((const bf16_t *)a.head_gate, row * a.ldhg + h));
             bf16_t *o = (bf16_t *)a.out + row * a.ldo + (int64_t)h * Dv;
 #pragma unroll
-            for (int t = 0; t < C / 16; ++t) if (t * 16 + lm < Dv) st_f(o, t * 16 + lm, acc[t][i] * f);
+            for (int x = 0; x < C / 64; ++x) if (lane + 64 * x < Dv) st_f(o, lane + 64 * x, d[x] * f);
         }
         return;
     }

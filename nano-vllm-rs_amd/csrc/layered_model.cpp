@@ -106,7 +106,7 @@ int LayeredModel::init(nvr_model_runner &r) {
     r.device = r.cfg.device_ordinal;
     NVR_HIP_CHECK(hipSetDevice(r.device));
     NVR_HIP_CHECK(hipStreamCreateWithFlags(&r.stream, hipStreamNonBlocking));
-    RC(kl::prepare()); RC(kl::prepare_blocks()); RC(kl::prepare_streams());
+    RC(kl::prepare()); RC(kl::prepare_blocks()); RC(kl::prepare_streams()); RC(kl::prepare_decode());
     if (r.f32) RC(nvr::kf::prepare());
     else { RC(nvr::kb::linear_stream_prepare()); RC(nvr::kb::gemm_tiled_prepare()); }
     { int v = 0; if (hipDeviceGetAttribute(&v, hipDeviceAttributeMultiprocessorCount, r.device) == hipSuccess && v > 0) r.num_cus = v; }
@@ -511,7 +511,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
         return (int)NVR_OK;
     };
     lw.resize(spec.layers.size());
-    int64_t max_kvx = 0, max_experts = 0, max_f = 0, max_maps = 0;
+    int64_t max_kvx = 0, max_experts = 0, max_f = 0, max_maps = 0, max_groups = 0;
     int64_t max_nmix = 0, max_q2 = 0, max_qabs = 0, max_ctx = 0, max_hv = 0, max_qlat = 0, max_hd = 0, max_ff = 0, max_rows_e = 0, max_e2f = 0, max_ef = 0;
     size_t block_bytes = 0;
     for (size_t i = 0; i < spec.layers.size(); ++i) {
@@ -547,6 +547,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             int64_t g = std::min<int64_t>(L.heads, 16);
             while (L.heads % g) --g;
             w.head_share = g;
+            max_groups = std::max(max_groups, (L.heads + 15) / 16);
             if (std::find(attn_groups.begin(), attn_groups.end(), g) == attn_groups.end()) attn_groups.push_back(g);
         } else if (L.mixer == LayeredSpec::GLA) {
             w.qcol = 0; w.kcol = hd; w.vcol = 2 * hd; w.gcol = 2 * hd + hv; w.nmix = 2 * hd + 2 * hv;
@@ -567,6 +568,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             // prompts and portions with values twice the size of a map's keys, key rows of 64 / 128 numbers: the flash kernel in its differential form
             w.flash = bf16 && 2 * L.dim == L.vdim && L.scale > 0 && hv % 8 == 0 && nvr::kb::flash_diff_ok((int)L.vdim, (int)L.heads, (int)L.kv_heads);
             if (w.flash) flash_kind(nvr::kb::flash_diff_tile_positions((int)L.heads, (int)L.kv_heads));
+            max_groups = std::max<int64_t>(max_groups, kl::attention_decode_groups(diff_args(w, L)));
             if (!kl::sink_attention_tiled_ok(diff_args(w, L), bf16, (int)r.block_size)) max_maps = std::max(max_maps, L.heads * 2 * L.vdim);
         } else return fail(NVR_ERR_UNSUPPORTED, "layer %zu: this mixer does not belong to the sequential layout", i);
         RC(named(&w.mix, (size_t)(w.nmix * W * esz))); RC(own(&w.wo, (size_t)(W * hv * esz)));
@@ -627,6 +629,7 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
     // activations
     RC(named((void **)&x, (size_t)(MT * W * 4)));
     if (spec.depth_average) RC(own(&kept, (size_t)((nL + 1) * MT * W * 4)));
+    if (bf16 && max_groups) { dec_tickets_n = r.max_seqs * max_groups; RC(own(&dec_tickets, (size_t)dec_tickets_n * 4)); }
     if (max_maps) RC(own(&maps_o, (size_t)(MT * max_maps * 4)));
     RC(named(&a1, (size_t)(MT * W * esz))); RC(named(&a2, (size_t)(MT * W * esz))); RC(named(&tmp, (size_t)(MT * W * esz)));
     RC(named(&proj, (size_t)(MT * max_nmix * esz))); RC(named(&cat, (size_t)(MT * max_hv * esz)));
@@ -658,6 +661,12 @@ kl::SinkAttnArgs LayeredModel::diff_args(const LayerW &w, const LayeredSpec::Lay
     a.window = (int32_t)L.window; a.keep_first = (int32_t)L.keep_first; a.v_grouped = w.flash ? 0 : 1;      // (a property of the layer: the pages keep one layout)
     a.lambda = w.lambda; a.out_scale = (float)(1.0 - L.diff); a.eps = (float)spec.eps; a.ldhg = w.nmix;
     return a;
+}
+
+// One position per sequence: up to four workgroups per compute unit share the keys.
+int LayeredModel::decode_attention(nvr_model_runner &r, const kl::SinkAttnArgs &a, const StepPlan &p) {
+    const int64_t pairs = (int64_t)p.b.B * kl::attention_decode_groups(a);
+    return kl::attention_decode(a, p.b, (int)std::max<int64_t>(1, 4 * (int64_t)r.num_cus / std::max<int64_t>(pairs, 1)), attn_ws, attn_ws_bytes, dec_tickets, (int)dec_tickets_n, r.stream);
 }
 
 // Tensors by the names of the checkpoint: "embed", "head", "final.norm" [W], "pos" [positions][W], "side.embed" [vocab][layers * side]; per layer i "l<i>.norm1" / "norm1b" / "norm2" / "norm2b" [W],
@@ -838,7 +847,8 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             a.q = qabs; a.ldq = L.heads * Dq; a.kc = st.kc; a.vc = st.kc; a.vld = Dq; a.H = (int32_t)L.heads; a.G = 1; a.D = (int32_t)Dq; a.Dv = (int32_t)rank;
             a.scale = (float)L.scale; a.out = ctx; a.ldo = L.heads * rank; a.sink = w.sink; a.window = (int32_t)L.window; a.keep_first = (int32_t)L.keep_first;
             kl::SinkAttnArgs a1s = a; a1s.H = (int32_t)w.head_share;
-            if (kl::sink_attention_tiled_ok(a1s, bf16, (int)r.block_size)) {
+            if (p.decode_sized && kl::attention_decode_ok(a, bf16)) RC(decode_attention(r, a, p));
+            else if (kl::sink_attention_tiled_ok(a1s, bf16, (int)r.block_size)) {
                 const size_t gi = (size_t)(std::find(attn_groups.begin(), attn_groups.end(), w.head_share) - attn_groups.begin());
                 const int64_t wgs = (int64_t)p.n_tiles[gi];
                 int64_t nsplit = 1;
@@ -876,7 +886,8 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
                 f.H = a.H; f.KVH = a.G; f.D = a.Dv; f.scale = a.scale; f.out = (uint16_t *)cat; f.ldo = hv; f.window = a.window; f.keep_first = a.keep_first;
                 f.lambda = a.lambda; f.out_scale = a.out_scale; f.eps = a.eps; f.head_gate = (const uint16_t *)a.head_gate; f.ldhg = a.ldhg;
                 RC(nvr::kb::flash_prefill(f, true, s));
-            } else if (tiled) {
+            } else if (p.decode_sized && kl::attention_decode_ok(a, bf16)) RC(decode_attention(r, a, p));
+            else if (tiled) {
                 const size_t gi = (size_t)(std::find(attn_groups.begin(), attn_groups.end(), 2 * L.heads / L.kv_heads) - attn_groups.begin());
                 const int64_t wgs = (int64_t)p.n_tiles[gi] * L.kv_heads, keys = L.window > 0 ? std::min<int64_t>(p.max_ctx, L.window + L.keep_first + 64) : p.max_ctx;
                 int64_t nsplit = 1;

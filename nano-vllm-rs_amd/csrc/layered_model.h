@@ -220,6 +220,7 @@ private:
     int load_sequential(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);
     int forward_sequential(nvr_model_runner &r, const StepPlan &p);
     int diff_share(LayerW &w, const LayeredSpec::Layer &L);
+    int decode_attention(nvr_model_runner &r, const kl::SinkAttnArgs &a, const StepPlan &p);
     kl::SinkAttnArgs diff_args(const LayerW &w, const LayeredSpec::Layer &L) const;
     int init_scaled(nvr_model_runner &r);
     int load_scaled(nvr_model_runner &r, const std::string &name, int dtype, const int64_t *shape, int ndim, const void *data);

@@ -32,11 +32,11 @@ MECHANISMS = {
                                                             latent(kv_from=0, kv_rank=32, heads=1, dim=40, vdim=8)]),
     "latent_one_head": make_config([latent(heads=1, dim=24, vdim=40, kv_rank=16, rot_dim=2)]),
     "latent_odd_sizes": make_config([latent(heads=5, dim=7, vdim=5, kv_rank=9, rot_dim=6), latent(kv_from=0, heads=3, dim=1, vdim=1, kv_rank=9, rot_dim=6)], width=60),
-    "latent_rank_above_everything": make_config([latent(heads=2, dim=8, vdim=8, kv_rank=200, rot_dim=40)]),
+    "latent_rank_above_everything": make_config([latent(heads=2, dim=8, vdim=8, kv_rank=200, rot_dim=40), latent(heads=3, dim=8, vdim=8, kv_rank=208, rot_dim=48)]),
     "latent_rows_past_the_matrix_core_kernel": make_config([latent(heads=2, dim=16, vdim=16, kv_rank=264, rot_dim=16)]),
     "latent_rows_of_88": make_config([latent(heads=3, dim=16, vdim=16, kv_rank=72, rot_dim=16)]),
-    "latent_fourteen_heads": make_config([latent(heads=14, dim=16, vdim=8, kv_rank=32, rot_dim=16)]),
-    "latent_thirty_four_heads": make_config([latent(heads=34, dim=8, vdim=8, kv_rank=24, rot_dim=8)]),
+    "latent_fourteen_heads": make_config([latent(heads=14, dim=16, vdim=8, kv_rank=16, rot_dim=16)]),
+    "latent_thirty_four_heads": make_config([latent(heads=34, dim=8, vdim=8, kv_rank=32, rot_dim=32)]),
     "latent_heads_of_64": make_config([latent(heads=3, dim=48, vdim=64, kv_rank=48, rot_dim=16), latent(heads=4, dim=56, vdim=64, kv_rank=48, rot_dim=16, kv_from=0)], width=96),
     "latent_heads_of_128": make_config([latent(heads=2, dim=64, vdim=128, kv_rank=96, rot_dim=64, base=30000.0)], width=96),
     "latent_windowed": make_config([latent(mask=(9, 2)), latent(heads=2, dim=56, vdim=64, kv_rank=48, rot_dim=8, mask=(20, 0))]),
