@@ -50,13 +50,12 @@ __device__ __forceinline__ float dot2(half2_t a, half2_t b, float c) {
 __device__ __forceinline__ float sigmoid_fast(float x) { return __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
 // what the gate g of a gated feed-forward is multiplied by: silu(g) = g sigmoid(g); the tanh form of gelu, g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) / 2 = g sigmoid(2 sqrt(2/pi) (g + 0.044715 g^3))
 __device__ __forceinline__ float gate_factor(float g, bool gelu) { return sigmoid_fast(gelu ? 1.5957691216057308f * (g + 0.044715f * g * g * g) : g); }
-// gelu with the error function, z Phi(z), for results that are rounded to 16 bits: erfc(|z| / sqrt 2) by the rational approximation 7.1.26 of Abramowitz and Stegun, Handbook of
-// Mathematical Functions (absolute error below 1.5e-7), one v_rcp and one v_exp
+// gelu with the error function, z Phi(z), for results that are rounded to 16 bits: erfc by the rational approximation 7.1.26 of Abramowitz and Stegun, Handbook of Mathematical
+// Functions (absolute error below 1.5e-7), one v_rcp and one v_exp; z Phi(z) = max(z, 0) - |z| erfc(|z| / sqrt 2) / 2
 __device__ __forceinline__ float gelu_erf_fast(float z) {
-    const float x = fabsf(z) * 0.70710678118654752f, t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.0f));
-    const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.061405429f, -1.453152027f), 1.421413741f), -0.284496736f), 0.254829592f);
-    const float half_c = 0.5f * poly * __builtin_amdgcn_exp2f(-1.4426950408889634f * x * x);
-    return z * (z >= 0.f ? 1.0f - half_c : half_c);
+    const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f * 0.70710678f, fabsf(z), 1.0f));
+    const float poly = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 0.5f * 1.061405429f, 0.5f * -1.453152027f), 0.5f * 1.421413741f), 0.5f * -0.284496736f), 0.5f * 0.254829592f);
+    return fmaf(-fabsf(z), poly * __builtin_amdgcn_exp2f(z * z * (-0.5f * 1.4426950408889634f)), fmaxf(z, 0.f));
 }
 
 // Activation block x[T, cols] (row stride ldx, columns col0 .. col0 + 8*cpr) -> LDS image of ROWS rows x cpr 16-byte chunks, chunk ch of

@@ -32,7 +32,7 @@
 
 namespace nvr { namespace NVR_DT_NS {
 
-enum { GEPI_F16 = 0, GEPI_RESID = 1, GEPI_SILU = 2, GEPI_ROPE = 3, GEPI_LMHEAD = 4, GEPI_RELU2 = 5, GEPI_GELU = 6, GEPI_GELU_ERF = 7 };   // GELU_ERF: y = gelu(x·Wᵀ) with the error function, RELU2: y = max(x·Wᵀ, 0)² (the product rounded to 16 bits first, as the unfused pair of launches does)
+enum { GEPI_F16 = 0, GEPI_RESID = 1, GEPI_SILU = 2, GEPI_ROPE = 3, GEPI_LMHEAD = 4, GEPI_RELU2 = 5, GEPI_GELU = 6, GEPI_GELU_ERF = 7 };   // GELU_ERF: y = gelu(x·Wᵀ) with the error function (from the unrounded product); RELU2: y = max(x·Wᵀ, 0)² (the product rounded to 16 bits first, as the unfused pair of launches does)
 constexpr bool g_glu(int epi) { return epi == GEPI_SILU || epi == GEPI_GELU; }      // gate and up rows in one tile, out = act(gate) * up (GELU: the tanh form)
 //   // RESID: y is the residual stream: y <- fp16(y + fp16(x·Wᵀ)) (qwen3.rs:382,389)
 // LMHEAD (r06): the LM head over >= 128 rows (ParallelLMHead::compute_logits, embed_head.rs:292-306, + the greedy branch of Sampler::forward,
@@ -368,7 +368,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const half_t *__restrict__
                             }
                             if (EPI == GEPI_GELU_ERF) {
 #pragma unroll
-                                for (int e = 0; e < 4; ++e) v[e] = gelu_erf_fast((float)(half_t)v[e]);
+                                for (int e = 0; e < 4; ++e) v[e] = gelu_erf_fast(v[e]);
                             }
                             pk[a][i][b][j] = (half4_t){(half_t)v[0], (half_t)v[1], (half_t)v[2], (half_t)v[3]};
                         }
@@ -559,7 +559,7 @@ int gemm256_relu2(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T
                                                                                           (int)N, (int)N, (half_t *)y, G256Epi{}, tx, tt / tx, g256_cg(tx, tt / tx, false));
     return g256_check("gemm256_relu2");
 }
-// y = gelu(x . W^T) with the error function (the product rounded to 16 bits first, as the unfused pair of launches does)
+// y = gelu(x . W^T) with the error function, of the unrounded product
 int gemm256_gelu(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, hipStream_t s) {
     if (!gemm256_ok(T, K, N, ldx)) return nvr::fail(NVR_ERR_UNSUPPORTED, "gemm256_gelu: T=%ld K=%ld N=%ld", (long)T, (long)K, (long)N);
     if (int rc = g256_prepare()) return rc;

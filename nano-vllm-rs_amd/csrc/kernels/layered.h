@@ -192,6 +192,15 @@ int moe_combine(const void *y, const int32_t *place_of, int64_t T, int64_t top, 
 // (z = Wg x rows of dim numbers -> g), and its last step inside layer_tail.
 int side_gate(const void *z, const int64_t *ids, const void *E, int64_t lde, int64_t ecol, int64_t dim, int64_t T, void *g, bool bf16, hipStream_t s);
 
+// The token input of few rows (up to 64) in one launch, with the join in front of it and the norm behind it: x += y / rms(y) * wb, u = proj (gelu_tanh(gate x) * E[id][ecol .. + dim)),
+// x += u / rms(u) * ws, out = x / rms(x) * wn (wn null: without).  gate: [dim][W], proj: [W][dim], y rows of the operand type.
+struct SideStepArgs { float *x; int32_t T, W, dim; float eps; const void *y; int64_t ldy; const float *wb; const void *gate, *proj; const int64_t *ids; const void *E; int64_t lde, ecol; const float *ws, *wn; void *out; int64_t ldo; };
+bool side_step_ok(const SideStepArgs &a, bool bf16);
+int side_step(const SideStepArgs &a, hipStream_t s);
+
+// x[t] = E[ids[t]] * scale + P[position of row t] (P null: without), out = x / sqrt(mean(x^2) + eps) * wn
+int embed_norm(const void *E, const void *P, bool bf16, const Batch &b, int64_t W, float scale, float *x, float eps, const float *wn, void *out, hipStream_t s);
+
 // The end of a layer, per row and each part optional: the token input's last step (x += side_y / rms(side_y) * side_norm; side_y rows of the operand type), the weighted
 // average over depth (this x becomes kept stream nx - 1; x <- sum_j mix[j] kept[j], kept: [streams][kept_rows][W] f32), and the next layer's first norm of the new x.
 struct LayerTailArgs {

@@ -901,52 +901,177 @@ __global__ __launch_bounds__(256) void gelu_erf8_kernel(const bf16_t *__restrict
     *reinterpret_cast<uint4 *>(out + t * ldo + c) = v;
 }
 
-// ------------------------------------------------------------------------------------------------ a normed row joins the stream
-// x += y / rms(y) * wb; then, where asked for, out = x / rms(x) * wn, or (plain) x itself in the operand type.  16-bit rows, widths that are multiples of 4, one norm group: NT threads
-// per row (64: a wave, four rows per workgroup, no barrier; 256: the workgroup), the row in registers.
-template <int NT, int NV>
-__global__ __launch_bounds__(256) void norm_join4_kernel(float *__restrict__ x, const bf16_t *__restrict__ y, int64_t ldy, int64_t T, int W, float eps, const float *__restrict__ wb,
-                                                         const float *__restrict__ wn, int plain, bf16_t *__restrict__ out, int64_t ldo) {
+// ------------------------------------------------------------------------------------------------ rows of the stream in registers
+// NJ_JOIN: x += y / rms(y) * wb; then, where asked for, out = x / rms(x) * wn, or (plain) x itself in the operand type.  NJ_NORM: out = x / rms(x) * wn alone, of the rows rows[r] (null: r).
+// NJ_START: x = E[id] scale + P[position] (P null: without), then out = x / rms(x) * wn.  16-bit operands, widths that are multiples of 4, one norm group: NT threads per row (64: a wave,
+// four rows per workgroup, no barrier; 256: the workgroup).
+enum { NJ_JOIN = 0, NJ_NORM = 1, NJ_START = 2 };
+struct NormJoin { float *x; const bf16_t *y; int64_t ldy, T; int W; float eps; const float *wb, *wn; int plain; bf16_t *out; int64_t ldo; const int32_t *rows; int64_t ldx; const bf16_t *E, *P; float scale; };
+__device__ __forceinline__ float4 unpack4(uint2 v) { return float4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)}; }
+__device__ __forceinline__ uint2 pack4(float4 v) {
+    bf16_t h[4];
+    st_f(h, 0, v.x); st_f(h, 1, v.y); st_f(h, 2, v.z); st_f(h, 3, v.w);
+    return uint2{(uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16)};
+}
+__device__ __forceinline__ float square4(float4 v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); }
+template <int NT, int NV, int KIND>
+__global__ __launch_bounds__(256) void norm_join4_kernel(NormJoin a, Batch b) {
     __shared__ float red[4];
-    const int W4 = W >> 2, l = threadIdx.x & (NT - 1);
+    const int W4 = a.W >> 2, l = threadIdx.x & (NT - 1);
     const int64_t t = (int64_t)blockIdx.x * (256 / NT) + threadIdx.x / NT;
-    if (NT == 64 && t >= T) return;                     // (a whole wave: nobody waits for it)
-    float *xr = x + t * W;
+    if (NT == 64 && t >= a.T) return;                   // (a whole wave: nobody waits for it)
+    float *xr = a.x + (KIND == NJ_NORM && a.rows ? (int64_t)a.rows[t] : t) * a.ldx;
+    const bf16_t *er = nullptr, *pr = nullptr;
+    if (KIND == NJ_START) {
+        er = a.E + b.ids[t] * (int64_t)a.W;
+        const int sq = b.row_seq[t];
+        if (a.P) pr = a.P + (int64_t)(b.start[sq] + ((int)t - b.cu[sq])) * a.W;
+    }
     float4 xs[NV], ys[NV];
-    float ss = 0.f;
+    float ss = 0.f, s2 = 0.f;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
         const int c4 = l + k * NT;
         xs[k] = ys[k] = float4{0.f, 0.f, 0.f, 0.f};
         if (c4 < W4) {
-            xs[k] = *reinterpret_cast<const float4 *>(xr + c4 * 4);
-            const uint2 v = *reinterpret_cast<const uint2 *>(y + t * ldy + c4 * 4);
-            ys[k] = float4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)};
+            if (KIND == NJ_START) {
+                const float4 e = unpack4(*reinterpret_cast<const uint2 *>(er + c4 * 4));
+                xs[k] = float4{e.x * a.scale, e.y * a.scale, e.z * a.scale, e.w * a.scale};
+                if (pr) { const float4 q = unpack4(*reinterpret_cast<const uint2 *>(pr + c4 * 4)); xs[k].x += q.x; xs[k].y += q.y; xs[k].z += q.z; xs[k].w += q.w; }
+                *reinterpret_cast<float4 *>(xr + c4 * 4) = xs[k];
+            } else xs[k] = *reinterpret_cast<const float4 *>(xr + c4 * 4);
+            if (KIND == NJ_JOIN) ys[k] = unpack4(*reinterpret_cast<const uint2 *>(a.y + t * a.ldy + c4 * 4));
         }
-        ss += (ys[k].x * ys[k].x + ys[k].y * ys[k].y) + (ys[k].z * ys[k].z + ys[k].w * ys[k].w);
+        if (KIND == NJ_JOIN) ss += square4(ys[k]); else s2 += square4(xs[k]);
     }
-    const float f = 1.0f / sqrtf((NT == 64 ? wave_sum(ss) : block_sum256(ss, red)) / (float)W + eps);
+    if (KIND == NJ_JOIN) {
+        const float f = 1.0f / sqrtf((NT == 64 ? wave_sum(ss) : block_sum256(ss, red)) / (float)a.W + a.eps);
+#pragma unroll
+        for (int k = 0; k < NV; ++k) {
+            const int c4 = l + k * NT;
+            if (c4 < W4) {
+                const float4 w = *reinterpret_cast<const float4 *>(a.wb + c4 * 4);
+                xs[k].x += ys[k].x * f * w.x; xs[k].y += ys[k].y * f * w.y; xs[k].z += ys[k].z * f * w.z; xs[k].w += ys[k].w * f * w.w;
+                *reinterpret_cast<float4 *>(xr + c4 * 4) = xs[k];
+                s2 += square4(xs[k]);
+            }
+        }
+        if (!a.wn && !a.plain) return;
+    }
+    const float f2 = a.wn ? 1.0f / sqrtf((NT == 64 ? wave_sum(s2) : block_sum256(s2, red)) / (float)a.W + a.eps) : 1.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = l + k * NT;
+        if (c4 < W4) {
+            const float4 w = a.wn ? *reinterpret_cast<const float4 *>(a.wn + c4 * 4) : float4{1.f, 1.f, 1.f, 1.f};
+            *reinterpret_cast<uint2 *>(a.out + t * a.ldo + c4 * 4) = pack4(float4{xs[k].x * f2 * w.x, xs[k].y * f2 * w.y, xs[k].z * f2 * w.z, xs[k].w * f2 * w.w});
+        }
+    }
+}
+
+// The end of a layer with a token input for few rows, a workgroup of 1024 per row: a sublayer's result joins (x += y / rms(y) * wb), z = Wg x, g = gelu_tanh(z) * E[id], u = Wp g,
+// x += u / rms(u) * ws, and the next norm.  The roundings are those of the launches it stands for (x, z, g and u as 16-bit operands).
+template <int NV>
+__global__ __launch_bounds__(1024) void side_step_kernel(SideStepArgs a) {
+    extern __shared__ __attribute__((aligned(16))) char sm_[];
+    bf16_t *xb = (bf16_t *)sm_; bf16_t *gs = xb + a.W;   // [W] x, [dim] g, operand type
+    __shared__ float red[16];
+    const int64_t t = blockIdx.x;
+    const int W = a.W, W4 = W >> 2, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, dim = a.dim;
+    auto sum_all = [&](float v) {
+        v = wave_sum(v);
+        __syncthreads();
+        if (lane == 0) red[wave] = v;
+        __syncthreads();
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s += red[i];
+        return s;
+    };
+    float *xr = a.x + t * W;
+    float4 xs[NV], ys[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = tid + k * 1024;
+        xs[k] = ys[k] = float4{0.f, 0.f, 0.f, 0.f};
+        if (c4 < W4) { xs[k] = *reinterpret_cast<const float4 *>(xr + c4 * 4); ys[k] = unpack4(*reinterpret_cast<const uint2 *>((const bf16_t *)a.y + t * a.ldy + c4 * 4)); }
+        ss += square4(ys[k]);
+    }
+    const float f = 1.0f / sqrtf(sum_all(ss) / (float)W + a.eps);
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = tid + k * 1024;
+        if (c4 < W4) {
+            const float4 w = *reinterpret_cast<const float4 *>(a.wb + c4 * 4);
+            xs[k].x += ys[k].x * f * w.x; xs[k].y += ys[k].y * f * w.y; xs[k].z += ys[k].z * f * w.z; xs[k].w += ys[k].w * f * w.w;
+            *reinterpret_cast<uint2 *>(xb + c4 * 4) = pack4(xs[k]);
+        }
+    }
+    __syncthreads();
+    const bf16_t *Wg = (const bf16_t *)a.gate, *er = (const bf16_t *)a.E + a.ids[t] * a.lde + a.ecol;
+    auto dot8 = [](uint4 u, uint4 v, float acc) {
+        const bf16_t *ue = reinterpret_cast<const bf16_t *>(&u), *ve = reinterpret_cast<const bf16_t *>(&v);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) acc = fmaf(ld_f(ue, k), ld_f(ve, k), acc);
+        return acc;
+    };
+    for (int d0 = wave * 4; d0 < dim; d0 += 64) {       // four numbers of z per wave at a time
+        float acc[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+        for (int c = lane * 8; c < W; c += 512) {
+            const uint4 xv = *reinterpret_cast<const uint4 *>(xb + c);
+            uint4 wv[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) wv[i] = *reinterpret_cast<const uint4 *>(Wg + (int64_t)min(d0 + i, dim - 1) * W + c);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) acc[i] = dot8(wv[i], xv, acc[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float z = wave_sum(acc[i]);
+            if (lane == 0 && d0 + i < dim) { bf16_t h; st_f(&h, 0, z); st_f(gs, d0 + i, gelu_tanh_f(ld_f(&h, 0)) * ld_f(er, d0 + i)); }
+        }
+    }
+    __syncthreads();
+    const bf16_t *Wp = (const bf16_t *)a.proj;
+    float s1 = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int c4 = tid + k * 1024;
+        ys[k] = float4{0.f, 0.f, 0.f, 0.f};
+        if (c4 < W4) {
+            float acc[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+            for (int d = 0; d < dim; d += 8) {
+                const uint4 gv = *reinterpret_cast<const uint4 *>(gs + d);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[i] = dot8(*reinterpret_cast<const uint4 *>(Wp + (int64_t)(c4 * 4 + i) * dim + d), gv, acc[i]);
+            }
+            ys[k] = unpack4(pack4(float4{acc[0], acc[1], acc[2], acc[3]}));
+        }
+        s1 += square4(ys[k]);
+    }
+    const float f1 = 1.0f / sqrtf(sum_all(s1) / (float)W + a.eps);
     float s2 = 0.f;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
-        const int c4 = l + k * NT;
+        const int c4 = tid + k * 1024;
         if (c4 < W4) {
-            const float4 w = *reinterpret_cast<const float4 *>(wb + c4 * 4);
-            xs[k].x += ys[k].x * f * w.x; xs[k].y += ys[k].y * f * w.y; xs[k].z += ys[k].z * f * w.z; xs[k].w += ys[k].w * f * w.w;
+            const float4 w = *reinterpret_cast<const float4 *>(a.ws + c4 * 4);
+            xs[k].x += ys[k].x * f1 * w.x; xs[k].y += ys[k].y * f1 * w.y; xs[k].z += ys[k].z * f1 * w.z; xs[k].w += ys[k].w * f1 * w.w;
             *reinterpret_cast<float4 *>(xr + c4 * 4) = xs[k];
-            s2 += (xs[k].x * xs[k].x + xs[k].y * xs[k].y) + (xs[k].z * xs[k].z + xs[k].w * xs[k].w);
+            s2 += square4(xs[k]);
         }
     }
-    if (!wn && !plain) return;
-    const float f2 = wn ? 1.0f / sqrtf((NT == 64 ? wave_sum(s2) : block_sum256(s2, red)) / (float)W + eps) : 1.f;
+    if (!a.wn) return;
+    const float f2 = 1.0f / sqrtf(sum_all(s2) / (float)W + a.eps);
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
-        const int c4 = l + k * NT;
+        const int c4 = tid + k * 1024;
         if (c4 < W4) {
-            const float4 w = wn ? *reinterpret_cast<const float4 *>(wn + c4 * 4) : float4{1.f, 1.f, 1.f, 1.f};
-            bf16_t h[4];
-            st_f(h, 0, xs[k].x * f2 * w.x); st_f(h, 1, xs[k].y * f2 * w.y); st_f(h, 2, xs[k].z * f2 * w.z); st_f(h, 3, xs[k].w * f2 * w.w);
-            *reinterpret_cast<uint2 *>(out + t * ldo + c4 * 4) = uint2{(uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16)};
+            const float4 w = *reinterpret_cast<const float4 *>(a.wn + c4 * 4);
+            *reinterpret_cast<uint2 *>((bf16_t *)a.out + t * a.ldo + c4 * 4) = pack4(float4{xs[k].x * f2 * w.x, xs[k].y * f2 * w.y, xs[k].z * f2 * w.z, xs[k].w * f2 * w.w});
         }
     }
 }
@@ -1058,22 +1183,54 @@ static bool aligned16(const void *p) { return ((uintptr_t)p & 15) == 0; }
 static bool norm_join4_ok(int64_t W, const float *x, const void *y, int64_t ldy, const float *wb, const float *wn, const void *out, int64_t ldo) {
     return W % 4 == 0 && W <= 8192 && ldy % 4 == 0 && ldo % 4 == 0 && aligned16(x) && aligned16(y) && aligned16(wb) && aligned16(wn) && aligned16(out);
 }
-static int norm_join4(float *x, const void *y, int64_t ldy, int64_t T, int64_t W, float eps, const float *wb, const float *wn, bool plain, void *out, int64_t ldo, hipStream_t s) {
-    const int64_t W4 = W / 4;
-    const bool wave = T >= 1024 && W4 <= 256;           // many rows: a wave per row up to 1024 numbers; few rows: a workgroup per row
-    const dim3 grid((unsigned)(wave ? (T + 3) / 4 : T)), blk(256);
-#define NVR_NJ(NT_, NV_) norm_join4_kernel<NT_, NV_><<<grid, blk, 0, s>>>(x, (const bf16_t *)y, ldy, T, (int)W, eps, wb, wn, plain ? 1 : 0, (bf16_t *)out, ldo)
+template <int KIND>
+static int norm_join4(const NormJoin &a, const Batch &b, hipStream_t s) {
+    const int64_t W4 = a.W / 4;
+    const bool wave = a.T >= 1024 && W4 <= 256;         // many rows: a wave per row up to 1024 numbers; few rows: a workgroup per row
+    const dim3 grid((unsigned)(wave ? (a.T + 3) / 4 : a.T)), blk(256);
+#define NVR_NJ(NT_, NV_) norm_join4_kernel<NT_, NV_, KIND><<<grid, blk, 0, s>>>(a, b)
     if (wave) { if (W4 <= 64) NVR_NJ(64, 1); else if (W4 <= 128) NVR_NJ(64, 2); else NVR_NJ(64, 4); }
     else if (W4 <= 256) NVR_NJ(256, 1); else if (W4 <= 512) NVR_NJ(256, 2); else if (W4 <= 1024) NVR_NJ(256, 4); else NVR_NJ(256, 8);
 #undef NVR_NJ
     return launched("norm_join4");
 }
 
+int embed_norm(const void *E, const void *P, bool bf16, const Batch &b, int64_t W, float scale, float *x, float eps, const float *wn, void *out, hipStream_t s) {
+    if (b.T == 0) return 0;
+    if (bf16 && norm_join4_ok(W, x, E, W, wn, wn, out, W) && aligned16(P)) {
+        NormJoin j{}; j.x = x; j.ldx = W; j.T = b.T; j.W = (int)W; j.eps = eps; j.wn = wn; j.out = (bf16_t *)out; j.ldo = W; j.E = (const bf16_t *)E; j.P = (const bf16_t *)P; j.scale = scale;
+        return norm_join4<NJ_START>(j, b, s);
+    }
+    if (int rc = embed_pos(E, P, bf16, b, W, scale, x, s)) return rc;
+    GroupNormArgs n{}; n.in = x; n.ldi = W; n.in_f32 = true; n.rows_n = b.T; n.W = W; n.groups = 1; n.eps = eps; n.w = wn; n.out = out; n.ldo = W;
+    return group_norm(n, bf16, s);
+}
+
+bool side_step_ok(const SideStepArgs &a, bool bf16) {
+    return bf16 && a.T <= 64 && a.W % 8 == 0 && a.W <= 8192 && a.dim % 8 == 0 && a.dim <= 4096 && a.ldy % 4 == 0 && a.ldo % 4 == 0 && aligned16(a.x) && aligned16(a.y) && aligned16(a.wb) && aligned16(a.ws) && aligned16(a.wn) &&
+           aligned16(a.out) && aligned16(a.gate) && aligned16(a.proj);
+}
+int side_step(const SideStepArgs &a, hipStream_t s) {
+    if (a.T == 0) return 0;
+    if (!side_step_ok(a, true)) return nvr::fail(NVR_ERR_UNSUPPORTED, "side_step: %d rows of %d numbers, token input of %d", a.T, a.W, a.dim);
+    const size_t lds = (size_t)(a.W + a.dim) * 2;
+    if (a.W <= 4096) side_step_kernel<1><<<dim3((unsigned)a.T), dim3(1024), lds, s>>>(a);
+    else side_step_kernel<2><<<dim3((unsigned)a.T), dim3(1024), lds, s>>>(a);
+    return launched("side_step");
+}
+
 int group_norm(const GroupNormArgs &a, bool bf16, hipStream_t s) {
     if (a.rows_n == 0) return 0;
     if (a.groups < 1 || a.W % a.groups) return nvr::fail(NVR_ERR_INVALID_ARG, "group_norm: %ld columns in %d groups", (long)a.W, a.groups);
     if (bf16 && a.xres && a.groups == 1 && !a.in_f32 && !a.rows && !(a.w2 && a.out_plain) && norm_join4_ok(a.W, a.xres, a.in, a.ldi, a.w, a.w2, a.out, a.ldo))
-        return norm_join4(a.xres, a.in, a.ldi, a.rows_n, a.W, a.eps, a.w, a.w2, a.out_plain, a.out, a.ldo, s);
+    {
+        NormJoin j{}; j.x = a.xres; j.ldx = a.W; j.y = (const bf16_t *)a.in; j.ldy = a.ldi; j.T = a.rows_n; j.W = (int)a.W; j.eps = a.eps; j.wb = a.w; j.wn = a.w2; j.plain = a.out_plain ? 1 : 0; j.out = (bf16_t *)a.out; j.ldo = a.ldo;
+        return norm_join4<NJ_JOIN>(j, Batch{}, s);
+    }
+    if (bf16 && !a.xres && a.groups == 1 && a.in_f32 && norm_join4_ok(a.W, (const float *)a.in, nullptr, a.ldi, nullptr, a.w, a.out, a.ldo)) {
+        NormJoin j{}; j.x = (float *)a.in; j.ldx = a.ldi; j.rows = a.rows; j.T = a.rows_n; j.W = (int)a.W; j.eps = a.eps; j.wn = a.w; j.out = (bf16_t *)a.out; j.ldo = a.ldo;
+        return norm_join4<NJ_NORM>(j, Batch{}, s);
+    }
     if (a.out_plain && (a.w2 || !a.xres)) return nvr::fail(NVR_ERR_INVALID_ARG, "group_norm: a plain copy leaves only with the residual sum, instead of the next norm");
     const dim3 grid((unsigned)a.rows_n), blk(256);
     const int W = (int)a.W;
@@ -1256,7 +1413,10 @@ int side_gate(const void *z, const int64_t *ids, const void *E, int64_t lde, int
 int layer_tail(const LayerTailArgs &a, bool bf16, hipStream_t s) {
     if (a.T == 0) return 0;
     if (bf16 && a.side_y && !a.kept && (!a.wnext || a.groups == 1) && norm_join4_ok(a.W, a.x, a.side_y, a.W, a.side_norm, a.wnext, a.out, a.W))
-        return norm_join4(a.x, a.side_y, a.W, a.T, a.W, a.eps, a.side_norm, a.wnext, false, a.out, a.W, s);
+    {
+        NormJoin j{}; j.x = a.x; j.ldx = a.W; j.y = (const bf16_t *)a.side_y; j.ldy = a.W; j.T = a.T; j.W = a.W; j.eps = a.eps; j.wb = a.side_norm; j.wn = a.wnext; j.out = (bf16_t *)a.out; j.ldo = a.W;
+        return norm_join4<NJ_JOIN>(j, Batch{}, s);
+    }
     const size_t lds = (size_t)2 * a.W * 4;
     if (lds > kMaxLds) return nvr::fail(NVR_ERR_UNSUPPORTED, "layer_tail: rows of %d numbers do not fit LDS", a.W);
     if (a.wnext && (a.groups < 1 || a.W % a.groups)) return nvr::fail(NVR_ERR_INVALID_ARG, "layer_tail: %d columns in %d groups", a.W, a.groups);

@@ -557,6 +557,8 @@ int LayeredModel::init_sequential(nvr_model_runner &r) {
             // mix rows: queries [H][2][D], keys [G][2][D], values [G][Dv], one gate number per head; a key row of the pages holds both maps' keys
             const int64_t kn = L.kv_heads * 2 * L.dim, vn = L.kv_heads * L.vdim;
             w.qcol = 0; w.kcol = pad16(2 * hd); w.vcol = w.kcol + pad16(kn); w.gcol = w.vcol + pad16(vn); w.nmix = w.gcol + pad16(L.heads);
+            const int64_t whole = (w.nmix + 255) / 256 * 256;
+            if (bf16 && (whole - w.nmix) * 16 <= w.nmix) w.nmix = whole;                 // (the 256 x 256 product takes whole tiles; the rows behind the gates stay zero)
             RC(own(&w.qn, (size_t)L.dim * 4)); RC(own(&w.kn, (size_t)L.dim * 4)); RC(own(&w.lambda, 4));
             for (auto &v : w.lam) v.assign((size_t)L.dim, 0.f);
             RC(diff_share(w, L));
@@ -801,9 +803,11 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
     const float eps = (float)spec.eps; const int groups = (int)spec.norm_groups;
     hipStream_t s = r.stream;
     auto at = [&](void *base, int64_t col) { return (void *)((char *)base + (size_t)(col * esz)); };
-    if (pos) RC(kl::embed_pos(embed, pos, bf16, b, W, (float)spec.embedding_scale, x, s));
-    else RC(kl::embed_keep(embed, bf16, b.ids, T, W, x, kept, s));
-    {   // the first layer's input; every later one leaves the end of the layer before it
+    if (!spec.depth_average && groups == 1) RC(kl::embed_norm(embed, pos, bf16, b, W, (float)spec.embedding_scale, x, eps, lw[0].n1, a1, s));
+    else {
+        if (pos) RC(kl::embed_pos(embed, pos, bf16, b, W, (float)spec.embedding_scale, x, s));
+        else RC(kl::embed_keep(embed, bf16, b.ids, T, W, x, kept, s));
+        // the first layer's input; every later one leaves the end of the layer before it
         kl::GroupNormArgs n{}; n.in = x; n.ldi = W; n.in_f32 = true; n.rows_n = T; n.W = W; n.groups = groups; n.eps = eps; n.w = lw[0].n1; n.out = a1; n.ldo = W;
         RC(kl::group_norm(n, bf16, s));
     }
@@ -907,7 +911,11 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             RC(kl::head_norm_gate(ret_o, proj, w.nmix, w.gcol, T, L.heads, L.vdim, eps, w.hnorm, cat, hv, bf16, s));
         }
         RC(gemm(r, cat, hv, w.wo, T, hv, W, tmp));
-        {   // the mixer's output joins the stream; the feed-forward's input leaves in the same pass
+        // few rows: the last join of the layer, the token input and the next layer's first norm are one launch
+        kl::SideStepArgs sd{}; sd.x = x; sd.T = (int32_t)T; sd.W = (int32_t)W; sd.dim = (int32_t)spec.side_dim; sd.eps = eps; sd.y = tmp; sd.ldy = W; sd.wb = L.has_mlp ? w.n2b : w.n1b; sd.gate = w.sgate; sd.proj = w.sproj;
+        sd.ids = b.ids; sd.E = side_embed; sd.lde = nL * spec.side_dim; sd.ecol = i * spec.side_dim; sd.ws = w.snorm; sd.wn = i + 1 < nL ? lw[(size_t)(i + 1)].n1 : nullptr; sd.out = a1; sd.ldo = W;
+        const bool one_step = spec.side_dim && !spec.depth_average && groups == 1 && kl::side_step_ok(sd, bf16);
+        if (L.has_mlp || !one_step) {   // the mixer's output joins the stream; the feed-forward's input leaves in the same pass
             kl::GroupNormArgs n{}; n.in = tmp; n.ldi = W; n.rows_n = T; n.W = W; n.groups = groups; n.eps = eps; n.w = w.n1b; n.xres = x;
             if (L.has_mlp) { n.w2 = w.n2; n.out = a2; n.ldo = W; }
             else if (spec.side_dim && bf16) { n.out_plain = true; n.out = a2; n.ldo = W; }       // (the token input's projection reads the stream in the operand type)
@@ -953,6 +961,7 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             }
             RC(kl::moe_combine(e_y, place_of, T, L.top, fs ? shared_y : nullptr, W, tmp, bf16, s));
         }
+        if (one_step) { RC(kl::side_step(sd, s)); continue; }
         if (L.has_mlp) {
             kl::GroupNormArgs n{}; n.in = tmp; n.ldi = W; n.rows_n = T; n.W = W; n.groups = groups; n.eps = eps; n.w = w.n2b; n.xres = x;
             if (spec.side_dim && bf16) { n.out_plain = true; n.out = a2; n.ldo = W; }
