@@ -63,7 +63,9 @@ int add_rmsnorm_slabs(half_bits *h, const float *slabs, int64_t S, const half_bi
 // qkv -> RoPE(q,k) + KV store, W [(H+2KVH)D, K] -> qkv [T,(H+2KVH)D] (roped q,k; v) and cache rows at slots
 int linear_silu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I,
                     half_bits *out, hipStream_t s, const half_bits *Wt = nullptr);
-// the same with gelu (tanh form) in silu's place
+// y = gelu(x . W^T), the form with the error function, where the kernel of this shape has it in its epilogue (*applied), else y = x . W^T
+int linear_gelu(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, bool *applied, hipStream_t s);
+// gate / up products with gelu (tanh form) in silu's place
 int linear_gelu_mul(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t I, half_bits *out, hipStream_t s);
 int linear_qkv_rope_store(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t H,
                           int64_t KVH, int64_t D, const int64_t *positions, const int32_t *slots, const float *cos_t,

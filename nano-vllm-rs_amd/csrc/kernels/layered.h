@@ -168,7 +168,7 @@ int poly_norm(const void *z, int64_t ldz, int64_t T, int64_t F, float eps, const
 // out = silu(gate) * up, or gelu(gate) * up (the tanh form); gu: rows [2 F] (gate columns, then up columns)
 int gelu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 int silu_mul(const void *gu, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
-// out = gelu(z), the form with the error function (rows of F numbers, strides ldz / ldo)
+// out = gelu(z), the form with the error function (rows of F numbers, strides ldz / ldo; in place too)
 int gelu_erf(const void *z, int64_t ldz, int64_t T, int64_t F, void *out, int64_t ldo, bool bf16, hipStream_t s);
 
 // Router of a mixture of experts: logits wr h in f32 (wr: [E][W] f32), the top largest per token -> sel / score (= sigmoid of the logit) [T][top]; then the rows

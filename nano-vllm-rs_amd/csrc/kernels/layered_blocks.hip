@@ -882,7 +882,7 @@ __global__ __launch_bounds__(256) void moe_combine8_kernel(const bf16_t *__restr
 
 // out = z Phi(z) (rows of F numbers)
 template <class CT>
-__global__ __launch_bounds__(256) void gelu_erf_kernel(const CT *__restrict__ z, int64_t ldz, int64_t T, int64_t F, CT *__restrict__ out, int64_t ldo) {
+__global__ __launch_bounds__(256) void gelu_erf_kernel(const CT *z, int64_t ldz, int64_t T, int64_t F, CT *out, int64_t ldo) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= T * F) return;
     const int64_t t = i / F, c = i - t * F;
@@ -890,7 +890,7 @@ __global__ __launch_bounds__(256) void gelu_erf_kernel(const CT *__restrict__ z,
 }
 
 // the same for 16-bit rows, 8 numbers per thread (F and both strides multiples of 8, 16-byte aligned rows)
-__global__ __launch_bounds__(256) void gelu_erf8_kernel(const bf16_t *__restrict__ z, int64_t ldz, int64_t T, int64_t F8, bf16_t *__restrict__ out, int64_t ldo) {
+__global__ __launch_bounds__(256) void gelu_erf8_kernel(const bf16_t *z, int64_t ldz, int64_t T, int64_t F8, bf16_t *out, int64_t ldo) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= T * F8) return;
     const int64_t t = i / F8, c = (i - t * F8) * 8;

@@ -36,24 +36,23 @@ __device__ __forceinline__ float wave_max(float v) {
     return v;
 }
 __device__ __forceinline__ bf16x4 read_tr(const char *p) { return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((__attribute__((address_space(3))) bf16x4 *)p); }
-__host__ __device__ constexpr int image_stride(int Dv) { return (Dv * 2 + 63) / 64 * 64 + 32; }      // bytes; an odd multiple of 32: the 8 rows 32 lanes read together sit on different banks
+// One build per size class C >= D, Dv, with no bound inside: a piece of a row past its end is read again from its last 16 bytes (the query's numbers there are zero, the output's are not stored).
+constexpr int image_stride(int C) { return C * 2 + 32; }             // bytes; an odd multiple of 32: the 8 rows 32 lanes read together sit on different banks
 
-// C: size class of D and Dv.  SHARED: the values are the first Dv numbers of the key rows.
+// SHARED: the values are the first Dv numbers of the key rows.  bs_shift: log2 of the page size, or -1.  g: query rows per key/value head, in nrb groups of up to 16.  Grid: shares, groups, sequences.
 template <int C, bool DIFF, bool SHARED>
-__global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Batch b, int nsplit, int nrb, float *__restrict__ part_o, float *__restrict__ part_ml,
-                                                             unsigned int *__restrict__ tickets) {
-    constexpr int NKS = C / 32, NDT = C / 16;
-    extern __shared__ __attribute__((aligned(16))) char smem[];      // the waves' value images; behind the last chunk their outputs [4][16][Dv + 4] f32
+__global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Batch b, int bs_shift, int g, int nsplit, int nrb, float *__restrict__ part_o,
+                                                             float *__restrict__ part_ml, unsigned int *__restrict__ tickets) {
+    constexpr int NKS = C / 32, NDT = C / 16, VS = image_stride(C), OS = C + 4;
+    extern __shared__ __attribute__((aligned(16))) char smem[];      // the waves' value images; behind the last chunk their outputs [4][16][OS] f32
     __shared__ float mls[4][16][2];
     __shared__ unsigned int ticket_s;
-    const int GG = a.G * nrb;                           // groups of rows per sequence
-    const int z = blockIdx.x % nsplit, pair = blockIdx.x / nsplit, grp = pair % GG, sq = pair / GG;
-    const int g = a.H * (DIFF ? 2 : 1) / a.G, kvh = grp / nrb, r0 = (grp % nrb) * 16, nr = min(16, g - r0);
+    const int z = blockIdx.x, grp = blockIdx.y, sq = blockIdx.z, pair = sq * gridDim.y + grp;
+    const int kvh = nrb == 1 ? grp : grp / nrb, r0 = (grp - kvh * nrb) * 16, nr = min(16, g - r0);
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, lm = lane & 15, lq = lane >> 4;
-    const int pos = b.start[sq], ctx = pos + 1, D = a.D, Dv = a.Dv, d32 = D >> 5, v32 = (Dv + 31) >> 5, dv16 = Dv >> 4, bs = b.block_size;
+    const int pos = b.start[sq], ctx = pos + 1, D = a.D, Dv = a.Dv, bs = b.block_size;
     const int32_t *bt = b.block_tables + (int64_t)sq * b.max_blocks;
     const bf16_t *kc = (const bf16_t *)a.kc, *vc = (const bf16_t *)a.vc;
-    const int VS = image_stride(Dv);
     char *img = smem + wave * CH * VS;
     const float scale2 = a.scale * kLog2e;
 
@@ -80,35 +79,37 @@ __global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Bat
     const int nch = kept + (ctx - j0 + CH - 1) / CH;
     for (int x = z * 4 + wave; x < nch; x += nsplit * 4) {
         const int base = x < kept ? x * CH : j0 + (x - kept) * CH;
-        uint4 kf[2][NKS], vf[2][NKS];
+        bf16x8 kf[2][NKS], vf[2][NKS];
+        int64_t row[2];
 #pragma unroll
         for (int mt = 0; mt < 2; ++mt) {
-            const int j = min(base + mt * 16 + lm, ctx - 1), blk = bt[j / bs];
-            const int64_t row = ((int64_t)blk * bs + j % bs) * a.G + kvh;
-            const bf16_t *kp = kc + row * D + lq * 8, *vp = vc + row * Dv;
+            const int j = min(base + mt * 16 + lm, ctx - 1), pg = bs_shift >= 0 ? j >> bs_shift : j / bs;
+            row[mt] = ((int64_t)bt[pg] * bs + (j - pg * bs)) * a.G + kvh;
+        }
 #pragma unroll
-            for (int ks = 0; ks < NKS; ++ks) {
-                if (ks < d32) kf[mt][ks] = *reinterpret_cast<const uint4 *>(kp + ks * 32);
-                if constexpr (!SHARED) { if (ks < v32) vf[mt][ks] = *reinterpret_cast<const uint4 *>(vp + min(ks * 32 + lq * 8, Dv - 8)); }
-            }
+        for (int mt = 0; mt < 2; ++mt) {
+            const bf16_t *kp = kc + row[mt] * D, *vp = vc + row[mt] * Dv;
+#pragma unroll
+            for (int ks = 0; ks < NKS; ++ks) kf[mt][ks] = *reinterpret_cast<const bf16x8 *>(kp + min(ks * 32 + lq * 8, D - 8));
+            if constexpr (!SHARED)
+#pragma unroll
+                for (int ks = 0; ks < NKS; ++ks) vf[mt][ks] = *reinterpret_cast<const bf16x8 *>(vp + min(ks * 32 + lq * 8, Dv - 8));
         }
         f32x4 s[2];
 #pragma unroll
         for (int mt = 0; mt < 2; ++mt) {
             s[mt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int ks = 0; ks < NKS; ++ks)
-                if (ks < d32) s[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[mt][ks]), qf[ks], s[mt], 0, 0, 0);
+            for (int ks = 0; ks < NKS; ++ks) s[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[mt][ks], qf[ks], s[mt], 0, 0, 0);
         }
 #pragma unroll
         for (int mt = 0; mt < 2; ++mt)
 #pragma unroll
-            for (int ks = 0; ks < NKS; ++ks)
-                if (ks < v32) {
-                    uint4 v;
-                    if constexpr (SHARED) v = kf[mt][ks]; else v = vf[mt][ks];
-                    if (ks * 32 + lq * 8 < Dv) *reinterpret_cast<uint4 *>(img + (mt * 16 + lm) * VS + (ks * 32 + lq * 8) * 2) = v;
-                }
+            for (int ks = 0; ks < NKS; ++ks) {
+                bf16x8 v;
+                if constexpr (SHARED) v = kf[mt][ks]; else v = vf[mt][ks];
+                *reinterpret_cast<bf16x8 *>(img + (mt * 16 + lm) * VS + (ks * 32 + lq * 8) * 2) = v;
+            }
         // scores of query lm: keys base + mt * 16 + lq * 4 + e
         float mx = -INFINITY;
 #pragma unroll
@@ -137,22 +138,20 @@ __global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Bat
         }
         asm volatile("" ::: "memory");                  // (a wave's LDS requests are served in order: its image is written before it is read, and read before it is written again)
 #pragma unroll
-        for (int t = 0; t < NDT; ++t)
-            if (t < dv16) {
-                const char *p = img + (lq * 4 + (lm >> 2)) * VS + t * 32 + (lm & 3) * 8;
-                const bf16x4 a0 = read_tr(p), a1 = read_tr(p + 16 * VS);
-                bf16x8 v;
+        for (int t = 0; t < NDT; ++t) {
+            const char *p = img + (lq * 4 + (lm >> 2)) * VS + t * 32 + (lm & 3) * 8;
+            const bf16x4 a0 = read_tr(p), a1 = read_tr(p + 16 * VS);
+            bf16x8 v;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) { v[e] = a0[e]; v[4 + e] = a1[e]; }
-                o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, o[t], 0, 0, 0);
-            }
+            for (int e = 0; e < 4; ++e) { v[e] = a0[e]; v[4 + e] = a1[e]; }
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, o[t], 0, 0, 0);
+        }
         asm volatile("" ::: "memory");
     }
     l += __shfl_xor(l, 16, 64); l += __shfl_xor(l, 32, 64);
     if (lq == 0) { mls[wave][lm][0] = m; mls[wave][lm][1] = l; }
     __syncthreads();
     // the waves' outputs in one unit per row, then their sums
-    const int OS = Dv + 4;
     float *om = (float *)smem;
     {
         const float mx = fmaxf(fmaxf(mls[0][lm][0], mls[1][lm][0]), fmaxf(mls[2][lm][0], mls[3][lm][0]));
@@ -160,7 +159,7 @@ __global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Bat
         if (lm < nr)
 #pragma unroll
             for (int t = 0; t < NDT; ++t)
-                if (t < dv16) *reinterpret_cast<f32x4 *>(om + (wave * 16 + lm) * OS + t * 16 + lq * 4) = o[t] * f;
+                *reinterpret_cast<f32x4 *>(om + (wave * 16 + lm) * OS + t * 16 + lq * 4) = o[t] * f;
     }
     __syncthreads();
     const int c4 = lane * 4;
@@ -234,16 +233,17 @@ __global__ __launch_bounds__(256, 1) void attn_decode_kernel(SinkAttnArgs a, Bat
 }
 
 const size_t kMaxLds = 160 * 1024 - 4096;
-size_t decode_lds(int Dv) { return std::max((size_t)4 * CH * image_stride(Dv), (size_t)4 * 16 * (Dv + 4) * 4); }
 
 template <int C>
 int launch(const SinkAttnArgs &a, const Batch &b, int nsplit, int nrb, float *po, float *pml, unsigned int *tickets, hipStream_t s) {
-    const dim3 grid((unsigned)((int64_t)b.B * a.G * nrb * nsplit)), blk(256);
-    const size_t lds = decode_lds(a.Dv);
+    const dim3 grid((unsigned)nsplit, (unsigned)(a.G * nrb), (unsigned)b.B), blk(256);
+    const int g = a.H * (a.lambda ? 2 : 1) / a.G;
+    const size_t lds = std::max((size_t)4 * CH * image_stride(C), (size_t)4 * 16 * (C + 4) * 4);
     const bool shared = a.vld != 0;
-    if (a.lambda) attn_decode_kernel<C, true, false><<<grid, blk, lds, s>>>(a, b, nsplit, nrb, po, pml, tickets);
-    else if (shared) attn_decode_kernel<C, false, true><<<grid, blk, lds, s>>>(a, b, nsplit, nrb, po, pml, tickets);
-    else attn_decode_kernel<C, false, false><<<grid, blk, lds, s>>>(a, b, nsplit, nrb, po, pml, tickets);
+    const int bs_shift = (b.block_size & (b.block_size - 1)) == 0 ? __builtin_ctz((unsigned)b.block_size) : -1;
+    if (a.lambda) attn_decode_kernel<C, true, false><<<grid, blk, lds, s>>>(a, b, bs_shift, g, nsplit, nrb, po, pml, tickets);
+    else if (shared) attn_decode_kernel<C, false, true><<<grid, blk, lds, s>>>(a, b, bs_shift, g, nsplit, nrb, po, pml, tickets);
+    else attn_decode_kernel<C, false, false><<<grid, blk, lds, s>>>(a, b, bs_shift, g, nsplit, nrb, po, pml, tickets);
     hipError_t e = hipGetLastError();
     if (e != hipSuccess) return nvr::fail(NVR_ERR_HIP, "attention_decode launch failed: %s", hipGetErrorString(e));
     return 0;
@@ -276,10 +276,11 @@ int attention_decode(const SinkAttnArgs &a, const Batch &b, int max_splits, void
     if (!attention_decode_ok(a, true)) return nvr::fail(NVR_ERR_UNSUPPORTED, "attention_decode: shape outside the kernel");
     const int nrb = row_blocks(a);
     const int64_t pairs = (int64_t)b.B * a.G * nrb;
+    if (b.B > 65535 || a.G * nrb > 65535) return nvr::fail(NVR_ERR_INVALID_ARG, "attention_decode: %d sequences of %d groups", b.B, a.G * nrb);
     const int keys = a.window > 0 ? std::min<int64_t>(b.max_ctx, (int64_t)a.window + std::max(a.keep_first, 0) + 2 * CH) : b.max_ctx;
-    // shares of the keys: at most a chunk per wave, at most what the workspace and a wave's lanes hold
+    // shares of the keys: two chunks per wave (one, or three and more, measured slower), at most what the workspace and a wave's lanes hold
     const size_t per = 16 * (size_t)(a.Dv + 2) * 4;
-    int64_t nsplit = std::min<int64_t>({(int64_t)max_splits, ((int64_t)keys + 4 * CH - 1) / (4 * CH), 64, (int64_t)(workspace_bytes / per / (size_t)pairs)});
+    int64_t nsplit = std::min<int64_t>({(int64_t)max_splits, ((int64_t)keys + 8 * CH - 1) / (8 * CH), 64, (int64_t)(workspace_bytes / per / (size_t)pairs)});
     if (nsplit < 1) nsplit = 1;
     if (nsplit > 1 && pairs > num_tickets) return nvr::fail(NVR_ERR_INVALID_ARG, "attention_decode: %ld groups of rows, %d counters", (long)pairs, num_tickets);
     float *po = (float *)workspace, *pml = po + pairs * nsplit * 16 * a.Dv;

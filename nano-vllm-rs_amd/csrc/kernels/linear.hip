@@ -41,7 +41,7 @@ struct LinEpi {
     int32_t kslice; int64_t slab_stride;
     // W is the TILED copy [N/16][K/32][16][32] (retile_weight): one wave-instruction reads 1 KiB contiguous
     int32_t tiled;
-    int32_t gelu;                          // EPI_SILU: gelu (tanh form) instead of silu
+    int32_t gelu;                          // EPI_SILU: gelu (tanh form) instead of silu; EPI_F16: gelu (error function) of the product
 };
 
 // W row handled by local row r (0..15) of n-tile i of workgroup bx
@@ -150,7 +150,10 @@ __global__ __launch_bounds__(WAVES * 64) void linear_skinny_kernel(const half_t 
     // C layout of the 16x16 MFMA: row (n) = q*4 + reg, col (token) = r
     if (EPI == EPI_F16 || EPI == EPI_F32 || EPI == EPI_SLAB) {
         for (int tile = wave; tile < NT * MT; tile += WAVES) {
-            const float4_t s = reduce(tile);
+            float4_t s = reduce(tile);
+            if (EPI == EPI_F16 && epi.gelu)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) s[e] = gelu_erf_fast(s[e]);
             const int i = tile / MT, j = tile % MT;
             const int n = (blockIdx.x * NT + i) * 16 + q * 4, m = m0 + j * 16 + r;
             if (m < T && n < N) {
@@ -270,21 +273,24 @@ static int launch_check(const char *what) {
     return 0;
 }
 
-int linear(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, void *y,
-           bool y_f32, hipStream_t s, const half_bits *Wt) {
+// gelu (not null): in, whether y = gelu(x . W^T) is wanted; out, whether the kernel this shape takes has applied it
+static int linear_routed(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, void *y, bool y_f32, hipStream_t s, const half_bits *Wt, bool *gelu) {
+    const bool act = gelu && *gelu;
     if (K % 32 || N % 16 || ldx % 8)
         return nvr::fail(NVR_ERR_UNSUPPORTED, "linear: K=%ld must be a multiple of 32, N=%ld of 16, ldx=%ld of 8",
                          (long)K, (long)N, (long)ldx);
     if (T == 0) return 0;
     // Routing by measured crossovers (scratch/gemm_route_sweep.py, profiles/r01_gemm_ablation.txt): prefer_256 above; the 128x128 kernel's
     // own single-tile latency (21-31 us) loses to the weight-streaming kernel run over 32-token blocks while T or T*N is small
-    if (!y_f32 && gemm256_ok(T, K, N, ldx) && prefer_256(T, K, N)) return gemm256(x, ldx, W, T, K, N, (half_bits *)y, s);   // prefill regime
+    if (!y_f32 && gemm256_ok(T, K, N, ldx) && prefer_256(T, K, N)) return act ? gemm256_gelu(x, ldx, W, T, K, N, (half_bits *)y, s) : gemm256(x, ldx, W, T, K, N, (half_bits *)y, s);   // prefill regime
+    if (gelu) *gelu = false;                               // (the tiled and the streaming kernel have no such epilogue)
     if (!y_f32 && gemm_tiled_ok(T, K, N, ldx) && !prefer_stream(T, N)) return gemm_tiled(x, ldx, W, T, K, N, (half_bits *)y, s);
     if (!y_f32 && linear_stream_ok(T, K, N, ldx)) return linear_stream(x, ldx, W, T, K, N, (half_bits *)y, s, Wt);   // large weights
     const half_t *xx = (const half_t *)x, *ww = (const half_t *)(Wt ? Wt : W);
     const int t = (int)T, k = (int)K, n = (int)N;
     LinEpi e{};
     e.tiled = Wt != nullptr;
+    if (act && !y_f32) { e.gelu = 1; *gelu = true; }
     const int64_t mtiles = (T + 31) / 32;
     // wide GEMMs (LM head, prefill slabs): 64 columns per workgroup amortise the x fragments; narrow ones keep
     // 16 columns per workgroup (more workgroups) and split k over more waves (more bytes in flight per CU)
@@ -313,6 +319,16 @@ int linear(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64
     }
 #undef NVR_LIN
     return launch_check("linear");
+}
+
+int linear(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, void *y,
+           bool y_f32, hipStream_t s, const half_bits *Wt) {
+    return linear_routed(x, ldx, W, T, K, N, y, y_f32, s, Wt, nullptr);
+}
+
+int linear_gelu(const half_bits *x, int64_t ldx, const half_bits *W, int64_t T, int64_t K, int64_t N, half_bits *y, bool *applied, hipStream_t s) {
+    *applied = true;
+    return linear_routed(x, ldx, W, T, K, N, y, false, s, nullptr, applied);
 }
 
 // split-k over S workgroups per tile: slabs[z][T][N] f32 partial sums (summed by add_rmsnorm_slabs); the narrow

@@ -926,11 +926,10 @@ int LayeredModel::forward_sequential(nvr_model_runner &r, const StepPlan &p) {
             RC(kl::poly_norm(gu, L.ff, T, L.ff, eps, w.act, act, L.ff, bf16, s));
             RC(gemm(r, act, L.ff, w.down, T, L.ff, W, tmp));
         } else if (L.ff_kind == LayeredSpec::FF_GELU) {
-            if (bf16 && nvr::kb::gemm256_preferred(T, W, L.ff, W)) RC(nvr::kb::gemm256_gelu((const uint16_t *)a2, W, (const uint16_t *)w.up, T, W, L.ff, (uint16_t *)act, s));   // (GELU in the product's epilogue)
-            else {
-                RC(gemm(r, a2, W, w.up, T, W, L.ff, gu));
-                RC(kl::gelu_erf(gu, L.ff, T, L.ff, act, L.ff, bf16, s));
-            }
+            bool applied = false;                           // (GELU in the product's epilogue where the shape's kernel has it)
+            if (bf16 && W % 32 == 0 && L.ff % 16 == 0) RC(nvr::kb::linear_gelu((const uint16_t *)a2, W, (const uint16_t *)w.up, T, W, L.ff, (uint16_t *)act, &applied, s));
+            else RC(gemm(r, a2, W, w.up, T, W, L.ff, act));
+            if (!applied) RC(kl::gelu_erf(act, L.ff, T, L.ff, act, L.ff, bf16, s));         // (in place)
             RC(gemm(r, act, L.ff, w.down, T, L.ff, W, tmp));
         } else if (L.ff_kind == LayeredSpec::FF_MOE) {
             const int64_t f = L.expert_ff, fs = L.shared_ff, n = T * L.top;

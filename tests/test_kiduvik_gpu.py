@@ -315,6 +315,23 @@ def test_long_prompts_and_decoding_side_by_side(width, dtype):
     check(np.concatenate(gb), wb, dtype, "second request")
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("count", [17, 70])
+def test_many_sequences_decode_side_by_side(count, dtype):
+    """More sequences in a decode-sized step than a tile of the products has rows, and more than the one-launch token input takes; contexts from 1 to 300 tokens."""
+    cfg = make_config([diff(heads=4, kv_heads=2, dim=32, vdim=64, rot=32, mask=(40, 9)), latent(heads=20, dim=48, vdim=64, kv_rank=48, rot_dim=16, mlp=None)], vocab=97, width=96, side=16)
+    w = make_weights(cfg, seed=61)
+    reqs = {"s%d" % k: tokens_of(4 + (k * 37) % 300 if k % 3 == 0 else 4 + k % 7, 97, 700 + k) for k in range(count)}
+    d = Driver(cfg, w, dtype, page=16, pages=count * 20, slots=count, max_tokens=8192, max_len=320)
+    got = {n: [] for n in reqs}
+    for cut in (slice(0, -3), slice(-3, -2), slice(-2, -1), slice(-1, None)):
+        out = d.step([(n, t[cut]) for n, t in reqs.items()])
+        for n in reqs:
+            got[n].append(out[n])
+    for n, t in reqs.items():
+        check(np.concatenate(got[n]), expected_logits(cfg, w, t), dtype, f"request {n}")
+
+
 def test_decode_steps_replay_a_graph():
     """Decode-sized steps are captured the second time their shape is seen and replayed from then on; every replay is compared."""
     for model, dtype in ((everything, "float32"), (with_flash, "bfloat16")):
