@@ -278,8 +278,8 @@ def kiduvik_config(s, window=512, keep=64):
     layers, src = [], None
     for i in range(s["layers"]):
         if i % 4 in (0, 3):
-            m = {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "scale": (D // 2) ** -0.5, "diff": 0.5, "mask": {"size": window, "keep_first": keep},
-                 "rot": {"dims": D // 2, "base": 1000000.0, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            m = {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "scale": (D // 2) ** -0.5, "diff": 0.4, "mask": {"size": window, "keep_first": keep},
+                 "rot": {"dims": D // 2, "base": 300000.0, "scaling": {"factor": 4.0, "original": 8192, "fast": 24.0, "slow": 2.0}}}
             layers.append({"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}})
         else:
             m = {"heads": H, "dim": D - 64, "rot_dim": 64, "vdim": D, "kv_rank": 192, "rot": {"dims": 64, "base": 10000.0}, "scale": D ** -0.5}
